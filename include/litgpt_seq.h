@@ -32,16 +32,17 @@ typedef struct ihipStream_t* lgs_stream_t; /* == hipStream_t */
 const char* lgs_last_error_string(void);
 int lgs_version(void);
 
-/* y[z] (+)= act(a[z] w[z]^T) for z < batch: a[z] = a + z stride_a (M rows of K, row stride lda), w[z] = w + z stride_w
+/* y[z] (+)= act(a[z] w[z]^T + bias) for z < batch: a[z] = a + z stride_a (M rows of K, row stride lda), w[z] = w + z stride_w
  * ([N][K]), y[z] = y + z stride_y (row stride ldy). M <= 8: streaming GEMV; otherwise 128x128 MFMA tiles (bf16) or
  * 64x64 FMA tiles (fp32). z_start (batch + 1 bounds, device) makes it grouped: batch z owns rows
  * [z_start[z], z_start[z+1]) of a list of at most M rows; list row i reads A row a_rows[i] (or i) and writes Y row i
  * (stride_a and stride_y are then ignored for the rows' place). a_bf16: A is a producer's bf16 copy (MFMA tiles with
  * bf16 weights only): the same values the fp32 stream would be rounded to, at half the operand traffic. y_bf16: the
- * result is written as bf16 (it feeds another bf16 product; MFMA tiles, no accumulate). */
+ * result is written as bf16 (it feeds another bf16 product; MFMA tiles, no accumulate). bias: N fp32 values (NULL:
+ * none), the same for every batch. */
 int lgs_linear(const void* a, long lda, long stride_a, const void* w, int w_f32, long stride_w, void* y, long ldy,
                long stride_y, int M, int N, int K, int batch, int accumulate, int act, const int* a_rows,
-               const int* z_start, int a_bf16, int y_bf16, lgs_stream_t stream);
+               const int* z_start, int a_bf16, int y_bf16, const float* bias, lgs_stream_t stream);
 /* x[t] = table[tokens[t]] * scale */
 int lgs_embed(const int* tokens, const void* table, int w_f32, float scale, float* x, int T, int W, int vocab,
               lgs_stream_t stream);
@@ -79,26 +80,26 @@ int lgs_retention(float* q, float* k, float* v, long ld, float* state, const flo
 int lgs_head_gate(float* o, const float* g, long ldg, int T, int H, int dv, int unit_norm, float eps, int act,
                   const float* weight, float post, void* o_bf16 /* optional rounded copy [T][H * dv] */,
                   const void* w_g2, int rank, int g2_f32, lgs_stream_t stream);
-/* latent attention, per token: c = rmsnorm(proj[kv_off .. + r]) * norm_w -> cache_c[slot][pos] (bf16, or fp32 with
- * cache_f32); rotary (pairs 2i, 2i + 1) of proj[kv_off + r .. + dr] -> cache_kr[slot][pos] (fp32); the rotated
- * part of every head's query (at q_off + h (d + dr) + d) is rotated in place. */
-int lgs_latent_prepare(float* proj, long ld, int q_off, int kv_off, void* cache_c, int cache_f32, float* cache_kr,
+/* latent attention, per token: c = rmsnorm(kv[t ldkv .. + r]) * norm_w -> cache_c[slot][pos] (bf16, or fp32 with
+ * cache_f32); rotary (pairs 2i, 2i + 1) of kv[t ldkv + r .. + dr] -> cache_kr[slot][pos] (fp32); the rotated
+ * part of every head's query (at q[t ldq + h (d + dr) + d]) is rotated in place. */
+int lgs_latent_prepare(float* q, long ldq, const float* kv, long ldkv, void* cache_c, int cache_f32, float* cache_kr,
                        const float* norm_w, const float* inv_freq, const int* slot, const int* pos, int T, int H,
                        int d, int dr, int r, int rot_dims, int max_seq, float eps, lgs_stream_t stream);
-/* out[t][h] = sum_j p_j c_j over cached rows j <= pos[t] of slot[t], p = softmax over
+/* out[t][h] = sum_j p_j c_j over cached rows j <= pos[t] of slot[t] (window > 0: the last `window` of them), p = softmax over
  * (qc[t][h] . c_j + q_rot[t][h] . kr_j) * scale with exp(sink[h]) added to the denominator (sink NULL: none).
  * r <= 1024, dr <= 128. splits > 1 spreads every (token, head)'s keys over that many workgroups (decode: few rows,
  * long contexts) and merges them in a second launch; part: T * H * splits * (r + 2) floats of workspace. */
 int lgs_latent_attention(const float* qc, const float* proj, long ld, int q_off, const void* cache_c, int cache_f32,
                          const float* cache_kr, const float* sink, const int* slot, const int* pos, float* out, int T,
-                         int H, int d, int dr, int r, int max_seq, float scale, int splits, float* part,
+                         int H, int d, int dr, int r, int max_seq, float scale, int splits, float* part, int window,
                          lgs_stream_t stream);
 /* the prompt form of lgs_latent_attention: tiles of 16 consecutive tokens of one sequence and one head against key
  * tiles of 16 cached rows, both products on fp32 MFMA; max_len = the most tokens any sequence brings. r % 64 == 0. */
 int lgs_latent_attention_tiles(const float* qc, const float* proj, long ld, int q_off, const void* cache_c,
                                int cache_f32, const float* cache_kr, const float* sink, const int* seq_start,
                                const int* seq_slot, const int* seq_pos0, float* out, int B, int max_len, int H, int d,
-                               int dr, int r, int max_seq, float scale, lgs_stream_t stream);
+                               int dr, int r, int max_seq, float scale, int window, lgs_stream_t stream);
 
 /* out[t][i] = act(a[t * ld + i]) * b[t * ld + i], i < n */
 int lgs_glu(const float* a, const float* b, long ld, void* out /* fp32, or bf16 with out_bf16 */, int out_bf16, int T,
@@ -173,25 +174,39 @@ int lgs_diffattn(const float* q, long ld, const void* cache_k, const void* cache
                  float eps, float post, lgs_stream_t stream);
 
 /* ---- softmax attention with one map per head: normed and / or rotated queries and keys, a sink, a head gate ---- */
-/* Per token: every query head at proj[q_off ..] is (norm != 0) divided by its root mean square (eps inside the root)
- * and multiplied by q_w [d] (NULL: no weight), then rotated on the pairs (i, i + rot_dims / 2) by position *
- * inv_freq[i] (rot_dims 0: not), then multiplied by the query temperature
+/* Per token: every query head at proj[q_off ..] is (norm 1) divided by its root mean square (eps inside the root)
+ * and multiplied by q_w [d] (NULL: no weight) or (norm 2) divided by the root mean square of all heads together and
+ * multiplied by q_w [H d], then rotated on the pairs (i, i + rot_dims / 2), or with interleaved (2i, 2i + 1), by
+ * position * inv_freq[i] (rot_dims 0: not), then multiplied by the query temperature
  * 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1) (temp_every 0: 1), in place; every key head at
  * proj[k_off ..] is normed (k_w) and rotated alike on its way to cache_k [slots][max_seq][G][d], the projection
  * itself stays as it is; the values at proj[v_off ..] go to cache_v [slots][max_seq][G][dv] (bf16, or fp32);
- * v_off == k_off with dv == d makes the values the keys as projected. */
+ * v_off == k_off with dv == d makes the values the keys as projected; v_freq [dv / 2] (NULL: not) rotates the values
+ * by their position over all dv dims in the same layout. pool > 0, in steps of one token per sequence only: the
+ * workgroup whose token completes block b of pool positions leaves the mean of the block's cached keys and values in
+ * row b of pool_k [slots][pool_rows][G][d] and pool_v [..][dv] (fp32). */
 int lgs_normattn_prepare(float* proj, long ld, int q_off, int k_off, int v_off, void* cache_k, void* cache_v,
                          int cache_f32, const int* slot, const int* pos, int T, int H, int G, int d, int dv, int max_seq,
                          float eps, float temp_coef, int temp_every, int norm, const float* q_w, const float* k_w,
-                         const float* inv_freq, int rot_dims, lgs_stream_t stream);
+                         const float* inv_freq, int rot_dims, int interleaved, const float* v_freq, float* pool_k,
+                         float* pool_v, int pool, int pool_rows, lgs_stream_t stream);
+/* The same means for every block that a step completes (any number of tokens per sequence; runs after the step's keys
+ * and values are cached). */
+int lgs_pool_blocks(const void* cache_k, const void* cache_v, int cache_f32, float* pool_k, float* pool_v,
+                    const int* seq_start, const int* seq_slot, const int* seq_pos0, int B, int max_len, int G, int d,
+                    int dv, int max_seq, int pool, int pool_rows, lgs_stream_t stream);
 /* out[t][h] = post * sum_j p_j v_j over the cached rows j of the mask (as lgs_diffattn's), p = softmax of
  * cap((q . k_j) * scale) with exp(sink[h]) added to the normaliser (sink NULL: none); grouped key / value heads.
  * One map per head: q rows hold d values per head. max_len, splits and part (T H splits (2 + dv) floats) as in
- * lgs_diffattn. gate (NULL: none): head h's output at row t is multiplied by sigmoid(gate[t * ldg + h]). */
+ * lgs_diffattn. gate (NULL: none): head h's output at row t is multiplied by sigmoid(gate[t * ldg + h]) (gate_cols 1)
+ * or column by column by sigmoid(gate[t * ldg + h dv + c]) (gate_cols dv). window > 0: position i sees the tokens j with
+ * 0 <= i - j < window and, with pool > 0, the pooled blocks b with b pool + pool - 1 <= i - window, in one softmax.
+ * v_freq: the output at position i is turned back by i * v_freq[m] (pair m, layout as above) ahead of the gate. */
 int lgs_sinkattn(const float* q, long ld, const void* cache_k, const void* cache_v, int cache_f32, const float* sink,
                  const int* seq_start, const int* seq_slot, const int* seq_pos0, float* out, void* out_bf16, float* part,
                  int splits, int B, int max_len, int H, int G, int d, int dv, int max_seq, int chunk, float scale,
-                 float cap, float post, const float* gate, long ldg, lgs_stream_t stream);
+                 float cap, float post, const float* gate, long ldg, int gate_cols, int window, const float* pool_k,
+                 const float* pool_v, int pool, int pool_rows, const float* v_freq, int interleaved, lgs_stream_t stream);
 
 /* ---- gated delta rule ---- */
 /* Per token, on rows qkv [T][ld] = q [G][d] | k [G][d] | v [H][dv] (after their convolution): q and k become unit
@@ -248,14 +263,31 @@ int lgs_gated_group_norm(const float* y, const float* z, long ldz, const float* 
 int lgs_glu_clamped(const float* a, const float* b, long ld, void* out, int out_bf16, int T, int n, float alpha,
                     float limit, float shift, lgs_stream_t stream);
 
-/* ---- sandwich norms ---- */
-/* One boundary between two sublayers whose input AND output are normed, rows of n values. With y0 (the sublayer that
+/* ---- selective scan with a diagonal state matrix per channel ---- */
+/* Over a packed batch: dt = softplus(raw), raw the inner columns of dt_raw (row stride ldt; already with their bias) or,
+ * with w_dt ([inner][rank], bf16 or fp32), w_dt times the rank columns of bc plus dt_bias;
+ * S[n][c] <- exp2(dt_c a2[n][c]) S[n][c] + dt_c x_c B_n, y_c = (sum_n S[n][c] C_n + D_c x_c) * silu(z_c).
+ * x [T][inner] (after the convolution), z: columns of the projection (row stride ldz), bc [T][ldbc] = dt inner values
+ * (rank) | B (N) | C (N), a2 [N][inner] = A log2(e), state [slots][N][inner] fp32, taken as zero when a sequence starts
+ * at position 0. out: fp32, or bf16 with out_bf16. ws (B max_chunks N inner floats) and wsum (B max_chunks inner) with
+ * max_chunks = ceil(max_len / 64): the prompt form, chunks of 64 tokens side by side (needs dt_raw); NULL: every
+ * sequence token by token. N <= 256. */
+int lgs_channel_scan(const float* x, const float* z, long ldz, const float* bc, long ldbc, int rank, const float* dt_raw,
+                     long ldt, const void* w_dt, int w_f32, const float* dt_bias, const float* a2, const float* D,
+                     float* state, const int* seq_start, const int* seq_slot, const int* seq_pos0, void* out,
+                     int out_bf16, int B, int inner, int N, float* ws, float* wsum, int max_chunks, lgs_stream_t stream);
+
+/* ---- boundaries between sublayers ---- */
+/* One boundary between two sublayers of one residual, rows of n values. With y0 (the sublayer that
  * ran; y1: an optional second branch): b_i = w_i ? y_i / rms(y_i) * w_i : y_i, s = coef * (b_0 + b_1),
- * x += s / rms(s) * post_w (post_w: the output norm's weight times the layer's per-channel scale). Then with next_w:
- * h = x / rms(x) * next_w, the next sublayer's input, as fp32 (h) and / or rounded to bf16 (h_bf16). */
-int lgs_sandwich_step(float* x, const float* y0, const float* w0, const float* y1, const float* w1, float coef,
-                      const float* post_w, const float* next_w, float* h, void* h_bf16, float eps, int rows, int n,
-                      lgs_stream_t stream);
+ * x = x_in + s / rms(s) * post_w (x_in NULL: x itself; post_w: the output norm's weight times the layer's per-channel
+ * scale, NULL: x = x_in + s). With depth_w (n_prev + 1 weights, device; the end of a layer in a design that averages over
+ * the depth): hist [hist_rows][rows][n] holds the earlier results X_0 .. X_(n_prev - 1); x is kept there as X_(n_prev)
+ * when n_prev < hist_rows, and x = sum_j depth_w[j] X_j goes on. Then with next_w: h = x / rms(x) * next_w, the next
+ * sublayer's input, as fp32 (h) and / or rounded to bf16 (h_bf16). */
+int lgs_sandwich_step(const float* x_in, float* x, const float* y0, const float* w0, const float* y1, const float* w1,
+                      float coef, const float* post_w, const float* next_w, float* h, void* h_bf16, float eps, int rows,
+                      int n, float* hist, const float* depth_w, int n_prev, int hist_rows, lgs_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -5,20 +5,28 @@
 // head's root mean square and scaled. Sink attention (one map per head): a plain softmax attention whose normaliser
 // also holds exp(sink) of the head. In both, query head h reads key/value head h / (H / G); scores are
 // (q . k) * scale, optionally soft-capped (cap * tanh(s / cap)); a query at position i sees keys lo(i) <= j <= i with
-// lo(i) = i - i % chunk for a chunked mask (chunks are aligned to the sequence's position 0) and 0 without one.
+// lo(i) = i - i % chunk for a chunked mask (chunks are aligned to the sequence's position 0), i - window + 1 for a
+// sliding window and 0 without either. Beside a window the one-map form can see pooled blocks: block b stands for the
+// positions b pool .. b pool + pool - 1 by the mean of their cached keys and of their values (fp32, kept next to the
+// cache), and is seen when it lies wholly before the window; tokens and blocks share one softmax.
 //
 //   lgs_diffattn_prepare  per token: rotary (interleaved pairs 2i, 2i + 1 of the first rot_dims dims of every map)
 //                         on the queries in place and on the keys on their way into the cache; values into the cache.
 //                         Without key / value columns (a layer that reads another layer's cache) only the queries.
-//   lgs_normattn_prepare  per token: queries optionally divided by their root mean square (optionally weighted),
-//                         optionally rotated (pairs i, i + rot_dims / 2) and multiplied by a temperature that grows
-//                         with the position, in place; keys normed and rotated alike on their way into the cache;
-//                         values (own columns, or the keys as projected) into the cache.
+//   lgs_normattn_prepare  per token: queries optionally divided by their root mean square (per head, or all heads
+//                         together; optionally weighted), optionally rotated (pairs i, i + rot_dims / 2 or 2i, 2i + 1)
+//                         and multiplied by a temperature that grows with the position, in place; keys normed and
+//                         rotated alike on their way into the cache; values (own columns, or the keys as projected;
+//                         optionally rotated by their position) into the cache. In a step of one token per sequence
+//                         the workgroup whose token completes a pooled block also makes the block's means.
+//   lgs_pool_blocks       the same means for the blocks that a prompt step completes.
 //   lgs_diffattn,         QT consecutive queries of one sequence and one head per workgroup (8 with two maps, 16 with
 //   lgs_sinkattn          one) against key tiles of 256 cached rows: a thread per key for the scores, an online
 //                         softmax per (query, map), a thread per value column for the weighted sums. One query per
 //                         workgroup (decode) can spread its keys over several workgroups, merged by a second launch.
 #include "seq_common.h"
+
+#include <type_traits>
 
 namespace lgs {
 
@@ -90,11 +98,33 @@ struct NormPrepArgs {
   const int *slot, *pos;
   int H, G, d, dv, S, temp_every;
   float eps, temp_coef;
-  int norm;                // 0: q and k as projected; 1: divided by their root mean square
-  const float *q_w, *k_w;  // optional weights [d] of the two norms, shared by the heads
-  const float* inv_freq;   // [rot_dims / 2]: rotary positions on pairs (i, i + rot_dims / 2) after the norm
-  int rot_dims;
+  int norm;                // 0: q and k as projected; 1: each head divided by its root mean square; 2: all heads of q
+                           // (of k) divided by one root mean square
+  const float *q_w, *k_w;  // optional weights of the two norms: [d], shared by the heads, or (norm 2) [H d] / [G d]
+  const float* inv_freq;   // [rot_dims / 2]: rotary positions after the norm
+  int rot_dims, interleaved;  // pairs (2i, 2i + 1), or (i, i + rot_dims / 2)
+  const float* v_freq;     // [dv / 2]: values rotated by their position, in the same layout over dv (null: as they are)
+  float *pool_k, *pool_v;  // [slots][pool_rows][G][d], [..][dv]: means of complete blocks of `pool` positions, made here
+  int pool, pool_rows;     // when the step brings one token per sequence (pool 0: not)
 };
+
+// the means of the cached keys and values of positions b pool .. b pool + pool - 1 of one sequence: thread i walks
+// columns i, i + 256, ...; rows in ascending order
+template <bool CF32>
+__device__ __forceinline__ void pool_block(const void* cache_k, const void* cache_v, float* pool_k, float* pool_v, size_t slot,
+                                           int b, int pool, int S, int pool_rows, int nk, int nv) {
+  const float inv = 1.0f / (float)pool;
+  const size_t row0 = slot * S + (size_t)b * pool, dst = slot * pool_rows + b;
+  for (int i = threadIdx.x; i < nk + nv; i += 256) {
+    const bool isv = i >= nk;
+    const int c = isv ? i - nk : i, n = isv ? nv : nk;
+    const void* src = isv ? cache_v : cache_k;
+    float acc = 0.0f;
+#pragma unroll 8
+    for (int j = 0; j < pool; ++j) acc += cload<CF32>(src, (row0 + j) * n + c);
+    (isv ? pool_v : pool_k)[dst * n + c] = acc * inv;
+  }
+}
 
 // grid (T): wave w takes the vectors w, w + 4, ... of the H query heads (normed, rotated and multiplied by the
 // position's query temperature, in place) and of the G key heads (normed and rotated on their way into the cache);
@@ -102,6 +132,7 @@ struct NormPrepArgs {
 // keys as projected): the keys are never changed in place.
 template <bool CF32>
 __global__ void __launch_bounds__(256) normattn_prepare_kernel(NormPrepArgs p) {
+  __shared__ float red[4];
   const size_t t = blockIdx.x;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int pos = p.pos[t], d = p.d, half = p.rot_dims / 2;
@@ -110,30 +141,46 @@ __global__ void __launch_bounds__(256) normattn_prepare_kernel(NormPrepArgs p) {
   const size_t crow = ((size_t)p.slot[t] * p.S + pos) * p.G;
   const float temp = p.temp_every > 0 ? 1.0f + p.temp_coef * logf((float)((pos + 1) / p.temp_every + 1)) : 1.0f;
   const float fpos = (float)pos;
+  float qf = 1.0f, kf = 1.0f;  // the joint norm's factors
+  if (p.norm == 2) {
+    const float *q = row + p.q_off, *k = row + p.k_off;
+    float sq = 0.0f, sk = 0.0f;
+    for (int i = threadIdx.x; i < p.H * d; i += 256) sq = fmaf(q[i], q[i], sq);
+    for (int i = threadIdx.x; i < p.G * d; i += 256) sk = fmaf(k[i], k[i], sk);
+    sq = block_sum_256(sq, red);
+    sk = block_sum_256(sk, red);
+    qf = 1.0f / sqrtf(sq / (float)(p.H * d) + p.eps);
+    kf = 1.0f / sqrtf(sk / (float)(p.G * d) + p.eps);
+  }
+  const int st = p.interleaved ? 2 : 1, mate = p.interleaved ? 1 : half;  // pair i: elements st i and st i + mate
   for (int vec = wave; vec < p.H + p.G; vec += 4) {
     const bool isk = vec >= p.H;
     float* x = row + (isk ? p.k_off + (size_t)(vec - p.H) * d : p.q_off + (size_t)vec * d);
     const float* w = isk ? p.k_w : p.q_w;
+    if (w && p.norm == 2) w += (size_t)(isk ? vec - p.H : vec) * d;
     float s = isk ? 1.0f : temp;  // the norm's factor and the query temperature as one number
-    if (p.norm) {
+    if (p.norm == 1) {
       float ss = 0.0f;
       for (int i = lane; i < d; i += 64) ss = fmaf(x[i], x[i], ss);
       ss = wave_sum(ss);
       s = s / sqrtf(ss / (float)d + p.eps);
+    } else if (p.norm == 2) {
+      s *= isk ? kf : qf;
     }
     const size_t kat = (crow + (vec - p.H)) * d;
     for (int i = lane; i < half; i += 64) {  // a lane owns both members of a rotated pair
-      float u = x[i] * s, v = x[i + half] * s;
-      if (w) u *= w[i], v *= w[i + half];
+      const int e = st * i, f = e + mate;
+      float u = x[e] * s, v = x[f] * s;
+      if (w) u *= w[e], v *= w[f];
       float sn, cs;
       sincosf(fpos * p.inv_freq[i], &sn, &cs);
       const float a = u * cs - v * sn, b = v * cs + u * sn;
       if (isk) {
-        cstore<CF32>(p.cache_k, kat + i, a);
-        cstore<CF32>(p.cache_k, kat + i + half, b);
+        cstore<CF32>(p.cache_k, kat + e, a);
+        cstore<CF32>(p.cache_k, kat + f, b);
       } else {
-        x[i] = a;
-        x[i + half] = b;
+        x[e] = a;
+        x[f] = b;
       }
     }
     for (int i = p.rot_dims + lane; i < d; i += 64) {
@@ -145,7 +192,42 @@ __global__ void __launch_bounds__(256) normattn_prepare_kernel(NormPrepArgs p) {
   }
   __syncthreads();
   const int nv = p.G * p.dv;
-  for (int i = threadIdx.x; i < nv; i += 256) cstore<CF32>(p.cache_v, crow * p.dv + i, row[p.v_off + i]);
+  if (p.v_freq) {
+    const int hv = p.dv / 2, vmate = p.interleaved ? 1 : hv;
+    for (int i = threadIdx.x; i < p.G * hv; i += 256) {
+      const int g = i / hv, m = i % hv, e = g * p.dv + st * m;
+      const float u = row[p.v_off + e], v = row[p.v_off + e + vmate];
+      float sn, cs;
+      sincosf(fpos * p.v_freq[m], &sn, &cs);
+      cstore<CF32>(p.cache_v, crow * p.dv + e, u * cs - v * sn);
+      cstore<CF32>(p.cache_v, crow * p.dv + e + vmate, v * cs + u * sn);
+    }
+  } else {
+    for (int i = threadIdx.x; i < nv; i += 256) cstore<CF32>(p.cache_v, crow * p.dv + i, row[p.v_off + i]);
+  }
+  if (p.pool > 0 && (pos + 1) % p.pool == 0 && (pos + 1) / p.pool <= p.pool_rows) {
+    __syncthreads();  // this token's key and value are in the cache, the block's earlier ones since earlier steps
+    pool_block<CF32>(p.cache_k, p.cache_v, p.pool_k, p.pool_v, (size_t)p.slot[t], (pos + 1) / p.pool - 1, p.pool, p.S,
+                     p.pool_rows, p.G * d, nv);
+  }
+}
+
+struct PoolArgs {
+  const void *cache_k, *cache_v;
+  float *pool_k, *pool_v;
+  const int *seq_start, *seq_slot, *seq_pos0;
+  int G, d, dv, S, pool, pool_rows;
+};
+
+// grid (ceil(max_len / pool), B): the j-th block that sequence b completes in this step
+template <bool CF32>
+__global__ void __launch_bounds__(256) pool_blocks_kernel(PoolArgs p) {
+  const int b = blockIdx.y, pos0 = p.seq_pos0[b];
+  const int end = min(pos0 + p.seq_start[b + 1] - p.seq_start[b], p.S);  // positions held after the step
+  const int blk = pos0 / p.pool + blockIdx.x;
+  if (blk >= end / p.pool || blk >= p.pool_rows) return;
+  pool_block<CF32>(p.cache_k, p.cache_v, p.pool_k, p.pool_v, (size_t)p.seq_slot[b], blk, p.pool, p.S, p.pool_rows, p.G * p.d,
+                   p.G * p.dv);
 }
 
 struct AttnArgs {
@@ -162,7 +244,19 @@ struct AttnArgs {
   const float* sink;  // one map: exp(sink[h]) joins the softmax normaliser (NULL: no sink)
   const float* gate;  // one map: the head's output is multiplied by sigmoid(gate[row * ldg + h]) (NULL: not)
   long ldg;
+  int gate_cols;      // 1: a gate per head (above); else one per output column, gate[row * ldg + h * dv + c]
+  int window;         // one map: a query sees the last `window` positions (0: all before it)
+  const float *pool_k, *pool_v;  // one map: pooled blocks [slots][pool_rows][G][d], [..][dv] before the window
+  int pool, pool_rows;           // (pool 0: none)
+  const float* v_freq;  // one map, [dv / 2]: the finished output is turned back by the query's position (values are
+  int interleaved;      // cached rotated), pairs (2m, 2m + 1) or (m, m + dv / 2)
 };
+
+// pooled blocks that the query at position i sees: those wholly before its window
+__device__ __forceinline__ int pooled_seen(int i, int window, int pool) {
+  const int n = i - window + 1;
+  return n > 0 ? n / pool : 0;
+}
 
 constexpr int kKeyTile = 256;
 // row stride of the score / weight tile in LDS, [key][(query, map)]: a key's weights for all queries and maps lie
@@ -185,8 +279,10 @@ __device__ __forceinline__ void diff_finish(float a1, float a2, float l1, float 
   }
 }
 
-// one map: o = a / (l + exp(sink - m)) times post, with a and l relative to the running maximum m
-__device__ __forceinline__ void sink_finish(float a, float m, float l, const AttnArgs& p, size_t row, int h) {
+// one map: o = a / (l + exp(sink - m)) times post, with a and l relative to the running maximum m; `xch` holds dv
+// floats (outputs that are turned back by the query's position). Called by all 256 threads.
+__device__ __forceinline__ void sink_finish(float a, float m, float l, const AttnArgs& p, size_t row, int h, int pos,
+                                            float* xch) {
   const int c = threadIdx.x;
   float den = l, num = a;
   if (p.sink) {
@@ -195,9 +291,23 @@ __device__ __forceinline__ void sink_finish(float a, float m, float l, const Att
     den = l * w + expf(s - top);
     num = a * w;
   }
+  float v = c < p.dv ? num / den * p.post : 0.0f;
+  if (p.v_freq) {
+    __syncthreads();  // (the previous query's exchange is read)
+    if (c < p.dv) xch[c] = v;
+    __syncthreads();
+    if (c < p.dv) {
+      const int hv = p.dv / 2;
+      const bool second = p.interleaved ? (c & 1) : c >= hv;
+      const int m = p.interleaved ? c >> 1 : (second ? c - hv : c);
+      const float o = xch[p.interleaved ? c ^ 1 : (second ? c - hv : c + hv)];
+      float sn, cs;
+      sincosf((float)pos * p.v_freq[m], &sn, &cs);
+      v = second ? v * cs - o * sn : v * cs + o * sn;  // the pair turned by -pos * f
+    }
+  }
   if (c < p.dv) {
-    float v = num / den * p.post;
-    if (p.gate) v *= sigmoid_f(p.gate[row * p.ldg + h]);
+    if (p.gate) v *= sigmoid_f(p.gate[row * p.ldg + (p.gate_cols == 1 ? (size_t)h : (size_t)h * p.dv + c)]);
     const size_t at = row * p.H * p.dv + (size_t)h * p.dv + c;
     p.out[at] = v;
     if (p.out16) p.out16[at] = f2bf(v);
@@ -207,10 +317,12 @@ __device__ __forceinline__ void sink_finish(float a, float m, float l, const Att
 // grid (B * tiles, H, splits). MAPS maps per head (2: differential attention, 1: plain softmax attention with an
 // optional sink). LDS: queries [QT][MAPS d], scores / weights [256][QT MAPS + 4], per (query, map) the running
 // maximum, normaliser and the rescale of the current tile, and the cross-subset sums of the value phase.
-template <int QT, int MAPS, bool CF32>
+// WIN: a sliding window, optionally with pooled blocks before it (one map).
+template <int QT, int MAPS, bool CF32, bool WIN>
 __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
   extern __shared__ float lds[];
   __shared__ float red[4];
+  __shared__ float xch[256];
   constexpr int NR = QT * MAPS;  // (query, map) rows
   const int d = p.d, dv = p.dv, d2 = MAPS * d;
   float* qs = lds;                       // [QT][d2]
@@ -230,10 +342,19 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
   const size_t slot = p.seq_slot[b];
   const int chunk = p.chunk;
   int lo = chunk > 0 ? pos_first - pos_first % chunk : 0, hi = pos_last + 1;
-  if (gridDim.z > 1) {  // (QT == 1) an equal share of the keys, in whole numbers
-    const int n = hi - lo, per = (n + gridDim.z - 1) / gridDim.z;
-    lo += blockIdx.z * per;
-    hi = min(hi, lo + per);
+  int plo = 0, phi = 0;  // pooled blocks
+  if (WIN) {
+    lo = max(0, pos_first - p.window + 1);
+    if (p.pool > 0) phi = min(pooled_seen(pos_last, p.window, p.pool), p.pool_rows);
+  }
+  if (gridDim.z > 1) {  // (QT == 1) an equal share of the blocks and keys, in whole numbers
+    const int np = phi, n = np + hi - lo, per = (n + gridDim.z - 1) / gridDim.z;
+    const int u0 = blockIdx.z * per, u1 = min(n, u0 + per);  // share of the blocks followed by the keys
+    plo = min(u0, np);
+    phi = max(plo, min(u1, np));
+    const int first = lo;
+    lo = first + max(u0 - np, 0);
+    hi = first + max(u1 - np, 0);
   }
   for (int i = tid; i < nq * d2; i += 256) qs[i] = p.q[(size_t)(r0 + i / d2) * p.ld + (size_t)h * d2 + i % d2];
   if (tid < NR) {
@@ -251,8 +372,12 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
     for (int m = 0; m < MAPS; ++m) acc[i][m] = 0.0f;
   __syncthreads();
 
-  for (int k0 = lo; k0 < hi; k0 += kKeyTile) {
-    const int nk = min(kKeyTile, hi - k0);
+  // key tiles of one source: the cached keys (pooled = false) or the pooled blocks, whose rows are fp32
+  auto walk = [&](auto src_f32, const bool pooled, const void* keys, const void* values, const int rows, const int from,
+                  const int to) {
+  constexpr bool KF32 = decltype(src_f32)::value;
+  for (int k0 = from; k0 < to; k0 += kKeyTile) {
+    const int nk = min(kKeyTile, to - k0);
     // ---- scores of key k0 + tid against every query and map
     {
       float s[QT][MAPS];
@@ -261,17 +386,17 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
 #pragma unroll
         for (int m = 0; m < MAPS; ++m) s[i][m] = 0.0f;
       if (tid < nk) {
-        const size_t kr = ((slot * p.S + k0 + tid) * p.G + g) * d2;
+        const size_t kr = ((slot * rows + k0 + tid) * p.G + g) * d2;
         if ((d & 3) == 0) {
 #pragma unroll
           for (int m = 0; m < MAPS; ++m)
             for (int e = 0; e < d; e += 4) {
               float kv[4];
-              if (CF32) {
-                const float4 t4 = *(const float4*)((const float*)p.cache_k + kr + m * d + e);
+              if (KF32) {
+                const float4 t4 = *(const float4*)((const float*)keys + kr + m * d + e);
                 kv[0] = t4.x, kv[1] = t4.y, kv[2] = t4.z, kv[3] = t4.w;
               } else {
-                const uint2 t2 = *(const uint2*)((const uint16_t*)p.cache_k + kr + m * d + e);
+                const uint2 t2 = *(const uint2*)((const uint16_t*)keys + kr + m * d + e);
                 kv[0] = bflo(t2.x), kv[1] = bfhi(t2.x), kv[2] = bflo(t2.y), kv[3] = bfhi(t2.y);
               }
 #pragma unroll
@@ -287,7 +412,7 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
 #pragma unroll
           for (int m = 0; m < MAPS; ++m)
             for (int e = 0; e < d; ++e) {
-              const float kv = cload<CF32>(p.cache_k, kr + m * d + e);
+              const float kv = cload<KF32>(keys, kr + m * d + e);
 #pragma unroll
               for (int i = 0; i < QT; ++i) s[i][m] = fmaf(qs[i * d2 + m * d + e], kv, s[i][m]);
             }
@@ -297,8 +422,13 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
 #pragma unroll
       for (int i = 0; i < QT; ++i) {
         const int qpos = pos_first + i;
-        const int qlo = chunk > 0 ? qpos - qpos % chunk : 0;
-        const bool see = tid < nk && i < nq && kpos <= qpos && kpos >= qlo;
+        bool see;
+        if (WIN && pooled) {
+          see = tid < nk && i < nq && kpos < pooled_seen(qpos, p.window, p.pool);
+        } else {
+          const int qlo = WIN ? qpos - p.window + 1 : (chunk > 0 ? qpos - qpos % chunk : 0);
+          see = tid < nk && i < nq && kpos <= qpos && kpos >= qlo;
+        }
 #pragma unroll
         for (int m = 0; m < MAPS; ++m) {
           float v = s[i][m] * p.scale;
@@ -344,7 +474,7 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
       if (col < dv) {
 #pragma unroll 4
         for (int j = ks; j < nk; j += KS) {
-          const float v = cload<CF32>(p.cache_v, ((slot * p.S + k0 + j) * p.G + g) * dv + col);
+          const float v = cload<KF32>(values, ((slot * rows + k0 + j) * p.G + g) * dv + col);
           float w[NR];
           if (NR == 1) {
             w[0] = sc[j * SCS];
@@ -367,6 +497,9 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
     }
     __syncthreads();
   }
+  };
+  if (WIN && phi > plo) walk(std::true_type{}, true, p.pool_k, p.pool_v, p.pool_rows, plo, phi);
+  walk(std::integral_constant<bool, CF32>{}, false, p.cache_k, p.cache_v, p.S, lo, hi);
   // ---- sum the key subsets (fixed order), then finish or leave the split's partial result
   float* xs = sc;  // [KS][NR][ncol] = 256 * NR floats <= the score tile
   if (KS > 1) {
@@ -401,7 +534,7 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
     } else if (MAPS == 2) {
       diff_finish(a[0], a[MAPS - 1], lrow[MAPS * i], lrow[MAPS * i + MAPS - 1], p, (size_t)(r0 + i), h, red);
     } else {
-      sink_finish(a[0], mrow[i], lrow[i], p, (size_t)(r0 + i), h);
+      sink_finish(a[0], mrow[i], lrow[i], p, (size_t)(r0 + i), h, pos_first + i, xch);
     }
   }
 }
@@ -410,6 +543,7 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
 template <int MAPS>
 __global__ void __launch_bounds__(256) diffattn_combine_kernel(AttnArgs p, int splits) {
   __shared__ float red[4];
+  __shared__ float xch[256];
   const size_t t = blockIdx.x;
   const int h = blockIdx.y, dv = p.dv, c = threadIdx.x;
   const int stride = MAPS * (2 + dv);
@@ -430,7 +564,7 @@ __global__ void __launch_bounds__(256) diffattn_combine_kernel(AttnArgs p, int s
     }
   }
   if (MAPS == 2) diff_finish(a[0], a[MAPS - 1], l[0], l[MAPS - 1], p, t, h, red);
-  else sink_finish(a[0], mx[0], l[0], p, t, h);
+  else sink_finish(a[0], mx[0], l[0], p, t, h, p.seq_pos0[t], xch);  // (one token per sequence: row t is sequence t)
 }
 
 template <int QT, int MAPS>
@@ -441,7 +575,9 @@ static size_t diffattn_lds(int d) {
 template <int QT, int MAPS>
 static int diffattn_launch(const AttnArgs& p, int cache_f32, dim3 grid, hipStream_t stream) {
   const size_t lds = diffattn_lds<QT, MAPS>(p.d);
-  auto* fn = cache_f32 ? diffattn_kernel<QT, MAPS, true> : diffattn_kernel<QT, MAPS, false>;
+  auto* fn = cache_f32 ? diffattn_kernel<QT, MAPS, true, false> : diffattn_kernel<QT, MAPS, false, false>;
+  if (MAPS == 1 && p.window > 0)
+    fn = cache_f32 ? diffattn_kernel<QT, MAPS, true, MAPS == 1> : diffattn_kernel<QT, MAPS, false, MAPS == 1>;
   if (lds > 48 * 1024) {
     const hipError_t e = hipFuncSetAttribute((const void*)fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) {
@@ -484,7 +620,7 @@ extern "C" int lgs_diffattn(const float* q, long ld, const void* cache_k, const 
   LGA_CHECK_ARG(splits >= 1 && splits <= 64 && (splits == 1 || (part && max_len == 1)),
                 "lgs_diffattn: splits need one token per sequence and a workspace");
   lgs::AttnArgs p{q, ld, cache_k, cache_v, seq_start, seq_slot, seq_pos0, out, (uint16_t*)out_bf16, part,
-                  H, G, d, dv, max_seq, chunk, 0, scale, cap, lambda, eps, post, nullptr, nullptr, 0};
+                  H, G, d, dv, max_seq, chunk, 0, scale, cap, lambda, eps, post};
   int rc;
   if (max_len == 1) {
     p.tiles = 1;
@@ -502,19 +638,37 @@ extern "C" int lgs_diffattn(const float* q, long ld, const void* cache_k, const 
 extern "C" int lgs_normattn_prepare(float* proj, long ld, int q_off, int k_off, int v_off, void* cache_k, void* cache_v,
                                     int cache_f32, const int* slot, const int* pos, int T, int H, int G, int d, int dv,
                                     int max_seq, float eps, float temp_coef, int temp_every, int norm, const float* q_w,
-                                    const float* k_w, const float* inv_freq, int rot_dims, hipStream_t stream) {
+                                    const float* k_w, const float* inv_freq, int rot_dims, int interleaved,
+                                    const float* v_freq, float* pool_k, float* pool_v, int pool, int pool_rows,
+                                    hipStream_t stream) {
   LGA_CHECK_ARG(proj && slot && pos && cache_k && cache_v && T > 0 && max_seq > 0, "lgs_normattn_prepare: bad arguments");
-  LGA_CHECK_ARG(H > 0 && G > 0 && H % G == 0 && d > 0 && dv > 0 && temp_every >= 0,
+  LGA_CHECK_ARG(H > 0 && G > 0 && H % G == 0 && d > 0 && dv > 0 && temp_every >= 0 && norm >= 0 && norm <= 2,
                 "lgs_normattn_prepare: heads must be a multiple of the key heads");
   LGA_CHECK_ARG(q_off >= 0 && q_off + (long)H * d <= ld && k_off >= 0 && k_off + (long)G * d <= ld && v_off >= 0 &&
                     v_off + (long)G * dv <= ld,
                 "lgs_normattn_prepare: queries, keys or values outside the row");
   LGA_CHECK_ARG(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= d && (rot_dims == 0 || inv_freq),
                 "lgs_normattn_prepare: rotary dims");
+  LGA_CHECK_ARG(!v_freq || dv % 2 == 0, "lgs_normattn_prepare: rotated values have an even size");
+  LGA_CHECK_ARG(pool >= 0 && (pool == 0 || (pool_k && pool_v && pool_rows > 0)), "lgs_normattn_prepare: pooled blocks");
   lgs::NormPrepArgs p{proj, ld, q_off, k_off, v_off, cache_k, cache_v, slot, pos, H, G, d, dv, max_seq, temp_every, eps,
-                      temp_coef, norm ? 1 : 0, q_w, k_w, inv_freq, rot_dims};
+                      temp_coef, norm, q_w, k_w, inv_freq, rot_dims, interleaved ? 1 : 0, v_freq, pool_k, pool_v, pool,
+                      pool_rows};
   if (cache_f32) lgs::normattn_prepare_kernel<true><<<T, 256, 0, stream>>>(p);
   else lgs::normattn_prepare_kernel<false><<<T, 256, 0, stream>>>(p);
+  LGA_LAUNCH_RETURN();
+}
+
+extern "C" int lgs_pool_blocks(const void* cache_k, const void* cache_v, int cache_f32, float* pool_k, float* pool_v,
+                               const int* seq_start, const int* seq_slot, const int* seq_pos0, int B, int max_len, int G,
+                               int d, int dv, int max_seq, int pool, int pool_rows, hipStream_t stream) {
+  LGA_CHECK_ARG(cache_k && cache_v && pool_k && pool_v && seq_start && seq_slot && seq_pos0, "lgs_pool_blocks: null pointer");
+  LGA_CHECK_ARG(B > 0 && B <= 65535 && max_len > 0 && G > 0 && d > 0 && dv > 0 && max_seq > 0 && pool > 0 && pool_rows > 0,
+                "lgs_pool_blocks: bad sizes");
+  lgs::PoolArgs p{cache_k, cache_v, pool_k, pool_v, seq_start, seq_slot, seq_pos0, G, d, dv, max_seq, pool, pool_rows};
+  const dim3 grid((max_len + pool - 1) / pool, B);
+  if (cache_f32) lgs::pool_blocks_kernel<true><<<grid, 256, 0, stream>>>(p);
+  else lgs::pool_blocks_kernel<false><<<grid, 256, 0, stream>>>(p);
   LGA_LAUNCH_RETURN();
 }
 
@@ -522,16 +676,23 @@ extern "C" int lgs_sinkattn(const float* q, long ld, const void* cache_k, const 
                             const float* sink, const int* seq_start, const int* seq_slot, const int* seq_pos0, float* out,
                             void* out_bf16, float* part, int splits, int B, int max_len, int H, int G, int d, int dv,
                             int max_seq, int chunk, float scale, float cap, float post, const float* gate, long ldg,
-                            hipStream_t stream) {
+                            int gate_cols, int window, const float* pool_k, const float* pool_v, int pool, int pool_rows,
+                            const float* v_freq, int interleaved, hipStream_t stream) {
   LGA_CHECK_ARG(q && cache_k && cache_v && seq_start && seq_slot && seq_pos0 && out, "lgs_sinkattn: null pointer");
-  LGA_CHECK_ARG(!gate || ldg >= H, "lgs_sinkattn: the head gates' row stride");
+  LGA_CHECK_ARG(!gate || ((gate_cols == 1 && ldg >= H) || (gate_cols == dv && ldg >= (long)H * dv)),
+                "lgs_sinkattn: gates per head or per output column, and their row stride");
   LGA_CHECK_ARG(B > 0 && max_len > 0 && H > 0 && H <= 65535 && G > 0 && H % G == 0, "lgs_sinkattn: bad sizes");
   LGA_CHECK_ARG(d > 0 && d <= 512 && dv > 0 && dv <= 256, "lgs_sinkattn: key dim <= 512, value dim <= 256");
   LGA_CHECK_ARG(ld >= (long)H * d && chunk >= 0 && max_seq > 0, "lgs_sinkattn: bad sizes");
+  LGA_CHECK_ARG(window >= 0 && (window == 0 || chunk == 0), "lgs_sinkattn: a window or chunks, not both");
+  LGA_CHECK_ARG(pool >= 0 && (pool == 0 || (window > 0 && pool_k && pool_v && pool_rows > 0)),
+                "lgs_sinkattn: pooled blocks stand before a window");
+  LGA_CHECK_ARG(!v_freq || dv % 2 == 0, "lgs_sinkattn: rotated values have an even size");
   LGA_CHECK_ARG(splits >= 1 && splits <= 64 && (splits == 1 || (part && max_len == 1)),
                 "lgs_sinkattn: splits need one token per sequence and a workspace");
   lgs::AttnArgs p{q, ld, cache_k, cache_v, seq_start, seq_slot, seq_pos0, out, (uint16_t*)out_bf16, part,
-                  H, G, d, dv, max_seq, chunk, 0, scale, cap, 0.0f, 0.0f, post, sink, gate, ldg};
+                  H, G, d, dv, max_seq, chunk, 0, scale, cap, 0.0f, 0.0f, post, sink, gate, ldg, gate_cols, window,
+                  pool_k, pool_v, pool, pool_rows, v_freq, interleaved ? 1 : 0};
   int rc;
   if (max_len == 1) {
     p.tiles = 1;

@@ -1,6 +1,6 @@
 // Linear layers, embedding and RMS norms of the layered models: fp32 activations, bf16 or fp32 weights.
 //
-//   lgs_linear     Y[z] (+)= act(A[z] W[z]^T): one entry point for every projection. Up to 8 rows run a streaming
+//   lgs_linear     Y[z] (+)= act(A[z] W[z]^T + bias): one entry point for every projection. Up to 8 rows run a streaming
 //                  GEMV (a wave per pair of output columns, 16-B weight loads, fp32 sums); more rows run 128x128
 //                  tiles of v_mfma_f32_16x16x32_bf16 (bf16 weights; A is rounded to bf16 while it is staged into
 //                  LDS) or 64x64 fp32 FMA tiles (fp32 weights). `batch` with strides runs per-head products (the
@@ -28,6 +28,7 @@ struct LinArgs {
   const int* z_start;  // batch z owns list rows [z_start[z], z_start[z + 1]) (null: rows [0, M) in every batch)
   const uint16_t* a16;  // MFMA tiles only: A as bf16 (a producer's rounded copy) instead of fp32 `a`
   uint16_t* y16;        // MFMA tiles only: Y written as bf16 (the operand of a following bf16 product), no accumulate
+  const float* bias;    // [N] added to the product ahead of the activation (null: none)
 };
 
 // ------------------------------------------------------------------------------------------------ GEMV, M <= 8
@@ -49,8 +50,12 @@ __global__ void __launch_bounds__(256) lin_gemv_kernel(LinArgs p) {
   const bool vec = (K % 8 == 0) && (p.lda % 4 == 0) && (((uintptr_t)a) % 16 == 0) && (p.sw % 8 == 0) &&
                    (((uintptr_t)p.w) % 16 == 0);
   int rows[R];
+  float bias[R];
 #pragma unroll
-  for (int r = 0; r < R; ++r) rows[r] = min(n0 + r, p.N - 1);
+  for (int r = 0; r < R; ++r) {
+    rows[r] = min(n0 + r, p.N - 1);
+    bias[r] = p.bias ? p.bias[rows[r]] : 0.0f;
+  }
   if (vec) {
 #pragma unroll 2
     for (int k = lane * 8; k < K; k += 512) {
@@ -104,7 +109,7 @@ __global__ void __launch_bounds__(256) lin_gemv_kernel(LinArgs p) {
       const float s = wave_sum(acc[m][r]);
       if (lane == 0 && m < p.M && n0 + r < p.N) {
         float* yp = p.y + (size_t)z * p.sy + (size_t)m * p.ldy + n0 + r;
-        const float v = act_f(p.act, s);
+        const float v = act_f(p.act, s + bias[r]);
         *yp = p.accumulate ? *yp + v : v;
       }
     }
@@ -226,6 +231,7 @@ __global__ void __launch_bounds__(256) lin_mfma_kernel(LinArgs p) {
   for (int j = 0; j < 4; ++j) {
     const int n = n0 + wn * 64 + j * 16 + fr;
     if (n >= p.N) continue;
+    const float bias = p.bias ? p.bias[n] : 0.0f;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
@@ -233,7 +239,7 @@ __global__ void __launch_bounds__(256) lin_mfma_kernel(LinArgs p) {
         const int m = m0 + wm * 64 + i * 16 + fk * 4 + r;
         if (m >= Mz) continue;
         const size_t at = (size_t)z * p.sy + (size_t)(r_lo + m) * p.ldy + n;
-        const float v = act_f(p.act, acc[i][j][r]);
+        const float v = act_f(p.act, acc[i][j][r] + bias);
         if (p.y16) p.y16[at] = f2bf(v);
         else p.y[at] = p.accumulate ? p.y[at] + v : v;
       }
@@ -303,7 +309,7 @@ __global__ void __launch_bounds__(256) lin_fma_kernel(LinArgs p) {
       const int n = n0 + tx + 16 * j;
       if (n >= p.N) continue;
       float* yp = ybase + (size_t)(r_lo + m) * p.ldy + n;
-      const float v = act_f(p.act, acc[i][j]);
+      const float v = act_f(p.act, acc[i][j] + (p.bias ? p.bias[n] : 0.0f));
       *yp = p.accumulate ? *yp + v : v;
     }
   }
@@ -415,7 +421,8 @@ __global__ void __launch_bounds__(256) gather_rows_kernel(const float* __restric
 
 extern "C" int lgs_linear(const void* a_any, long lda, long stride_a, const void* w, int w_f32, long stride_w, void* y_any,
                           long ldy, long stride_y, int M, int N, int K, int batch, int accumulate, int act,
-                          const int* a_rows, const int* z_start, int a_bf16, int y_bf16, hipStream_t stream) {
+                          const int* a_rows, const int* z_start, int a_bf16, int y_bf16, const float* bias,
+                          hipStream_t stream) {
   const float* a = (const float*)a_any;  // (bf16 when a_bf16)
   float* y = (float*)y_any;              // (bf16 when y_bf16)
   LGA_CHECK_ARG(a && w && y, "lgs_linear: null pointer");
@@ -427,7 +434,7 @@ extern "C" int lgs_linear(const void* a_any, long lda, long stride_a, const void
   LGA_CHECK_ARG(!y_bf16 || (!w_f32 && !accumulate && (M > 8 || z_start || a_rows)),
                 "lgs_linear: a bf16 result comes from the MFMA tiles (bf16 weights, more than 8 rows, no accumulate)");
   lgs::LinArgs p{a, lda, stride_a, w, stride_w, y, ldy, stride_y, M, N, K, accumulate, act, a_rows, z_start,
-                 a_bf16 ? (const uint16_t*)a : nullptr, y_bf16 ? (uint16_t*)y : nullptr};
+                 a_bf16 ? (const uint16_t*)a : nullptr, y_bf16 ? (uint16_t*)y : nullptr, bias};
   if (M <= 8 && !z_start && !a_rows) {
     const int R = N >= 16384 ? 4 : (N >= 4096 ? 2 : 1);
     const dim3 grid((N + 4 * R - 1) / (4 * R), batch);

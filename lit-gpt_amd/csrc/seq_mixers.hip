@@ -348,9 +348,10 @@ __global__ void __launch_bounds__(256) head_gate_kernel(float* __restrict__ o, c
 
 // ------------------------------------------------------------------------------------------------ latent attention
 struct LatPrepArgs {
-  float* proj;  // row t: queries at q_off (head h at h * (d + dr): d unrotated, dr rotated), latent row at kv_off
-  long ld;
-  int q_off, kv_off;
+  float* q;  // row t: head h at h * (d + dr): d unrotated, dr rotated
+  long ldq;
+  const float* kv;  // row t: r latent values, dr of the shared key part
+  long ldkv;
   void* cache_c;    // [slots][S][r] bf16 or fp32
   float* cache_kr;  // [slots][S][dr]
   const float* norm_w;    // [r]
@@ -367,8 +368,7 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(LatPrepArgs p) {
   const int t = blockIdx.x, tid = threadIdx.x;
   const int ps = p.pos[t];
   if (ps < 0 || ps >= p.max_seq) return;  // the host sizes the cache; never write out of bounds
-  float* row = p.proj + (size_t)t * p.ld;
-  const float* kv = row + p.kv_off;
+  const float* kv = p.kv + (size_t)t * p.ldkv;
   const size_t crow = (size_t)p.slot[t] * p.max_seq + ps;
   float ss = 0.0f;
   for (int i = tid; i < p.r; i += 256) ss = fmaf(kv[i], kv[i], ss);
@@ -394,7 +394,7 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(LatPrepArgs p) {
   }
   for (int it = tid; it < p.H * half; it += 256) {
     const int h = it / half, i = it % half;
-    float* qr = row + p.q_off + (size_t)h * (p.d + p.dr) + p.d + 2 * i;
+    float* qr = p.q + (size_t)t * p.ldq + (size_t)h * (p.d + p.dr) + p.d + 2 * i;
     float sn, cs;
     sincosf(fpos * p.inv_freq[i], &sn, &cs);
     const float u = qr[0], v = qr[1];
@@ -416,9 +416,10 @@ struct LatAttArgs {
   float* out;  // [T][H][r]
   int H, d, dr, r, max_seq;
   float scale;
+  int window;  // a query sees the last `window` rows (0: all up to its own)
 };
 
-// grid (T, H, splits): split z of (token, head) owns an equal share of the keys 0 .. pos; its wave w walks keys
+// grid (T, H, splits): split z of (token, head) owns an equal share of the keys it sees; its wave w walks keys
 // lo + w, lo + w + 4, ... four at a time (their loads in flight together) with an online softmax; lanes hold dims
 // lane + 64 e. One split finishes in place (the sink joins the denominator); several leave (max, sum, weighted sum)
 // per split in `part` [T][H][splits][r + 2] for latent_combine_kernel.
@@ -431,8 +432,9 @@ __global__ void __launch_bounds__(256) latent_attention_kernel(LatAttArgs p, flo
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r = p.r, dr = p.dr;
   const int last = min(p.pos[t], p.max_seq - 1);
-  const int share = (last + splits) / splits;  // ceil((last + 1) / splits)
-  const int lo = z * share, hi = min(last, lo + share - 1);
+  const int first = p.window > 0 ? max(0, last - p.window + 1) : 0;
+  const int share = (last - first + splits) / splits;  // ceil((last - first + 1) / splits)
+  const int lo = first + z * share, hi = min(last, lo + share - 1);
   const size_t base = (size_t)p.slot[t] * p.max_seq;
   const float* qc = p.qc + ((size_t)t * p.H + h) * r;
   const float* qr = p.proj + (size_t)t * p.ld + p.q_off + (size_t)h * (p.d + dr) + p.d;
@@ -524,8 +526,9 @@ __global__ void __launch_bounds__(256) latent_attention_vec_kernel(LatAttArgs p,
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int r = p.r, dr = p.dr;
   const int last = min(p.pos[t], p.max_seq - 1);
-  const int share = (last + splits) / splits;
-  const int lo = z * share, hi = min(last, lo + share - 1);
+  const int first = p.window > 0 ? max(0, last - p.window + 1) : 0;
+  const int share = (last - first + splits) / splits;
+  const int lo = first + z * share, hi = min(last, lo + share - 1);
   const size_t base = (size_t)p.slot[t] * p.max_seq;
   const bool live = 8 * lane < r;
   const float* qc = p.qc + ((size_t)t * p.H + h) * r + 8 * lane;
@@ -722,9 +725,10 @@ __global__ void __launch_bounds__(256) latent_attention_tile_kernel(LatTileArgs 
     prow[j] = min(pos_first + fk * 4 + j, pos_last);  // rows past the sequence's end repeat the last (not stored)
   }
   const int nkt = pos_last / 16 + 1;
-  gload(0);
+  const int kt0 = p.window > 0 ? max(0, pos_first - p.window + 1) / 16 : 0;
+  gload(kt0);
   __syncthreads();  // Kt's zero padding
-  for (int kt = 0; kt < nkt; ++kt) {
+  for (int kt = kt0; kt < nkt; ++kt) {
     lstore();
     __syncthreads();
     if (kt + 1 < nkt) gload(kt + 1);
@@ -751,16 +755,18 @@ __global__ void __launch_bounds__(256) latent_attention_tile_kernel(LatTileArgs 
       const int row = fk * 4 + j;
       float sc = ((Sp[row * 17 + fr] + Sp[(16 + row) * 17 + fr]) + (Sp[(32 + row) * 17 + fr] + Sp[(48 + row) * 17 + fr])) *
                  p.scale;
-      if (kt * 16 + fr > prow[j]) sc = -INFINITY;
+      const int key = kt * 16 + fr;
+      if (key > prow[j] || (p.window > 0 && key + p.window <= prow[j])) sc = -INFINITY;
       float mx = sc;
 #pragma unroll
       for (int x = 8; x > 0; x >>= 1) mx = fmaxf(mx, __shfl_xor(mx, x));
       const float mn = fmaxf(m[j], mx);
-      const float w = expf(sc - mn);
+      // (a window's first tile may hold no key of a row: its maximum is then still -inf)
+      const float w = mn == -INFINITY ? 0.0f : expf(sc - mn);
       float sum = w;
 #pragma unroll
       for (int x = 8; x > 0; x >>= 1) sum += __shfl_xor(sum, x);
-      corr[j] = expf(m[j] - mn);
+      corr[j] = mn == -INFINITY ? 0.0f : expf(m[j] - mn);
       l[j] = l[j] * corr[j] + sum;
       m[j] = mn;
       pj[j] = w;
@@ -892,15 +898,16 @@ extern "C" int lgs_head_gate(float* o, const float* g, long ldg, int T, int H, i
   LGA_LAUNCH_RETURN();
 }
 
-extern "C" int lgs_latent_prepare(float* proj, long ld, int q_off, int kv_off, void* cache_c, int cache_f32,
+extern "C" int lgs_latent_prepare(float* q, long ldq, const float* kv, long ldkv, void* cache_c, int cache_f32,
                                   float* cache_kr, const float* norm_w, const float* inv_freq, const int* slot,
                                   const int* pos, int T, int H, int d, int dr, int r, int rot_dims, int max_seq,
                                   float eps, hipStream_t stream) {
-  LGA_CHECK_ARG(proj && cache_c && cache_kr && norm_w && slot && pos, "lgs_latent_prepare: null pointer");
+  LGA_CHECK_ARG(q && kv && cache_c && cache_kr && norm_w && slot && pos, "lgs_latent_prepare: null pointer");
   LGA_CHECK_ARG(T > 0 && H > 0 && d >= 0 && dr >= 0 && r > 0 && max_seq > 0, "lgs_latent_prepare: bad sizes");
+  LGA_CHECK_ARG(ldq >= (long)H * (d + dr) && ldkv >= (long)r + dr, "lgs_latent_prepare: rows shorter than their parts");
   LGA_CHECK_ARG(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dr && (rot_dims == 0 || inv_freq),
                 "lgs_latent_prepare: bad rotary dims");
-  lgs::LatPrepArgs p{proj, ld, q_off, kv_off, cache_c, cache_kr, norm_w, inv_freq, slot, pos,
+  lgs::LatPrepArgs p{q, ldq, kv, ldkv, cache_c, cache_kr, norm_w, inv_freq, slot, pos,
                      H, d, dr, r, rot_dims, max_seq, eps};
   if (cache_f32) lgs::latent_prepare_kernel<true><<<T, 256, 0, stream>>>(p);
   else lgs::latent_prepare_kernel<false><<<T, 256, 0, stream>>>(p);
@@ -910,13 +917,14 @@ extern "C" int lgs_latent_prepare(float* proj, long ld, int q_off, int kv_off, v
 extern "C" int lgs_latent_attention(const float* qc, const float* proj, long ld, int q_off, const void* cache_c,
                                     int cache_f32, const float* cache_kr, const float* sink, const int* slot,
                                     const int* pos, float* out, int T, int H, int d, int dr, int r, int max_seq,
-                                    float scale, int splits, float* part, hipStream_t stream) {
+                                    float scale, int splits, float* part, int window, hipStream_t stream) {
   LGA_CHECK_ARG(qc && proj && cache_c && cache_kr && slot && pos && out, "lgs_latent_attention: null pointer");
   LGA_CHECK_ARG(T > 0 && H > 0 && H <= 65535 && r > 0 && r <= 1024 && dr >= 0 && dr <= 128 && max_seq > 0,
                 "lgs_latent_attention: latent rank must be <= 1024 and the rotated part <= 128");
   LGA_CHECK_ARG(splits >= 1 && splits <= 256 && (splits == 1 || part),
                 "lgs_latent_attention: splits in [1, 256], with a workspace of T * H * splits * (r + 2) floats");
-  lgs::LatAttArgs p{qc, proj, ld, q_off, cache_c, cache_kr, sink, slot, pos, out, H, d, dr, r, max_seq, scale};
+  LGA_CHECK_ARG(window >= 0, "lgs_latent_attention: window");
+  lgs::LatAttArgs p{qc, proj, ld, q_off, cache_c, cache_kr, sink, slot, pos, out, H, d, dr, r, max_seq, scale, window};
   const dim3 grid(T, H, splits);
   const size_t lds = (size_t)4 * r * sizeof(float);
 #define LGS_LAT(NR)                                                                                    \
@@ -940,14 +948,15 @@ extern "C" int lgs_latent_attention_tiles(const float* qc, const float* proj, lo
                                           int cache_f32, const float* cache_kr, const float* sink,
                                           const int* seq_start, const int* seq_slot, const int* seq_pos0, float* out,
                                           int B, int max_len, int H, int d, int dr, int r, int max_seq, float scale,
-                                          hipStream_t stream) {
+                                          int window, hipStream_t stream) {
   LGA_CHECK_ARG(qc && proj && cache_c && cache_kr && seq_start && seq_slot && seq_pos0 && out,
                 "lgs_latent_attention_tiles: null pointer");
-  LGA_CHECK_ARG(B > 0 && B <= 65535 && max_len > 0 && H > 0 && H <= 65535 && max_seq > 0,
+  LGA_CHECK_ARG(B > 0 && B <= 65535 && max_len > 0 && H > 0 && H <= 65535 && max_seq > 0 && window >= 0,
                 "lgs_latent_attention_tiles: bad sizes");
   LGA_CHECK_ARG(r > 0 && r <= 512 && r % 64 == 0 && dr >= 0 && dr <= 128,
                 "lgs_latent_attention_tiles: latent rank must be a multiple of 64 up to 512, the rotated part <= 128");
-  lgs::LatTileArgs p{{qc, proj, ld, q_off, cache_c, cache_kr, sink, nullptr, nullptr, out, H, d, dr, r, max_seq, scale},
+  lgs::LatTileArgs p{{qc, proj, ld, q_off, cache_c, cache_kr, sink, nullptr, nullptr, out, H, d, dr, r, max_seq, scale,
+                      window},
                      seq_start, seq_slot, seq_pos0};
   const int D = r + dr, DQ = (D + 15) / 16 * 4, KP = (4 * DQ + 31) / 32 * 32 + 2;
   const size_t lds = (size_t)(16 * KP + 2 * 4 * 16 * 17) * sizeof(float);

@@ -7,6 +7,9 @@
 //                        S <- a S + dt B x^T (S is N x dv, fp32, one per cache slot), y = S^T C + D x;
 //                        heads share B and C in groups. Token by token (decode, short portions), or for prompts
 //                        in chunks of 64 tokens as fp32 matrix products with the chunks side by side
+//   lgs_channel_scan     the selective scan with a diagonal state matrix per channel (the Mamba form):
+//                        S[n][c] <- exp(dt_c A[c][n]) S[n][c] + dt_c x_c B_n, y_c = (S C)_c + D_c x_c, times silu(z_c);
+//                        token by token, or for prompts in chunks of 64 tokens side by side
 //   lgs_gated_group_norm out = unit_rms_per_group(y * silu(z)) * w: gating first, the grouped norm on the gated values
 #include "seq_common.h"
 
@@ -368,6 +371,185 @@ static size_t ssd_lds(int N) {
   return sizeof(float) * ((size_t)2 * kSC * (NP + 4) + kSC * kXS + kSC * kGS + 3 * kSC);
 }
 
+// ------------------------------------------------------------------------------------------------ channel scan
+// Selective scan with a step size per channel and a diagonal state matrix A (channels x N): nothing is shared between
+// channels but B and C, and the decay exp(dt_c A[c][n]) differs for every (channel, state) pair, so the work is
+// elementwise: L lanes of a wave share one channel, each with NR of its N states in registers, and sum the output
+// with shuffles. Lanes of one wave that hold the same states lie side by side, so that every access to the state, the
+// inputs and the outputs is 64 / L consecutive floats. Tokens are taken kChanBatch at a time: the batch's x, z and step
+// sizes are fetched into registers, its B and C rows into LDS.
+// MODE 0, grid (blocks, 1, B): every sequence token by token from its stored state, outputs and final state.
+// The prompt form runs chunks of kChanChunk tokens side by side, grid (blocks, max_chunks, B): MODE 1 leaves every
+// chunk's state from a zero start in ws and the sum of its step sizes in wsum; channel_carry_kernel turns these into the
+// state at each chunk's start (the decay over a chunk is exp(A sum dt)) and leaves the final state in the slot;
+// MODE 2 walks every chunk from its start state and makes the outputs.
+struct ChanArgs {
+  const float* x;   // [T][inner]
+  const float* z;   // [T][ldz]
+  long ldz;
+  const float* bc;  // [T][ldbc]: dt inner values (rank) | B (N) | C (N)
+  long ldbc;
+  int rank;
+  const float* dt;  // [T][ldt] raw step sizes with their bias (null: w_dt)
+  long ldt;
+  const void* w_dt;  // [inner][rank]
+  const float* dt_bias;
+  const float* a2;   // [N][inner]
+  const float* D;
+  float* state;      // [slots][N][inner]
+  const int *seq_start, *seq_slot, *seq_pos0;
+  float* out;        // [T][inner]
+  uint16_t* out16;   // instead of out
+  int inner, N;
+  float *ws, *wsum;
+  int max_chunks;
+};
+
+constexpr int kChanChunk = 64, kChanBatch = 8;
+
+template <int L, int NR, int MODE, bool LOWRANK, bool WF32>
+__global__ void __launch_bounds__(256) channel_scan_kernel(ChanArgs p) {
+  extern __shared__ float lds[];  // [kChanBatch][2 NP] B | C of the batch's tokens; LOWRANK: then [kChanBatch][rank]
+  constexpr int NP = L * NR, CW = 64 / L;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int part = lane / CW, c = (blockIdx.x * 4 + wave) * CW + lane % CW;
+  const int b = blockIdx.z, N = p.N, inner = p.inner;
+  const bool live = c < inner;
+  const int r0 = p.seq_start[b], n_seq = p.seq_start[b + 1] - r0;
+  const int first = MODE == 0 ? 0 : blockIdx.y * kChanChunk;
+  if (first >= n_seq) return;
+  const int last = MODE == 0 ? n_seq : min(n_seq, first + kChanChunk);
+  const size_t slot = p.seq_slot[b], chunk = (size_t)b * p.max_chunks + blockIdx.y;
+  const int n0 = part * NR;
+  float S[NR], a2[NR];
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const bool in = live && n0 + i < N;
+    const size_t at = (size_t)(n0 + i) * inner + c;
+    a2[i] = in ? p.a2[at] : 0.0f;
+    S[i] = 0.0f;
+    if (MODE == 0 && in && p.seq_pos0[b] > 0) S[i] = p.state[slot * N * inner + at];
+    if (MODE == 2 && in) S[i] = p.ws[chunk * N * inner + at];
+  }
+  const float Dc = live ? p.D[c] : 0.0f;
+  const float bias = (LOWRANK && live) ? p.dt_bias[c] : 0.0f;
+  float dsum = 0.0f;
+  float* dlow = lds + kChanBatch * 2 * NP;
+  for (int t0 = first; t0 < last; t0 += kChanBatch) {
+    const int nb = min(kChanBatch, last - t0);
+    float xv[kChanBatch], zv[kChanBatch], dv[kChanBatch];
+#pragma unroll
+    for (int t = 0; t < kChanBatch; ++t) {
+      const size_t r = (size_t)(r0 + t0 + t);
+      const bool in = live && t < nb;
+      xv[t] = in ? p.x[r * inner + c] : 0.0f;
+      zv[t] = (MODE != 1 && in) ? p.z[r * p.ldz + c] : 0.0f;
+      dv[t] = (!LOWRANK && in) ? p.dt[r * p.ldt + c] : 0.0f;
+    }
+    __syncthreads();  // the previous batch's rows are read
+    for (int i = tid; i < nb * 2 * NP; i += 256) {
+      const int t = i / (2 * NP), e = i % (2 * NP), half = e / NP, n = e % NP;
+      lds[i] = n < N ? p.bc[(size_t)(r0 + t0 + t) * p.ldbc + p.rank + half * N + n] : 0.0f;
+    }
+    if (LOWRANK)
+      for (int i = tid; i < nb * p.rank; i += 256)
+        dlow[i] = aop<WF32>(p.bc[(size_t)(r0 + t0 + i / p.rank) * p.ldbc + i % p.rank]);
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < kChanBatch; ++t) {
+      if (t >= nb) break;
+      float d = dv[t];
+      if (LOWRANK) {  // the channel's lanes share its row of the step-size map
+        float acc = 0.0f;
+        if (live) {
+          const float* xr = dlow + t * p.rank;
+          if ((p.rank & 7) == 0) {
+            for (int r = 8 * part; r < p.rank; r += 8 * L) {
+              float u[8];
+              wload8<WF32>(p.w_dt, (size_t)c * p.rank + r, u);
+#pragma unroll
+              for (int e = 0; e < 8; ++e) acc = fmaf(xr[r + e], u[e], acc);
+            }
+          } else {
+            for (int r = part; r < p.rank; r += L) acc = fmaf(xr[r], wload<WF32>(p.w_dt, (size_t)c * p.rank + r), acc);
+          }
+        }
+#pragma unroll
+        for (int x = CW; x < 64; x <<= 1) acc += __shfl_xor(acc, x);
+        d = acc + bias;
+      }
+      d = softplus_f(d);
+      const float* Bt = lds + t * 2 * NP + n0;
+      const float dx = d * xv[t];
+      float acc = 0.0f;
+      if (MODE == 1) dsum += d;
+#pragma unroll
+      for (int i = 0; i < NR; ++i) {
+        S[i] = fmaf(__builtin_amdgcn_exp2f(d * a2[i]), S[i], Bt[i] * dx);
+        if (MODE != 1) acc = fmaf(S[i], Bt[NP + i], acc);
+      }
+      if (MODE != 1) {
+#pragma unroll
+        for (int x = CW; x < 64; x <<= 1) acc += __shfl_xor(acc, x);
+        if (part == 0 && live) {
+          const float zz = zv[t];
+          const float v = fmaf(Dc, xv[t], acc) * (zz / (1.0f + expf(-zz)));
+          const size_t at = (size_t)(r0 + t0 + t) * inner + c;
+          if (p.out16) p.out16[at] = f2bf(v);
+          else p.out[at] = v;
+        }
+      }
+    }
+  }
+  if (MODE == 2 || !live) return;
+  float* dst = MODE == 0 ? p.state + slot * N * inner : p.ws + chunk * N * inner;
+#pragma unroll
+  for (int i = 0; i < NR; ++i)
+    if (n0 + i < N) dst[(size_t)(n0 + i) * inner + c] = S[i];
+  if (MODE == 1 && part == 0) p.wsum[chunk * inner + c] = dsum;
+}
+
+// grid (ceil(N inner / 256), B): per (state, channel) the recurrence over the chunks of a sequence
+__global__ void __launch_bounds__(256) channel_carry_kernel(ChanArgs p) {
+  const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x, ni = (size_t)p.N * p.inner;
+  if (i >= ni) return;
+  const int b = blockIdx.y, c = (int)(i % p.inner);
+  const int n_seq = p.seq_start[b + 1] - p.seq_start[b], chunks = (n_seq + kChanChunk - 1) / kChanChunk;
+  float* st = p.state + (size_t)p.seq_slot[b] * ni + i;
+  const float a2 = p.a2[i];
+  float S = p.seq_pos0[b] > 0 ? *st : 0.0f;
+#pragma unroll 4
+  for (int k = 0; k < chunks; ++k) {
+    const size_t chunk = (size_t)b * p.max_chunks + k;
+    float* w = p.ws + chunk * ni + i;
+    const float local = *w;
+    *w = S;
+    S = fmaf(__builtin_amdgcn_exp2f(p.wsum[chunk * p.inner + c] * a2), S, local);
+  }
+  *st = S;
+}
+
+template <int L, int NR>
+static int channel_scan_launch(const ChanArgs& p, int w_f32, int B, hipStream_t stream) {
+  constexpr int CB = 4 * (64 / L);  // channels per workgroup
+  const dim3 one((p.inner + CB - 1) / CB, 1, B);
+  size_t lds = sizeof(float) * kChanBatch * 2 * L * NR;
+  if (p.w_dt) {
+    lds += sizeof(float) * kChanBatch * p.rank;
+    if (w_f32) channel_scan_kernel<L, NR, 0, true, true><<<one, 256, lds, stream>>>(p);
+    else channel_scan_kernel<L, NR, 0, true, false><<<one, 256, lds, stream>>>(p);
+  } else if (!p.ws) {
+    channel_scan_kernel<L, NR, 0, false, true><<<one, 256, lds, stream>>>(p);
+  } else {
+    const dim3 grid(one.x, p.max_chunks, B);
+    channel_scan_kernel<L, NR, 1, false, true><<<grid, 256, lds, stream>>>(p);
+    const size_t ni = (size_t)p.N * p.inner;
+    channel_carry_kernel<<<dim3((unsigned)((ni + 255) / 256), B), 256, 0, stream>>>(p);
+    channel_scan_kernel<L, NR, 2, false, true><<<grid, 256, lds, stream>>>(p);
+  }
+  return 0;
+}
+
 // grid (T, groups): out[t][g n + i] = v / sqrt(mean_g(v^2) + eps) * w[g n + i], v = y * silu(z)
 __global__ void __launch_bounds__(256) gated_group_norm_kernel(const float* __restrict__ y, const float* __restrict__ z,
                                                                long ldz, const float* __restrict__ w, float eps,
@@ -445,6 +627,41 @@ extern "C" int lgs_ssm_scan(const float* xbc, long ldx, const float* dt, long ld
   else if (nr <= 16) lgs::ssm_scan_kernel<16><<<grid, 256, 0, stream>>>(p);
   else if (nr <= 32) lgs::ssm_scan_kernel<32><<<grid, 256, 0, stream>>>(p);
   else lgs::ssm_scan_kernel<64><<<grid, 256, 0, stream>>>(p);
+  LGA_LAUNCH_RETURN();
+}
+
+extern "C" int lgs_channel_scan(const float* x, const float* z, long ldz, const float* bc, long ldbc, int rank,
+                                const float* dt_raw, long ldt, const void* w_dt, int w_f32, const float* dt_bias,
+                                const float* a2, const float* D, float* state, const int* seq_start, const int* seq_slot,
+                                const int* seq_pos0, void* out, int out_bf16, int B, int inner, int N, float* ws,
+                                float* wsum, int max_chunks, hipStream_t stream) {
+  LGA_CHECK_ARG(x && z && bc && a2 && D && state && seq_start && seq_slot && seq_pos0 && out,
+                "lgs_channel_scan: null pointer");
+  LGA_CHECK_ARG(B > 0 && B <= 65535 && inner > 0 && N > 0 && N <= 256 && rank > 0, "lgs_channel_scan: state size 1 to 256");
+  LGA_CHECK_ARG(ldz >= inner && ldbc >= (long)rank + 2L * N, "lgs_channel_scan: rows shorter than their parts");
+  LGA_CHECK_ARG((dt_raw && !w_dt && ldt >= inner) || (!dt_raw && w_dt && dt_bias && rank <= 1024),
+                "lgs_channel_scan: raw step sizes, or their low-rank map (rank <= 1024) and bias");
+  LGA_CHECK_ARG(!ws || (wsum && dt_raw && max_chunks > 0 && max_chunks <= 65535),
+                "lgs_channel_scan: the prompt form needs both workspaces and the step sizes");
+  lgs::ChanArgs p{x, z, ldz, bc, ldbc, rank, dt_raw, ldt, w_dt, dt_bias, a2, D, state, seq_start, seq_slot, seq_pos0,
+                  out_bf16 ? nullptr : (float*)out, out_bf16 ? (uint16_t*)out : nullptr, inner, N, ws, wsum, max_chunks};
+  int rc;
+  if (ws) {  // many chunks fill the chip: up to 16 states per lane
+    if (N <= 8) rc = lgs::channel_scan_launch<1, 8>(p, w_f32, B, stream);
+    else if (N <= 16) rc = lgs::channel_scan_launch<1, 16>(p, w_f32, B, stream);
+    else if (N <= 32) rc = lgs::channel_scan_launch<2, 16>(p, w_f32, B, stream);
+    else if (N <= 64) rc = lgs::channel_scan_launch<4, 16>(p, w_f32, B, stream);
+    else if (N <= 128) rc = lgs::channel_scan_launch<8, 16>(p, w_f32, B, stream);
+    else rc = lgs::channel_scan_launch<16, 16>(p, w_f32, B, stream);
+  } else {  // few tokens: more lanes per channel
+    if (N <= 4) rc = lgs::channel_scan_launch<1, 4>(p, w_f32, B, stream);
+    else if (N <= 8) rc = lgs::channel_scan_launch<2, 4>(p, w_f32, B, stream);
+    else if (N <= 16) rc = lgs::channel_scan_launch<4, 4>(p, w_f32, B, stream);
+    else if (N <= 32) rc = lgs::channel_scan_launch<8, 4>(p, w_f32, B, stream);
+    else if (N <= 64) rc = lgs::channel_scan_launch<16, 4>(p, w_f32, B, stream);
+    else rc = lgs::channel_scan_launch<16, 16>(p, w_f32, B, stream);
+  }
+  if (rc) return rc;
   LGA_LAUNCH_RETURN();
 }
 

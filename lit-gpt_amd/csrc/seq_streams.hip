@@ -7,9 +7,10 @@
 //   lgs_embed_streams   x[t][j] = table[tokens[t]] * scale for every stream j
 //   lgs_streams_step    one launch per sublayer boundary: the write-back of the sublayer that just ran (optional)
 //                       followed by the read + norm of the next one (optional), so the streams are read once
-//   lgs_sandwich_step   the boundary of layers whose sublayers are normed on the way in and out (one stream): the
-//                       norms and the average of up to two branch outputs, the output norm times the layer scale,
-//                       the residual add and the next sublayer's input norm in one launch
+//   lgs_sandwich_step   the boundary of layers with one residual whose sublayers are normed on the way in (and
+//                       optionally out): the norms and the average of up to two branch outputs, the output norm times
+//                       the layer scale, the residual add, a learned average over the depth at a layer's end, and the
+//                       next sublayer's input norm in one launch
 #include "seq_common.h"
 
 namespace lgs {
@@ -190,10 +191,13 @@ static bool streams_step_reg(const StreamArgs& p, int T, hipStream_t stream) {
 // ------------------------------------------------------------------------------------------------ sandwich norms
 // One boundary between two sublayers of a layer whose sublayers are normed on the way in AND on the way out.
 // With y0 (the sublayer that ran; up to two branches): b_i = w_i ? y_i / rms(y_i) * w_i : y_i, s = coef * sum_i b_i,
-// x <- x + s / rms(s) * post_w (post_w: the output norm's weight times the layer's per-channel scale). Then with
-// next_w: h = x / rms(x) * next_w, the next sublayer's input (fp32 and / or its bf16 rounding). Every root mean
+// x <- x + s / rms(s) * post_w (post_w: the output norm's weight times the layer's per-channel scale; null: no output
+// norm, x <- x + s). With depth_w (a layer's end, average over the depth): this x is the layer's result X_n, kept in row
+// block n of `hist` when there is room, and x <- depth_w[n] X_n + sum_{j < n} depth_w[j] hist[j]. x may be read from
+// another place (x_in) than it is written to. Then with next_w: h = x / rms(x) * next_w, the next sublayer's input (fp32 and / or its bf16 rounding). Every root mean
 // square has eps inside the root. grid (rows); a row lives in registers up to 256 * CPT columns, else it is re-read.
 struct SandwichArgs {
+  const float* x_in;
   float* x;
   const float *y0, *w0, *y1, *w1;
   float coef;
@@ -203,6 +207,9 @@ struct SandwichArgs {
   uint16_t* h16;
   float eps;
   int n;
+  float* hist;  // [hist_rows][rows][n]: X_0, X_1, ...
+  const float* depth_w;
+  int n_prev, hist_rows;
 };
 
 // sums of two values over the 256 threads of a workgroup at once (`red` holds 8 floats)
@@ -219,12 +226,13 @@ __device__ __forceinline__ void block_sum2_256(float& u, float& v, float* red) {
   v = (red[4] + red[5]) + (red[6] + red[7]);
 }
 
-template <int CPT>
+template <int CPT, bool DEPTH>
 __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
   __shared__ float red[8];
   const size_t r = blockIdx.x;
   const int n = p.n, tid = threadIdx.x;
   float* xr = p.x + r * n;
+  const float* xi = p.x_in + r * n;
   const float inv_n = 1.0f / (float)n;
   // every operand of the registers' share of the row is fetched up front, so that the reductions below wait for
   // one batch of loads only
@@ -234,13 +242,29 @@ __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
   for (int e = 0; e < CPT; ++e) {
     const int i = tid + 256 * e;
     const bool in = i < n;
-    xv[e] = in ? xr[i] : 0.0f;
+    xv[e] = in ? xi[i] : 0.0f;
     av[e] = (a && in) ? a[i] : 0.0f;
     bv[e] = (b && in) ? b[i] : 0.0f;
     w0[e] = (a && p.w0 && in) ? p.w0[i] : 1.0f;
     w1[e] = (b && p.w1 && in) ? p.w1[i] : 1.0f;
-    wp[e] = (a && in) ? p.post_w[i] : 0.0f;
+    wp[e] = (p.post_w && in) ? p.post_w[i] : 0.0f;
     wn[e] = (p.next_w && in) ? p.next_w[i] : 0.0f;
+  }
+  // the earlier layers' share of the average needs nothing of this sublayer: its loads run beside the reductions
+  const size_t hs = (size_t)gridDim.x * n;
+  float hv[CPT];
+  if (DEPTH) {
+#pragma unroll
+    for (int e = 0; e < CPT; ++e) hv[e] = 0.0f;
+#pragma unroll 2
+    for (int j = 0; j < p.n_prev; ++j) {
+      const float c = p.depth_w[j];
+#pragma unroll
+      for (int e = 0; e < CPT; ++e) {
+        const int i = tid + 256 * e;
+        if (i < n) hv[e] = fmaf(c, p.hist[j * hs + r * n + i], hv[e]);
+      }
+    }
   }
   if (a) {
     float sa = 0.0f, sb = 0.0f;
@@ -277,22 +301,47 @@ __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
       const float s = joined_at(i);
       ss = fmaf(s, s, ss);
     }
-    const float rs = 1.0f / sqrtf(block_sum_256(ss, red) * inv_n + p.eps);
+    float rs = 1.0f;
+    if (p.post_w) rs = 1.0f / sqrtf(block_sum_256(ss, red) * inv_n + p.eps);
 #pragma unroll
     for (int e = 0; e < CPT; ++e) {
       const int i = tid + 256 * e;
       if (i < n) {
-        xv[e] = fmaf(av[e] * rs, wp[e], xv[e]);
+        xv[e] = p.post_w ? fmaf(av[e] * rs, wp[e], xv[e]) : xv[e] + av[e];
+        if (!DEPTH) xr[i] = xv[e];
+      }
+    }
+    for (int i = tid + 256 * CPT; i < n; i += 256) {
+      const float s = joined_at(i);
+      xr[i] = p.post_w ? fmaf(s * rs, p.post_w[i], xi[i]) : xi[i] + s;
+    }
+  }
+  if (DEPTH) {
+    const float cn = p.depth_w[p.n_prev];
+    float* keep = p.n_prev < p.hist_rows ? p.hist + p.n_prev * hs + r * n : nullptr;
+#pragma unroll
+    for (int e = 0; e < CPT; ++e) {
+      const int i = tid + 256 * e;
+      if (i < n) {
+        if (keep) keep[i] = xv[e];
+        xv[e] = fmaf(cn, xv[e], hv[e]);
         xr[i] = xv[e];
       }
     }
-    for (int i = tid + 256 * CPT; i < n; i += 256) xr[i] = fmaf(joined_at(i) * rs, p.post_w[i], xr[i]);
+    for (int i = tid + 256 * CPT; i < n; i += 256) {
+      const float x = a ? xr[i] : xi[i];  // (a: written by this thread above)
+      float v = 0.0f;
+      for (int j = 0; j < p.n_prev; ++j) v = fmaf(p.depth_w[j], p.hist[j * hs + r * n + i], v);
+      if (keep) keep[i] = x;
+      xr[i] = fmaf(cn, x, v);
+    }
   }
   if (!p.next_w) return;
   float sx = 0.0f;
 #pragma unroll
   for (int e = 0; e < CPT; ++e) sx = fmaf(xv[e], xv[e], sx);
-  for (int i = tid + 256 * CPT; i < n; i += 256) sx = fmaf(xr[i], xr[i], sx);  // (written by this thread above)
+  const float* xs = (a || DEPTH) ? xr : xi;  // (xr: written by this thread above)
+  for (int i = tid + 256 * CPT; i < n; i += 256) sx = fmaf(xs[i], xs[i], sx);
   const float rx = 1.0f / sqrtf(block_sum_256(sx, red) * inv_n + p.eps);
 #pragma unroll
   for (int e = 0; e < CPT; ++e) {
@@ -304,7 +353,7 @@ __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
     }
   }
   for (int i = tid + 256 * CPT; i < n; i += 256) {
-    const float o = xr[i] * rx * p.next_w[i];
+    const float o = xs[i] * rx * p.next_w[i];
     if (p.h) p.h[r * n + i] = o;
     if (p.h16) p.h16[r * n + i] = f2bf(o);
   }
@@ -340,17 +389,26 @@ extern "C" int lgs_streams_step(float* x, const float* y, const float* mix, cons
   LGA_LAUNCH_RETURN();
 }
 
-extern "C" int lgs_sandwich_step(float* x, const float* y0, const float* w0, const float* y1, const float* w1,
-                                 float coef, const float* post_w, const float* next_w, float* h, void* h_bf16, float eps,
-                                 int rows, int n, hipStream_t stream) {
+extern "C" int lgs_sandwich_step(const float* x_in, float* x, const float* y0, const float* w0, const float* y1,
+                                 const float* w1, float coef, const float* post_w, const float* next_w, float* h,
+                                 void* h_bf16, float eps, int rows, int n, float* hist, const float* depth_w, int n_prev,
+                                 int hist_rows, hipStream_t stream) {
   LGA_CHECK_ARG(x && rows > 0 && n > 0, "lgs_sandwich_step: bad arguments");
-  LGA_CHECK_ARG(!y0 || post_w, "lgs_sandwich_step: a sublayer's output needs the output norm's weight");
   LGA_CHECK_ARG(y0 || !y1, "lgs_sandwich_step: a second branch without a first");
-  LGA_CHECK_ARG(y0 || next_w, "lgs_sandwich_step: nothing to do");
+  LGA_CHECK_ARG(y0 || next_w || depth_w, "lgs_sandwich_step: nothing to do");
   LGA_CHECK_ARG(!next_w || h || h_bf16, "lgs_sandwich_step: the next input needs a place");
-  lgs::SandwichArgs p{x, y0, w0, y1, w1, coef, post_w, next_w, h, (uint16_t*)h_bf16, eps, n};
-  if (n <= 1024) lgs::sandwich_step_kernel<4><<<rows, 256, 0, stream>>>(p);
-  else if (n <= 2048) lgs::sandwich_step_kernel<8><<<rows, 256, 0, stream>>>(p);
-  else lgs::sandwich_step_kernel<16><<<rows, 256, 0, stream>>>(p);
+  LGA_CHECK_ARG(!depth_w || (hist && n_prev >= 1 && n_prev <= hist_rows),
+                "lgs_sandwich_step: the average over the depth needs the earlier results");
+  lgs::SandwichArgs p{x_in ? x_in : x, x, y0, w0, y1, w1, coef, post_w, next_w, h, (uint16_t*)h_bf16, eps, n,
+                      hist, depth_w, n_prev, hist_rows};
+#define LGS_SANDWICH(CPT)                                                              \
+  do {                                                                                 \
+    if (depth_w) lgs::sandwich_step_kernel<CPT, true><<<rows, 256, 0, stream>>>(p);    \
+    else lgs::sandwich_step_kernel<CPT, false><<<rows, 256, 0, stream>>>(p);           \
+  } while (0)
+  if (n <= 1024) LGS_SANDWICH(4);
+  else if (n <= 2048) LGS_SANDWICH(8);
+  else LGS_SANDWICH(16);
+#undef LGS_SANDWICH
   LGA_LAUNCH_RETURN();
 }

@@ -171,15 +171,18 @@ name_to_config: Dict[str, Dict[str, Any]] = {c["name"]: c for c in configs}
 class RotarySpec:
     dims: int = 0
     base: float = 10000.0
-    # band-wise rescaling of the frequencies for contexts longer than the ``original`` one: wavelengths above
-    # original / low are slowed down by ``factor``, those below original / high are kept, the band between blends
-    # the two linearly in original / wavelength. Keys: factor, low, high, original.
+    # rescaling of the frequencies for longer contexts. Keys: factor alone: every frequency is divided by it (linear
+    # scaling). factor, low, high, original: band by band, wavelengths above original / low are slowed down by
+    # ``factor``, those below original / high are kept, the band between blends the two linearly in
+    # original / wavelength.
     scaling: Optional[Dict[str, float]] = None
 
     def inv_freq(self) -> List[float]:
-        """f_i = base^(-2i / dims), i < dims / 2, rescaled band by band when ``scaling`` is set; in double precision
-        (rounded once to fp32 by the caller)."""
+        """f_i = base^(-2i / dims), i < dims / 2, rescaled when ``scaling`` is set; in double precision (rounded once to
+        fp32 by the caller)."""
         out = [float(self.base) ** (-2.0 * i / self.dims) for i in range(self.dims // 2)]
+        if self.scaling and "original" not in self.scaling:
+            return [f / float(self.scaling["factor"]) for f in out]
         if self.scaling:
             factor, low, high, orig = (float(self.scaling[k]) for k in ("factor", "low", "high", "original"))
             for i, f in enumerate(out):
@@ -207,6 +210,9 @@ class MixerSpec:
     diff: float = 0.0  # differential attention: the constant of lambda; the output is scaled by 1 - diff
     softcap: float = 0.0  # attention: scores pass cap * tanh(s / cap) (0: not)
     mask_size: int = 0  # attention: a query sees keys of its own aligned chunk of this many positions (0: all before it)
+    window: int = 0  # attention: a query sees the last ``window`` keys up to its own (0: all before it)
+    pool: int = 0  # attention: beside the window, the mean key / value of every aligned block of this many positions that
+    # lies wholly before the window (0: none)
     kv_from: Optional[int] = None  # attention: the layer whose cached keys and values this layer reads
     conv: int = 0  # mamba2: taps of the short convolution
     groups: int = 0  # mamba2: groups of heads that share B and C
@@ -224,10 +230,18 @@ class MixerSpec:
     # "right.out") before the weighted sum
     # one-map softmax attention ("sink_attention" and its relatives):
     qk_norm: str = "unit"  # "none" | "unit" (divided by the root mean square) | "weight" (and times "q.norm" / "k.norm")
+    # | "joint" (all heads of q, and of k, share one root mean square; weights of the whole projection's size)
+    rot_layout: str = "half"  # rotary pairs: "half" (i, i + dims / 2) | "interleaved" (2i, 2i + 1)
+    rot_values: bool = False  # values are rotated by their position over all vdim dims, outputs turned back by the query's
+    bias: bool = False  # q, k and v have biases ("q.b" / "k.b" / "v.b")
+    out_gate: bool = False  # the concatenated heads times sigmoid(W_g h), one number per output column ("g")
     sink_kind: str = "learned"  # "none" | "learned" (a scalar per head, "sink") | "one" (a sink of score 0: 1 + sum exp)
     values: str = "own"  # "own" (a value projection) | "keys" (the keys as projected, before their norm)
     head_gate: bool = False  # every head's output times sigmoid(W_g h)_h, one number per head ("g")
     tau: float = 0.0  # gated_linear: the decay is sigmoid(z)^(1 / tau)
+    q_rank: int = 0  # latent attention: queries come from a normed latent of this size (0: straight from the input)
+    inner: int = 0  # mamba: channels
+    dt_rank: int = 0  # mamba: inner size of the low-rank step-size map
 
 
 @dataclass
@@ -253,10 +267,15 @@ class LayerSpec:
 # "key_value_attention": softmax attention whose values are the keys as projected, weighted q / k norms, a query
 # temperature and a gate per head; "gated_linear": the gated rule without the correction and a decay per key channel,
 # S <- diag(alpha) S + k v^T; "lightning": the constant-decay rule on silu(q), silu(k), silu(v);
+# "pooled_attention": biased rotary softmax attention over a window of tokens and the pooled blocks before it, a learned
+# sink, an elementwise output gate; "rotated_value_attention": windowed rotary softmax attention with jointly normed
+# queries and keys and rotated values; "mamba": selective scan with a diagonal state matrix per channel;
 # "parallel": two of these side by side (which two, the design says)
 MIXER_KINDS = ("retention", "latent_attention", "attention", "mamba2", "channel_delta", "gated_delta",
-               "sink_attention", "parallel", "rotary_attention", "key_value_attention", "gated_linear", "lightning")
-SOFTMAX_KINDS = ("sink_attention", "rotary_attention", "key_value_attention")
+               "sink_attention", "parallel", "rotary_attention", "key_value_attention", "gated_linear", "lightning",
+               "pooled_attention", "rotated_value_attention", "mamba")
+SOFTMAX_KINDS = ("sink_attention", "rotary_attention", "key_value_attention", "pooled_attention",
+                 "rotated_value_attention")
 
 
 @dataclass(frozen=True)
@@ -266,7 +285,8 @@ class LayeredDesign:
     # "parallel": x += mixer(h) + ff(h), one norm; "sequential": x += mixer(norm1 x), then x += ff(norm2 x);
     # "post": the sublayers read x itself and their OUTPUT is normed: x += m norm1(mixer(x)), then x += m norm2(ff(x))
     # "sandwich": normed on the way in and out, with a per-channel scale: x += ls1 * norm1b(mixer(norm1 x)), then
-    # x += ls2 * norm2b(ff(norm2 x))
+    # x += ls2 * norm2b(ff(norm2 x)); "prenorm": the same boundaries without an output norm, x += mixer(norm1 x), then
+    # x += ff(norm2 x) on one residual
     block: str
     norm_offset: float  # the norm multiplies by offset + stored weight
     tied_head: bool  # logits from the embedding table itself, or from a matrix of their own ("head")
@@ -281,6 +301,11 @@ class LayeredDesign:
     # "sigmoid": scores = sigmoid of every router output, the largest chosen, the score scales the expert's INPUT,
     # experts W_down relu(W_up h)^2, optional shared expert behind a sigmoid gate per token
     moe: str = "top_logits"
+    mask: str = "chunk"  # what a mixer's mask.size means: "chunk" (aligned chunks) or "window" (the last size positions)
+    # after every layer the residual becomes a learned average over the embedding output and all layers' results so far
+    # (weights "<layer>.dwa")
+    depth_average: bool = False
+    latent_sink: bool = True  # latent attention layers have a learned sink per head
     # layer type (config.json) -> (left kind, right kind, branch_norm) of the designs' two-branch mixers
     pairs: Dict[str, tuple] = field(default_factory=lambda: {"parallel": ("sink_attention", "gated_delta", False)})
 
@@ -292,6 +317,9 @@ DESIGNS: Dict[str, LayeredDesign] = {
     "Gatutar": LayeredDesign("sandwich", 0.0, False, "relu2", moe="sigmoid",
                              pairs={"parallel": ("rotary_attention", "gated_linear", True),
                                     "parallel_2": ("key_value_attention", "lightning", True)}),
+    "Zaronex": LayeredDesign("prenorm", 0.0, False, "gelu_tanh", mask="window", depth_average=True, latent_sink=False,
+                             pairs={"parallel": ("pooled_attention", "gated_linear", True),
+                                    "parallel_2": ("rotated_value_attention", "mamba", True)}),
 }
 
 
@@ -327,6 +355,8 @@ class LayeredConfig:
         n = len(self.layers)
         if not (0 <= self.loop_start <= self.loop_stop <= n) or self.loop_times < 1:
             raise ValueError(f"loop [{self.loop_start}, {self.loop_stop}) x {self.loop_times} does not fit {n} layers")
+        if self.design.depth_average and self.loop_stop > self.loop_start and self.loop_times > 1:
+            raise ValueError("a depth average has one weight vector per layer: no looped layers")
         if self.design.positions == "learned" and self.max_positions < 1:
             raise ValueError("max_positions: the design adds a learned position vector")
         for i, spec in enumerate(self.layers):
@@ -350,7 +380,15 @@ class LayeredConfig:
                         raise ValueError(f"layer {i}: tau must be positive")
                     if q.kind == "lightning" and (q.decay is None or len(q.decay) != q.heads):
                         raise ValueError(f"layer {i}: one decay per head")
-                if q.kind in ("rotary_attention", "key_value_attention"):
+                if q.kind == "mamba":
+                    if q.inner < 1 or q.dt_rank < 1 or not 1 <= q.state <= 256 or not 1 <= q.conv <= 16:
+                        raise ValueError(f"layer {i}: inner {q.inner} / dt_rank {q.dt_rank} / state {q.state} (<= 256) / "
+                                         f"convolution taps {q.conv} (<= 16)")
+                if q.kind in SOFTMAX_KINDS and (q.window < 0 or q.pool < 0 or (q.pool > 0 and q.window < 1)):
+                    raise ValueError(f"layer {i}: window {q.window} / pooled blocks of {q.pool}")
+                if q.kind in SOFTMAX_KINDS and q.rot_values and q.vdim % 2:
+                    raise ValueError(f"layer {i}: rotated values of odd size {q.vdim}")
+                if q.kind in SOFTMAX_KINDS and q.kind != "sink_attention":
                     if q.kv_heads < 1 or q.heads % q.kv_heads or not 1 <= q.dim <= 512 or not 1 <= q.vdim <= 256:
                         raise ValueError(f"layer {i}: heads {q.heads} / key heads {q.kv_heads} / dims {q.dim}, {q.vdim}")
                     if q.rot.dims % 2 or q.rot.dims > q.dim or q.q_temp_every < 0:
@@ -367,8 +405,7 @@ class LayeredConfig:
                         raise ValueError(f"layer {i}: heads {q.heads} / key heads {q.kv_heads} / dims {q.dim}, {q.vdim}")
                     if q.q_temp_every < 0:
                         raise ValueError(f"layer {i}: q_temp.every must be positive")
-            if m.kind in ("channel_delta", "gated_delta", "sink_attention", "parallel", "rotary_attention",
-                          "key_value_attention", "gated_linear", "lightning"):
+            if m.kind in ("channel_delta", "gated_delta", "parallel", "gated_linear", "lightning", "mamba") + SOFTMAX_KINDS:
                 continue
             if m.kind == "retention" and (m.decay is None or len(m.decay) != m.heads):
                 raise ValueError(f"layer {i}: retention needs one decay per head")
@@ -380,6 +417,11 @@ class LayeredConfig:
                 continue
             if m.rot.dims % 2 or m.rot.dims > (m.rot_dim if m.kind == "latent_attention" else m.dim):
                 raise ValueError(f"layer {i}: rotary dims {m.rot.dims} do not fit the head")
+            if m.kind == "latent_attention":
+                if min(m.heads, m.vdim, m.kv_rank) < 1 or m.kv_rank > 1024 or min(m.dim, m.rot_dim, m.q_rank) < 0 or \
+                        m.rot_dim > 128 or m.window < 0:
+                    raise ValueError(f"layer {i}: kv_rank {m.kv_rank} (<= 1024) / rot_dim {m.rot_dim} (<= 128) / "
+                                     f"q_rank {m.q_rank} / window {m.window}")
             if m.kind == "attention":
                 if m.kv_heads < 1 or m.heads % m.kv_heads or m.mask_size < 0 or m.vdim > 256:
                     raise ValueError(f"layer {i}: heads {m.heads} / key heads {m.kv_heads} / value dim {m.vdim}")
@@ -405,8 +447,8 @@ class LayeredConfig:
             left, right, normed = pairs[kind]
             half = 0.5 if normed else 1.0  # normed branches are averaged
             return MixerSpec(kind="parallel", heads=0, dim=0, vdim=0, rot=RotarySpec(),
-                             left=LayeredConfig._mixer_spec(left, m["left"]),
-                             right=LayeredConfig._mixer_spec(right, m["right"]),
+                             left=LayeredConfig._mixer_spec(left, m["left"], design),
+                             right=LayeredConfig._mixer_spec(right, m["right"], design),
                              left_scale=float(m.get("left_scale", half)), right_scale=float(m.get("right_scale", half)),
                              branch_norm=normed)
         rot = m.get("rot") or {}
@@ -417,6 +459,16 @@ class LayeredConfig:
             extra = dict(qk_norm="none", sink_kind="one")
         elif kind == "key_value_attention":
             extra = dict(qk_norm="weight", sink_kind="none", values="keys", head_gate=True)
+        elif kind == "pooled_attention":
+            extra = dict(qk_norm="none", sink_kind="learned", bias=True, out_gate=True)
+        elif kind == "rotated_value_attention":
+            extra = dict(qk_norm="joint", sink_kind="none", rot_layout="interleaved", rot_values=True)
+        elif kind == "latent_attention" and design is not None and not design.latent_sink:
+            extra = dict(sink_kind="none")
+        elif kind == "mamba":
+            return MixerSpec(kind=kind, heads=1, dim=0, vdim=0, rot=RotarySpec(), inner=int(m["inner"]),
+                             dt_rank=int(m["dt_rank"]), state=int(m["state"]), conv=int(m["conv"]))
+        windowed = design is not None and design.mask == "window"
         scaling = rot.get("scaling")
         return MixerSpec(kind=kind, heads=int(m["heads"]), dim=int(m.get("dim", 0)), vdim=int(m["vdim"]),
                          rot=RotarySpec(int(rot.get("dims", 0)), float(rot.get("base", 10000.0)),
@@ -426,7 +478,9 @@ class LayeredConfig:
                          kv_rank=int(m.get("kv_rank", 0)), rot_dim=int(m.get("rot_dim", 0)),
                          scale=float(m.get("scale", 1.0)), kv_heads=int(m.get("kv_heads", m["heads"])),
                          diff=float(m.get("diff", 0.0)), softcap=float(m.get("softcap") or 0.0),
-                         mask_size=int(mask.get("size") or 0),
+                         mask_size=0 if windowed else int(mask.get("size") or 0),
+                         window=int(mask.get("size") or 0) if windowed else 0,
+                         pool=int(mask.get("pool") or 0) if windowed else 0, q_rank=int(m.get("q_rank") or 0),
                          kv_from=int(m["kv_from"]) if m.get("kv_from") is not None else None,
                          conv=int(m.get("conv", 0)), groups=int(m.get("groups", 1)),
                          norm_groups=int(m.get("norm_groups", 1)), state=int(m.get("state", 0)),
@@ -470,7 +524,7 @@ class LayeredConfig:
 
 # architecture name (config.json) -> "module:class" of the model that serves it
 ARCHITECTURES: Dict[str, str] = {name: "lit_gpt.layered:LayeredGPT"
-                                 for name in ("Bavesun", "Rigulorn", "Ravelorn", "Gatutar")}
+                                 for name in ("Bavesun", "Rigulorn", "Ravelorn", "Gatutar", "Zaronex")}
 
 
 def load_config(checkpoint_dir: Union[str, Path]) -> Union[Config, LayeredConfig]:

@@ -26,6 +26,10 @@ The design named by ``config.architecture`` fixes the layer's shape (``config.de
   (RMS norms with plain weights). A two-branch mixer whose branches are each normed over the width hands both
   outputs to the boundary launch, which norms and averages them, applies the output norm and the scale, adds the
   residual and leaves the next sublayer's normed input (fp32 or its bf16 copy): one launch per sublayer boundary.
+* prenorm — the same boundaries without an output norm: x <- x + mixer(norm1 x), then x <- x + ff(norm2 x). With
+  ``depth_average`` the boundary at a layer's end also keeps the layer's result X_(i+1) and goes on with
+  x <- sum_j dwa_i[j] X_j over the embedding output X_0 and all results so far (fp32; the rows of one step only: the
+  average mixes layers, never positions).
 """
 
 from __future__ import annotations
@@ -37,7 +41,7 @@ import torch
 import torch.nn as nn
 
 from lit_gpt import seq_ops
-from lit_gpt.config import LayeredConfig, LayerSpec
+from lit_gpt.config import SOFTMAX_KINDS, LayeredConfig, LayerSpec
 from lit_gpt.mixers import (MIXERS, DenseFeedForward, GatedFeedForward, SparseFeedForward, StepBatch, StreamLinks,
                             TokenSide)
 from lit_gpt.rmsnorm import StreamRMSNorm
@@ -63,22 +67,9 @@ class LayeredBlock(nn.Module):
         if side_table is not None and "side.gate" in w:
             self.side = TokenSide(index, config.side_dim, side_table, _sub(w, "side."), eps, device, dtype)
         # one input projection for everything that reads the norm's output
-        parts, offsets, at = [], [{}, {}], 0
-        for k, mod in enumerate((self.mixer, self.mlp)):
-            if mod is None:
-                continue
-            for name, t in mod.in_parts():
-                offsets[k][name] = at
-                parts.append(t)
-                at += t.shape[0]
-                pad = -at % 8  # every part starts on a 32-byte boundary of the fp32 row
-                if pad:
-                    parts.append(torch.zeros(pad, W, dtype=t.dtype))
-                    at += pad
-        self.mixer.bind(offsets[0])
-        if self.mlp is not None:
-            self.mlp.bind(offsets[1])
-        self.register_buffer("w_in", torch.cat(parts).to(device=device, dtype=dtype).contiguous())
+        w_in, b_in = _fuse_rows([self.mixer] if self.mlp is None else [self.mixer, self.mlp], W, device, dtype)
+        self.register_buffer("w_in", w_in)
+        self.register_buffer("b_in", b_in)
 
     def forward(self, x: torch.Tensor, step: StepBatch, cache: nn.Module) -> None:
         """x (T, width) fp32, updated in place."""
@@ -88,7 +79,7 @@ class LayeredBlock(nn.Module):
         h, h16 = self.norm1(x, bf16_copy=True) if tiles16 else (self.norm1(x), None)
         n_in, W = self.w_in.shape
         proj = torch.empty(step.T, n_in, dtype=torch.float32, device=x.device)
-        seq_ops.linear(h16 if tiles16 else h, self.w_in, M=step.T, N=n_in, K=W, y=proj, lda=W, ldy=n_in)
+        seq_ops.linear(h16 if tiles16 else h, self.w_in, M=step.T, N=n_in, K=W, y=proj, lda=W, ldy=n_in, bias=self.b_in)
         self.mixer(proj, step, cache, x)
         if self.mlp is not None:
             self.mlp(proj, h, x, h16=h16)
@@ -96,19 +87,33 @@ class LayeredBlock(nn.Module):
             self.side(x, step.tokens)
 
 
-def _fuse_rows(parts, width: int, device, dtype) -> Tuple[torch.Tensor, Dict[str, int]]:
+def _fuse_rows(modules, width: int, device, dtype) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
     """Row-wise concatenation of the matrices that read one norm output, every part on a 32-byte boundary of the
-    fp32 result row; returns the matrix and each part's first row."""
-    rows, offsets, at = [], {}, 0
-    for name, t in parts:
-        offsets[name] = at
-        rows.append(t)
-        at += t.shape[0]
-        pad = -at % 8
-        if pad:
-            rows.append(torch.zeros(pad, width, dtype=t.dtype))
-            at += pad
-    return torch.cat(rows).to(device=device, dtype=dtype).contiguous(), offsets
+    fp32 result row, and of their biases (fp32, zeros for parts without one; None when no part has one). Tells every
+    module where its parts begin (``bind``)."""
+    rows, biases, at = [], {}, 0
+    for mod in modules:
+        offsets, bias = {}, mod.in_bias()
+        for name, t in mod.in_parts():
+            offsets[name] = at
+            if name in bias:
+                if bias[name].numel() != t.shape[0]:
+                    raise ValueError(f"{name}: a bias of {bias[name].numel()} values for {t.shape[0]} rows")
+                biases[at] = bias[name]
+            rows.append(t)
+            at += t.shape[0]
+            pad = -at % 8
+            if pad:
+                rows.append(torch.zeros(pad, width, dtype=t.dtype))
+                at += pad
+        mod.bind(offsets)
+    b_in = None
+    if biases:
+        b_in = torch.zeros(at, dtype=torch.float32)
+        for r0, b in biases.items():
+            b_in[r0:r0 + b.numel()] = b.to(device="cpu", dtype=torch.float32)
+        b_in = b_in.to(device)
+    return torch.cat(rows).to(device=device, dtype=dtype).contiguous(), b_in
 
 
 class Sublayer(nn.Module):
@@ -119,9 +124,9 @@ class Sublayer(nn.Module):
         super().__init__()
         self.module, self.links = module, links
         self.register_buffer("norm_w", norm_w.to(device=device, dtype=torch.float32).contiguous())
-        w_in, offsets = _fuse_rows(module.in_parts(), width, device, dtype)
-        module.bind(offsets)
+        w_in, b_in = _fuse_rows([module], width, device, dtype)
         self.register_buffer("w_in", w_in)
+        self.register_buffer("b_in", b_in)
 
     def wants_bf16(self, rows: int) -> bool:
         """Whether the norm that feeds this sublayer should also leave a bf16 copy (bf16 MFMA tiles read it)."""
@@ -131,7 +136,8 @@ class Sublayer(nn.Module):
         """h (T, width): the normed read of the streams. Returns the sublayer's output (T, width) fp32."""
         n_in, W = self.w_in.shape
         proj = torch.empty(step.T, n_in, dtype=torch.float32, device=h.device)
-        seq_ops.linear(h if h16 is None else h16, self.w_in, M=step.T, N=n_in, K=W, y=proj, lda=W, ldy=n_in)
+        seq_ops.linear(h if h16 is None else h16, self.w_in, M=step.T, N=n_in, K=W, y=proj, lda=W, ldy=n_in,
+                       bias=self.b_in)
         y = torch.empty(step.T, W, dtype=torch.float32, device=h.device)
         if cache is None:
             self.module(proj, h, y, h16=h16, accumulate=False)
@@ -179,9 +185,9 @@ class PostSublayer(nn.Module):
             raise ValueError("norm: weight and bias must have the model's width")
         self.register_buffer("norm_w", norm_w.to(device=device, dtype=torch.float32).contiguous())
         self.register_buffer("norm_b", None if norm_b is None else norm_b.to(device=device, dtype=torch.float32).contiguous())
-        w_in, offsets = _fuse_rows(module.in_parts(), width, device, dtype)
-        module.bind(offsets)
+        w_in, b_in = _fuse_rows([module], width, device, dtype)
         self.register_buffer("w_in", w_in)
+        self.register_buffer("b_in", b_in)
 
     def forward(self, x: torch.Tensor, x16: Optional[torch.Tensor], step: StepBatch, cache) -> torch.Tensor:
         """x (T, width): the residual (x16: its bf16 copy for the MFMA tiles). Returns the sublayer's output, unnormed."""
@@ -189,7 +195,8 @@ class PostSublayer(nn.Module):
         proj = None
         if self.module.wants_proj(step.T):
             proj = torch.empty(step.T, n_in, dtype=torch.float32, device=x.device)
-            seq_ops.linear(x if x16 is None else x16, self.w_in, M=step.T, N=n_in, K=W, y=proj, lda=W, ldy=n_in)
+            seq_ops.linear(x if x16 is None else x16, self.w_in, M=step.T, N=n_in, K=W, y=proj, lda=W, ldy=n_in,
+                           bias=self.b_in)
         y = torch.empty(step.T, W, dtype=torch.float32, device=x.device)
         if cache is None:
             self.module(proj, x, y, h16=x16, accumulate=False)
@@ -221,27 +228,28 @@ class PostNormBlock(nn.Module):
 
 
 class SandwichSublayer(nn.Module):
-    """One sublayer of a sandwich layer: the input norm's weight, the fused input projection of everything that reads
-    the normed input (none when the module makes its own product), the module, and the output norm's weight times the
-    layer's per-channel scale (folded once, in fp32)."""
+    """One sublayer of a sandwich or pre-norm layer: the input norm's weight, the fused input projection of everything
+    that reads the normed input (none when the module makes its own product), the module, and the output norm's weight
+    times the layer's per-channel scale (folded once, in fp32; a pre-norm layer has neither)."""
 
-    def __init__(self, module: nn.Module, norm_w: torch.Tensor, post_w: torch.Tensor, scale: Optional[torch.Tensor],
-                 width: int, device, dtype) -> None:
+    def __init__(self, module: nn.Module, norm_w: torch.Tensor, post_w: Optional[torch.Tensor],
+                 scale: Optional[torch.Tensor], width: int, device, dtype) -> None:
         super().__init__()
         self.module = module
-        for t in (norm_w, post_w) + ((scale,) if scale is not None else ()):
-            if t.numel() != width:
+        for t in (norm_w, post_w, scale):
+            if t is not None and t.numel() != width:
                 raise ValueError("norm / layer scale: one value per channel of the model's width")
         self.register_buffer("norm_w", norm_w.to(device=device, dtype=torch.float32).contiguous())
-        post = post_w.to(device=device, dtype=torch.float32)
-        if scale is not None:
-            post = post * scale.to(device=device, dtype=torch.float32)
-        self.register_buffer("post_w", post.contiguous())
+        self.register_buffer("post_w", None)
+        if post_w is not None:
+            post = post_w.to(device=device, dtype=torch.float32)
+            if scale is not None:
+                post = post * scale.to(device=device, dtype=torch.float32)
+            self.post_w = post.contiguous()
         self.register_buffer("w_in", None)
-        parts = module.in_parts()
-        if parts:
-            self.w_in, offsets = _fuse_rows(parts, width, device, dtype)
-            module.bind(offsets)
+        self.register_buffer("b_in", None)
+        if module.in_parts():
+            self.w_in, self.b_in = _fuse_rows([module], width, device, dtype)
 
     def wants_bf16(self, rows: int) -> bool:
         """Whether the norm that feeds this sublayer should leave a bf16 copy (bf16 MFMA tiles read it)."""
@@ -259,7 +267,7 @@ class SandwichSublayer(nn.Module):
         if self.w_in is not None and self.module.wants_proj(T):
             n_in = self.w_in.shape[0]
             proj = torch.empty(T, n_in, dtype=torch.float32, device=src.device)
-            seq_ops.linear(src, self.w_in, M=T, N=n_in, K=W, y=proj, lda=W, ldy=n_in)
+            seq_ops.linear(src, self.w_in, M=T, N=n_in, K=W, y=proj, lda=W, ldy=n_in, bias=self.b_in)
         y = torch.empty(T, W, dtype=torch.float32, device=src.device)
         if cache is None:
             self.module(proj, h, y, h16=h16, accumulate=False)
@@ -295,14 +303,47 @@ class SandwichBlock(nn.Module):
         return [self.sub1] if self.sub2 is None else [self.sub1, self.sub2]
 
 
+class PreNormBlock(nn.Module):
+    """x <- x + mixer(norm1 x), then x <- x + ff(norm2 x) when the layer has a feed-forward; with a depth average ``dwa``,
+    the weights of X_0 .. X_(i+1) in what the layer hands on (layer ``index`` has index + 2 of them)."""
+
+    def __init__(self, index: int, spec: LayerSpec, config: LayeredConfig, w: Dict[str, torch.Tensor], device,
+                 dtype) -> None:
+        super().__init__()
+        W, eps, design = config.width, config.norm_eps, config.design
+        if design.norm != "rms" or design.norm_offset != 0.0:
+            raise NotImplementedError("pre-norm layers use RMS norms with plain weights")
+        self.mixer = MIXERS[spec.mixer.kind](spec.mixer, W, eps, _sub(w, "mix."), device, dtype)
+        self.sub1 = SandwichSublayer(self.mixer, w["norm1"], None, None, W, device, dtype)
+        self.sub2 = None
+        if spec.mlp is not None:
+            if spec.mlp.kind != "dense" or design.dense_ff != "gelu_tanh":
+                raise NotImplementedError("pre-norm layers serve the gated dense feed-forward")
+            mlp = GatedFeedForward(spec.mlp, W, _sub(w, "mlp."), device, dtype)
+            self.sub2 = SandwichSublayer(mlp, w["norm2"], None, None, W, device, dtype)
+        self.register_buffer("dwa", None)
+        if design.depth_average:
+            if w["dwa"].numel() != index + 2:
+                raise ValueError(f"l{index}.dwa: {w['dwa'].numel()} weights, expected {index + 2}")
+            self.dwa = w["dwa"].to(device=device, dtype=torch.float32).contiguous()
+
+    def sublayers(self) -> List[SandwichSublayer]:
+        return [self.sub1] if self.sub2 is None else [self.sub1, self.sub2]
+
+
 def _mixer_shapes(p: str, m, W: int) -> Dict[str, Tuple[int, ...]]:
-    """Name -> shape of the tensors of a gated delta rule, a sink attention or a pair of them under prefix p."""
+    """Name -> shape of the tensors of a delta / gated linear / constant-decay rule, a channel scan, a one-map softmax
+    attention or a pair of them under prefix p."""
     if m.kind == "parallel":
         out = {**_mixer_shapes(p + "left.", m.left, W), **_mixer_shapes(p + "right.", m.right, W)}
         if m.branch_norm:
             out.update({p + "left.out": (W,), p + "right.out": (W,)})
         return out
-    if m.kind in ("sink_attention", "rotary_attention", "key_value_attention"):
+    if m.kind == "mamba":
+        return {p + "in": (2 * m.inner, W), p + "conv": (m.inner, m.conv), p + "conv.b": (m.inner,),
+                p + "x": (m.dt_rank + 2 * m.state, m.inner), p + "dt": (m.inner, m.dt_rank), p + "dt.b": (m.inner,),
+                p + "A_log": (m.inner, m.state), p + "D": (m.inner,), p + "o": (W, m.inner)}
+    if m.kind in SOFTMAX_KINDS:
         out = {p + "q": (m.heads * m.dim, W), p + "k": (m.kv_heads * m.dim, W)}
         if m.values == "own":
             out[p + "v"] = (m.kv_heads * m.vdim, W)
@@ -311,8 +352,16 @@ def _mixer_shapes(p: str, m, W: int) -> Dict[str, Tuple[int, ...]]:
         out[p + "o"] = (W, m.heads * m.vdim)
         if m.qk_norm == "weight":
             out.update({p + "q.norm": (m.dim,), p + "k.norm": (m.dim,)})
+        elif m.qk_norm == "joint":
+            out.update({p + "q.norm": (m.heads * m.dim,), p + "k.norm": (m.kv_heads * m.dim,)})
+        if m.bias:
+            out.update({p + "q.b": (m.heads * m.dim,), p + "k.b": (m.kv_heads * m.dim,)})
+            if m.values == "own":
+                out[p + "v.b"] = (m.kv_heads * m.vdim,)
         if m.head_gate:
             out[p + "g"] = (m.heads, W)
+        elif m.out_gate:
+            out[p + "g"] = (m.heads * m.vdim, W)
         return out
     if m.kind in ("gated_linear", "lightning"):
         qk, v = m.heads * m.dim, m.heads * m.vdim
@@ -360,7 +409,7 @@ class LayeredGPT(nn.Module):
         design = config.design
         self.sequential = design.block == "sequential"
         self.post = design.block == "post"
-        self.sandwich = design.block == "sandwich"
+        self.sandwich = design.block in ("sandwich", "prenorm")
         self.register_buffer("pos_table", None)
         if design.positions == "learned":
             t = weights["pos"]
@@ -374,8 +423,9 @@ class LayeredGPT(nn.Module):
                                         for i, spec in enumerate(config.layers))
         elif self.sandwich:
             if config.side_dim or config.streams != 1:
-                raise NotImplementedError("sandwich layers have one residual stream and no per-layer token input")
-            self.blocks = nn.ModuleList(SandwichBlock(i, spec, config, _sub(weights, f"l{i}."), device, dtype)
+                raise NotImplementedError("sandwich and pre-norm layers have one residual stream and no per-layer token input")
+            block = SandwichBlock if design.block == "sandwich" else PreNormBlock
+            self.blocks = nn.ModuleList(block(i, spec, config, _sub(weights, f"l{i}."), device, dtype)
                                         for i, spec in enumerate(config.layers))
         elif self.sequential:
             if config.side_dim:
@@ -440,6 +490,8 @@ class LayeredGPT(nn.Module):
                 out.update({p + "norm1b": (W,), p + "ls1": (W,)})
                 if spec.mlp is not None:
                     out.update({p + "norm2b": (W,), p + "ls2": (W,)})
+            if config.design.depth_average:
+                out[p + "dwa"] = (i + 2,)
             if biased:
                 out.update({name + ".b": (W,) for name in (p + "norm1", p + "norm2") if name in out})
             if config.stream_weights:
@@ -455,8 +507,7 @@ class LayeredGPT(nn.Module):
                 if m.kv_from is None:
                     out.update({p + "mix.k": (2 * m.kv_heads * m.dim, W), p + "mix.v": (m.kv_heads * m.vdim, W)})
                 out.update({p + f"mix.{n}": (m.dim,) for n in ("lq1", "lk1", "lq2", "lk2")})
-            elif m.kind in ("channel_delta", "gated_delta", "sink_attention", "parallel", "rotary_attention",
-                            "key_value_attention", "gated_linear", "lightning"):
+            elif m.kind in ("channel_delta", "gated_delta", "parallel", "gated_linear", "lightning", "mamba") + SOFTMAX_KINDS:
                 out.update(_mixer_shapes(p + "mix.", m, W))
             elif m.kind == "mamba2":
                 inner, bc = m.heads * m.vdim, 2 * m.groups * m.state
@@ -464,10 +515,17 @@ class LayeredGPT(nn.Module):
                             p + "mix.conv.b": (inner + bc,), p + "mix.dt_bias": (m.heads,), p + "mix.A_log": (m.heads,),
                             p + "mix.D": (m.heads,), p + "mix.norm": (inner,), p + "mix.o": (W, inner)})
             else:
-                out.update({p + "mix.q": (m.heads * (m.dim + m.rot_dim), W), p + "mix.dkv": (m.kv_rank + m.rot_dim, W),
+                nq = m.heads * (m.dim + m.rot_dim)
+                if m.q_rank:
+                    out.update({p + "mix.dq": (m.q_rank, W), p + "mix.dq.norm": (m.q_rank,), p + "mix.uq": (nq, m.q_rank)})
+                else:
+                    out[p + "mix.q"] = (nq, W)
+                out.update({p + "mix.dkv": (m.kv_rank + m.rot_dim, W),
                             p + "mix.dkv.norm": (m.kv_rank,), p + "mix.uk": (m.heads * m.dim, m.kv_rank),
-                            p + "mix.uv": (m.heads * m.vdim, m.kv_rank), p + "mix.sink": (m.heads,),
+                            p + "mix.uv": (m.heads * m.vdim, m.kv_rank),
                             p + "mix.g": (m.heads * m.vdim, W), p + "mix.o": (W, m.heads * m.vdim)})
+                if m.sink_kind == "learned":
+                    out[p + "mix.sink"] = (m.heads,)
             f = spec.mlp
             if f is not None and f.kind == "dense" and config.design.dense_ff == "relu2":
                 out.update({p + "mlp.up": (f.ff, W), p + "mlp.down": (W, f.ff)})
@@ -507,6 +565,13 @@ class LayeredGPT(nn.Module):
                 t = 1.0 + 0.2 * torch.randn(shape, generator=g)
             elif name.endswith("a2.b"):
                 t = 2.0 + torch.randn(shape, generator=g)
+            elif leaf == "dwa":  # mostly the layer's own result, a little of every other
+                t = 0.15 * torch.randn(shape, generator=g)
+                t[-1] += 0.8
+            elif name.endswith(("q.b", "k.b", "v.b")):
+                t = 0.3 * torch.randn(shape, generator=g)
+            elif name.endswith("dt.b"):
+                t = -1.5 + torch.randn(shape, generator=g)
             elif name.endswith(("norm1.b", "norm2.b", "final.norm.b", "correction")):
                 t = 0.1 * torch.randn(shape, generator=g)
             elif name == "pos":
@@ -620,29 +685,42 @@ class LayeredGPT(nn.Module):
         return x
 
     def _forward_sandwich(self, step: StepBatch, after_layer=None) -> torch.Tensor:
-        """The sandwich layers. Every boundary between two sublayers is one launch: the branch norms and the average of
-        a two-branch mixer, the output norm times the layer scale, the residual add, and the next sublayer's normed
-        input (for more than 8 rows with bf16 weights only its bf16 copy, unless the next module also reads it in
-        fp32). ``after_layer(run, x)``: a hook that sees the residual (T, width) after each layer run (for tests)."""
-        eps = self.config.norm_eps
-        x = seq_ops.embed(step.tokens, self.embed, self.config.embedding_scale)
-        chain = [(run, sub, self.caches[run] if k == 0 else None)
+        """The sandwich and pre-norm layers. Every boundary between two sublayers is one launch: the branch norms and the
+        average of a two-branch mixer, the output norm times the layer scale (sandwich layers), the residual add, at a
+        layer's end the average over the depth (designs that have it), and the next sublayer's normed input (for more
+        than 8 rows with bf16 weights only its bf16 copy, unless the next module also reads it in fp32).
+        ``after_layer(run, x)``: a hook that sees the residual (T, width) after each layer run (for tests)."""
+        eps, W = self.config.norm_eps, self.config.width
+        chain = [(run, self.blocks[layer], sub, self.caches[run] if k == 0 else None)
                  for run, layer in enumerate(self.runs) for k, sub in enumerate(self.blocks[layer].sublayers())]
+        hist, x_in = None, None
+        if self.config.design.depth_average:
+            # X_0 .. X_L of the step's rows; the first sublayer reads X_0 in place and the residual goes on in a row of its
+            # own (the last layer's result need not be kept)
+            hist = torch.empty(len(self.runs), step.T, W, dtype=torch.float32, device=self.device)
+            x_in = seq_ops.embed(step.tokens, self.embed, self.config.embedding_scale, out=hist[0])
+            x = torch.empty(step.T, W, dtype=torch.float32, device=self.device)
+        else:
+            x = seq_ops.embed(step.tokens, self.embed, self.config.embedding_scale)
 
         def reads(sub):  # (fp32 input wanted, bf16 copy wanted)
             b16 = sub.wants_bf16(step.T)
             return (not b16) or getattr(sub.module, "reads_f32", False), b16
 
-        f32, b16 = reads(chain[0][1])
-        h, h16 = seq_ops.sandwich_step(x, next_w=chain[0][1].norm_w, eps=eps, want_f32=f32, bf16_copy=b16)
-        for n, (run, sub, cache) in enumerate(chain):
+        f32, b16 = reads(chain[0][2])
+        h, h16 = seq_ops.sandwich_step(x if x_in is None else x_in, next_w=chain[0][2].norm_w, eps=eps, want_f32=f32,
+                                       bf16_copy=b16)
+        for n, (run, block, sub, cache) in enumerate(chain):
             branches, coef = sub(h, h16, step, cache)
-            nxt = chain[n + 1][1] if n + 1 < len(chain) else None
+            nxt = chain[n + 1][2] if n + 1 < len(chain) else None
+            ends = nxt is None or chain[n + 1][0] != run
             f32, b16 = reads(nxt) if nxt is not None else (False, False)
             h, h16 = seq_ops.sandwich_step(x, branches=branches, coef=coef, post_w=sub.post_w,
                                            next_w=nxt.norm_w if nxt is not None else None, eps=eps, want_f32=f32,
-                                           bf16_copy=b16)
-            if after_layer is not None and (nxt is None or chain[n + 1][0] != run):
+                                           bf16_copy=b16, x_in=x_in, hist=hist if ends else None,
+                                           depth_w=block.dwa if ends and hist is not None else None)
+            x_in = None
+            if after_layer is not None and ends:
                 after_layer(run, x)
         return x
 

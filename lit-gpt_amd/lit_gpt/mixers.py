@@ -7,10 +7,10 @@ module's rows of that matrix, ``bind`` tells it where they landed. Outputs are a
 stream ``x`` by the epilogue of the out-projection (or the expert combine), so a layer needs no add kernel.
 
 Mixers here: ``Retention`` (and its preset ``Lightning``: the constant-decay rule on activated projections),
-``LatentAttention``, ``DiffAttention``, ``SelectiveScan``, ``GatedDelta`` (the gated delta rule with a decay per head or
+``LatentAttention``, ``DiffAttention``, ``SelectiveScan`` (Mamba-2 form), ``ChannelScan`` (Mamba form), ``GatedDelta`` (the gated delta rule with a decay per head or
 per head and key channel), ``GatedLinearAttention`` (the gated rule without the correction), ``SinkAttention`` (one-map
-softmax attention: optional q / k norms, rotary positions, a query temperature, a learned or constant sink, values that
-are the keys, a gate per head) and ``ParallelMixer`` (two of them side by side on one input projection).
+softmax attention: optional biases, q / k norms, rotary positions, a query temperature, a window with pooled blocks
+before it, a learned or constant sink, values that are the keys or are rotated, a gate per head or per column) and ``ParallelMixer`` (two of them side by side on one input projection).
 
 A step is a packed batch (``StepBatch``): the tokens of all sequences row after row, with per-token cache slot and
 position and per-sequence row range, slot and first position, all int32 on the device. Sizes, decays, scales, rotary
@@ -27,7 +27,7 @@ import torch
 import torch.nn as nn
 
 from lit_gpt import seq_ops
-from lit_gpt.config import FeedForwardSpec, MixerSpec
+from lit_gpt.config import FeedForwardSpec, MixerSpec, RotarySpec
 from lit_gpt.model import CachePair, HeadKVCache, LatentKVCache, RetentionState, ScanState
 
 
@@ -79,6 +79,10 @@ class InputReader(nn.Module):
 
     def in_parts(self) -> List[Tuple[str, torch.Tensor]]:
         raise NotImplementedError
+
+    def in_bias(self) -> Dict[str, torch.Tensor]:
+        """Biases of some of ``in_parts``, by the part's name; added in the shared projection."""
+        return {}
 
     def bind(self, offsets: Dict[str, int]) -> None:
         self.off = dict(offsets)
@@ -150,24 +154,34 @@ class LatentAttention(InputReader):
     one rotated key part shared by all heads (interleaved rotary pairs 2i, 2i + 1). The score of head h is
     (q_h . W_uk,h c + q_rot,h . k_rot) * scale; a learned per-head sink scalar adds its exponential to the softmax normaliser. The kernels never expand
     keys or values: the query is mapped through W_uk,h first (one product per head), attention runs over the cached
-    rows [c | k_rot] for all heads alike, and W_uv,h maps the weighted latent back. Output gate sigmoid(W_g h)."""
+    rows [c | k_rot] for all heads alike, and W_uv,h maps the weighted latent back. Output gate sigmoid(W_g h).
+    ``q_rank`` > 0: the queries come from a latent of their own, q = W_uq rmsnorm(W_dq h); ``window`` > 0: a position sees
+    the last ``window`` keys."""
 
     def __init__(self, spec: MixerSpec, width: int, eps: float, w: Dict[str, torch.Tensor], device, dtype) -> None:
         super().__init__()
         self.H, self.d, self.dr, self.dv, self.r = spec.heads, spec.dim, spec.rot_dim, spec.vdim, spec.kv_rank
         self.eps, self.scale, self.rot_dims, self.dtype = eps, spec.scale, spec.rot.dims, dtype
+        self.q_rank, self.window = spec.q_rank, spec.window
         H, d, dr, dv, r = self.H, self.d, self.dr, self.dv, self.r
-        for name, shape in (("q", (H * (d + dr), width)), ("dkv", (r + dr, width)), ("g", (H * dv, width)),
-                            ("uk", (H * d, r)), ("uv", (H * dv, r)), ("o", (width, H * dv))):
+        q_shapes = (("dq", (self.q_rank, width)), ("dq.norm", (self.q_rank,)), ("uq", (H * (d + dr), self.q_rank))) \
+            if self.q_rank else (("q", (H * (d + dr), width)),)
+        for name, shape in q_shapes + (("dkv", (r + dr, width)), ("dkv.norm", (r,)), ("g", (H * dv, width)),
+                                       ("uk", (H * d, r)), ("uv", (H * dv, r)), ("o", (width, H * dv))):
             if tuple(w[name].shape) != shape:
                 raise ValueError(f"latent_attention.{name}: shape {tuple(w[name].shape)}, expected {shape}")
-        self._in = [(n, w[n]) for n in ("q", "dkv", "g")]
+        self._in = [(n, w[n]) for n in ("dq" if self.q_rank else "q", "dkv", "g")]
+        self.register_buffer("w_uq", None)
+        self.register_buffer("q_norm_w", None)
+        if self.q_rank:
+            self.w_uq = w["uq"].to(device=device, dtype=dtype).contiguous()
+            self.q_norm_w = _f32(w["dq.norm"], device)
         # per head (r, d): the key up-projection transposed, so that q_h (d values) maps to r latent coordinates
         self.register_buffer("w_ukT", w["uk"].to(device=device, dtype=dtype).view(H, d, r).transpose(1, 2).contiguous())
         self.register_buffer("w_uv", w["uv"].to(device=device, dtype=dtype).contiguous())
         self.register_buffer("w_o", w["o"].to(device=device, dtype=dtype).contiguous())
         self.register_buffer("norm_w", _f32(w["dkv.norm"], device))
-        self.register_buffer("sink", _f32(w["sink"], device) if "sink" in w else None)
+        self.register_buffer("sink", _f32(w["sink"], device) if spec.sink_kind == "learned" and "sink" in w else None)
         self.register_buffer("inv_freq", torch.tensor(spec.rot.inv_freq() or [1.0], dtype=torch.float64)
                              .to(device=device, dtype=torch.float32))
 
@@ -181,19 +195,24 @@ class LatentAttention(InputReader):
                 accumulate: bool = True) -> None:
         H, d, dr, dv, r = self.H, self.d, self.dr, self.dv, self.r
         T, ld = proj.shape
-        q_off = self.off["q"]
-        seq_ops.latent_prepare(proj, q_off, self.off["dkv"], cache.c, cache.kr, self.norm_w, self.inv_freq, step.slot,
+        if self.q_rank:  # queries from their own normed latent
+            cq = seq_ops.norm_columns(proj, self.off["dq"], self.q_norm_w, eps=self.eps, bf16=_tiles16(T, self.w_uq))
+            q, q_off, ldq = torch.empty(T, H * (d + dr), dtype=torch.float32, device=proj.device), 0, H * (d + dr)
+            seq_ops.linear(cq, self.w_uq, M=T, N=ldq, K=self.q_rank, y=q, lda=self.q_rank, ldy=ldq)
+        else:
+            q, q_off, ldq = proj, self.off["q"], ld
+        seq_ops.latent_prepare(q, q_off, proj, self.off["dkv"], cache.c, cache.kr, self.norm_w, self.inv_freq, step.slot,
                                step.pos, H=H, d=d, dr=dr, r=r, rot_dims=self.rot_dims, eps=self.eps)
         qc = torch.empty(T, H * r, dtype=torch.float32, device=proj.device)
-        seq_ops.linear(proj, self.w_ukT, M=T, N=r, K=d, y=qc, a_off=q_off, lda=ld, ldy=H * r, batch=H,
+        seq_ops.linear(q, self.w_ukT, M=T, N=r, K=d, y=qc, a_off=q_off, lda=ldq, ldy=H * r, batch=H,
                        stride_a=d + dr, stride_w=r * d, stride_y=r)
         if r % 64 == 0 and r <= 512 and T >= 8 * step.B:  # a prompt: 16-token tiles on the matrix cores
-            lat = seq_ops.latent_attention_tiles(qc, proj, q_off, cache.c, cache.kr, self.sink, step.seq_start,
+            lat = seq_ops.latent_attention_tiles(qc, q, q_off, cache.c, cache.kr, self.sink, step.seq_start,
                                                  step.seq_slot, step.seq_pos0, step.max_len or T, H=H, d=d, dr=dr,
-                                                 r=r, scale=self.scale)
+                                                 r=r, scale=self.scale, window=self.window)
         else:
-            lat = seq_ops.latent_attention(qc, proj, q_off, cache.c, cache.kr, self.sink, step.slot, step.pos, H=H,
-                                           d=d, dr=dr, r=r, scale=self.scale)
+            lat = seq_ops.latent_attention(qc, q, q_off, cache.c, cache.kr, self.sink, step.slot, step.pos, H=H,
+                                           d=d, dr=dr, r=r, scale=self.scale, window=self.window)
         att = torch.empty(T, H * dv, dtype=torch.float32, device=proj.device)
         seq_ops.linear(lat, self.w_uv, M=T, N=dv, K=r, y=att, lda=H * r, ldy=H * dv, batch=H, stride_a=r,
                        stride_w=dv * r, stride_y=dv)
@@ -301,6 +320,60 @@ class SelectiveScan(InputReader):
                                      bf16_copy=_tiles16(step.T, self.w_o))
         W = x.shape[1]
         seq_ops.linear(g, self.w_o, M=step.T, N=W, K=inner, y=x, lda=inner, ldy=W, accumulate=accumulate)
+
+
+class ChannelScan(InputReader):
+    """Selective scan in the Mamba form. W_in h is [x | z] (``inner`` channels each); x passes a short causal per-channel
+    convolution with bias and silu; W_x x is [step-size inner values (dt_rank) | B | C] (``state`` values each);
+    dt = softplus(W_dt . + bias), one per channel; per channel c and state n
+    S <- exp(-exp(A_log)[c, n] dt_c) S + dt_c x_c B_n, y_c = sum_n S[c, n] C_n + D_c x_c; then y silu(z), projected. The
+    state (S and the convolution's last taps - 1 inputs) is fp32 and lives in a cache slot."""
+
+    LOWRANK_ROWS = 8  # steps of up to this many tokens make the step sizes inside the scan's launch
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, w: Dict[str, torch.Tensor], device, dtype) -> None:
+        super().__init__()
+        self.inner, self.N, self.rank, self.taps = spec.inner, spec.state, spec.dt_rank, spec.conv
+        inner, N, R = self.inner, self.N, self.rank
+        for name, shape in (("in", (2 * inner, width)), ("conv", (inner, self.taps)), ("conv.b", (inner,)),
+                            ("x", (R + 2 * N, inner)), ("dt", (inner, R)), ("dt.b", (inner,)), ("A_log", (inner, N)),
+                            ("D", (inner,)), ("o", (width, inner))):
+            if tuple(w[name].shape) != shape:
+                raise ValueError(f"mamba.{name}: shape {tuple(w[name].shape)}, expected {shape}")
+        self._in = [("in", w["in"])]
+        for name, key in (("conv_w", "conv"), ("conv_b", "conv.b"), ("w_x", "x"), ("w_dt", "dt"), ("w_o", "o")):
+            self.register_buffer(name, w[key].to(device=device, dtype=dtype).contiguous())
+        self.register_buffer("dt_bias", _f32(w["dt.b"], device))
+        self.register_buffer("D", _f32(w["D"], device))
+        # A in units of log 2 (the kernels take powers of two), state-major so that neighbouring channels lie side by side
+        a2 = -torch.exp(w["A_log"].double()) * math.log2(math.e)
+        self.register_buffer("a2", _f32(a2.t(), device))
+
+    def in_parts(self):
+        return self._in
+
+    def build_cache(self, slots: int, max_seq_length: int, device, dtype) -> ScanState:
+        return ScanState(slots, 1, self.N, self.inner, self.taps, self.inner, device=device)
+
+    def forward(self, proj: torch.Tensor, step: StepBatch, cache: ScanState, x: torch.Tensor, accumulate: bool = True,
+                post: float = 1.0) -> None:
+        if post != 1.0:
+            raise NotImplementedError("a scaled channel scan")
+        T, W = x.shape
+        inner, N, R, dev = self.inner, self.N, self.rank, proj.device
+        tables = (step.seq_start, step.seq_slot, step.seq_pos0)
+        xc = seq_ops.conv_silu(proj, self.off["in"], self.conv_w, self.conv_b, cache.conv, *tables, step.max_len or T)
+        bc = torch.empty(T, R + 2 * N, dtype=torch.float32, device=dev)
+        seq_ops.linear(xc, self.w_x, M=T, N=R + 2 * N, K=inner, y=bc, lda=inner, ldy=R + 2 * N)
+        kw = dict(max_len=step.max_len or T, bf16=_tiles16(T, self.w_o))
+        if T <= self.LOWRANK_ROWS and R <= 1024:
+            y = seq_ops.channel_scan(xc, proj, self.off["in"] + inner, bc, R, self.a2, self.D, cache.s, *tables,
+                                     w_dt=self.w_dt, dt_bias=self.dt_bias, **kw)
+        else:
+            dt = torch.empty(T, inner, dtype=torch.float32, device=dev)
+            seq_ops.linear(bc, self.w_dt, M=T, N=inner, K=R, y=dt, lda=R + 2 * N, ldy=inner, bias=self.dt_bias)
+            y = seq_ops.channel_scan(xc, proj, self.off["in"] + inner, bc, R, self.a2, self.D, cache.s, *tables, dt=dt, **kw)
+        seq_ops.linear(y, self.w_o, M=T, N=W, K=inner, y=x, lda=inner, ldy=W, accumulate=accumulate)
 
 
 class GatedDelta(InputReader):
@@ -411,7 +484,12 @@ class SinkAttention(InputReader):
     values shared by the heads); rotary positions on the pairs (i, i + rot.dims / 2) of the first ``rot.dims`` dims
     after the norm (frequencies optionally rescaled band by band); ``sink_kind`` "none" / "learned" / "one" (a sink of
     score 0: the denominator is 1 + sum exp); ``values`` "keys": no value projection, the values are the keys as
-    projected, before their norm; ``head_gate``: head h's output times sigmoid(W_g h)_h, one number per head."""
+    projected, before their norm; ``head_gate``: head h's output times sigmoid(W_g h)_h, one number per head;
+    ``out_gate``: one number per output column; ``qk_norm`` "joint": all heads of q (of k) share one root mean square;
+    ``rot_layout`` "interleaved": pairs (2i, 2i + 1); ``bias``: biases on q, k and v, added in the shared projection;
+    ``rot_values``: values are rotated by their position over all vdim dims (base of the keys' rotation, not rescaled) and
+    every output is turned back by the query's position; ``window`` / ``pool``: a position sees the last ``window``
+    tokens, and the mean key and value of every block of ``pool`` tokens that lies wholly before these."""
 
     def __init__(self, spec: MixerSpec, width: int, eps: float, w: Dict[str, torch.Tensor], device, dtype) -> None:
         super().__init__()
@@ -423,14 +501,17 @@ class SinkAttention(InputReader):
         H, G, d, dv = self.H, self.G, self.d, self.dv
         shapes = [("q", (H * d, width)), ("k", (G * d, width)), ("o", (width, H * dv))]
         shapes += [("v", (G * dv, width))] if self.own_values else []
-        shapes += [("g", (H, width))] if self.head_gate else []
+        self.joint, self.interleaved, self.out_gate = spec.qk_norm == "joint", spec.rot_layout == "interleaved", spec.out_gate
+        self.window, self.pool = spec.window, spec.pool
+        shapes += [("g", (H, width))] if self.head_gate else ([("g", (H * dv, width))] if self.out_gate else [])
         for name, shape in shapes:
             if tuple(w[name].shape) != shape:
                 raise ValueError(f"{spec.kind}.{name}: shape {tuple(w[name].shape)}, expected {shape}")
         if not self.own_values and dv != d:
             raise ValueError(f"{spec.kind}: values that are the keys have the keys' size")
         self._in = [(n, w[n]) for n in (("q", "k", "v") if self.own_values else ("q", "k"))]
-        self._in += [("g", w["g"])] if self.head_gate else []
+        self._in += [("g", w["g"])] if self.head_gate or self.out_gate else []
+        self._bias = {n: w[n + ".b"] for n in ("q", "k") + (("v",) if self.own_values else ())} if spec.bias else {}
         self.register_buffer("sink", None)
         if spec.sink_kind == "one":
             self.sink = torch.zeros(H, dtype=torch.float32, device=device)
@@ -440,33 +521,48 @@ class SinkAttention(InputReader):
             self.sink = _f32(w["sink"], device)
         self.register_buffer("q_norm", None)
         self.register_buffer("k_norm", None)
-        if self.qk_norm == "weight":
-            if w["q.norm"].numel() != d or w["k.norm"].numel() != d:
-                raise ValueError(f"{spec.kind}: q.norm / k.norm hold {d} values")
+        if self.qk_norm in ("weight", "joint"):
+            if w["q.norm"].numel() != (H * d if self.joint else d) or w["k.norm"].numel() != (G * d if self.joint else d):
+                raise ValueError(f"{spec.kind}: q.norm / k.norm hold {w['q.norm'].numel()} / {w['k.norm'].numel()} values")
             self.q_norm, self.k_norm = _f32(w["q.norm"], device), _f32(w["k.norm"], device)
         self.register_buffer("inv_freq", None)
         if self.rot_dims > 0:
             self.inv_freq = torch.tensor(spec.rot.inv_freq(), dtype=torch.float64).to(device=device, dtype=torch.float32)
+        self.register_buffer("v_freq", None)
+        if spec.rot_values:
+            self.v_freq = torch.tensor(RotarySpec(dv, spec.rot.base).inv_freq(), dtype=torch.float64).to(
+                device=device, dtype=torch.float32)
         self.register_buffer("w_o", w["o"].to(device=device, dtype=dtype).contiguous())
 
     def in_parts(self):
         return self._in
 
+    def in_bias(self):
+        return self._bias
+
     def build_cache(self, slots: int, max_seq_length: int, device, dtype) -> HeadKVCache:
-        return HeadKVCache(slots, max_seq_length, self.G, self.d, self.dv, device=device, dtype=dtype)
+        return HeadKVCache(slots, max_seq_length, self.G, self.d, self.dv, device=device, dtype=dtype, pool=self.pool)
 
     def forward(self, proj: torch.Tensor, step: StepBatch, cache: HeadKVCache, x: torch.Tensor, accumulate: bool = True,
                 post: float = 1.0) -> None:
         H, G, d, dv = self.H, self.G, self.d, self.dv
+        one = step.max_len == 1  # one token per sequence: blocks that it completes are pooled inside the preparation
         seq_ops.normattn_prepare(proj, self.off["q"], self.off["k"], self.off["v" if self.own_values else "k"], cache.k,
                                  cache.v, step.slot, step.pos, H=H, G=G, d=d, dv=dv, eps=self.eps,
-                                 temp_coef=self.temp_coef, temp_every=self.temp_every, norm=self.qk_norm != "none",
+                                 temp_coef=self.temp_coef, temp_every=self.temp_every,
+                                 norm=0 if self.qk_norm == "none" else (2 if self.joint else 1),
                                  q_weight=self.q_norm, k_weight=self.k_norm, inv_freq=self.inv_freq,
-                                 rot_dims=self.rot_dims)
+                                 rot_dims=self.rot_dims, interleaved=self.interleaved, v_freq=self.v_freq,
+                                 pooled=cache.pooled if one else None, pool=self.pool)
+        if self.pool and not one:
+            seq_ops.pool_blocks(cache.k, cache.v, cache.pooled, self.pool, step.seq_start, step.seq_slot, step.seq_pos0,
+                                step.max_len or step.T)
         att = seq_ops.sinkattn(proj, self.off["q"], cache.k, cache.v, self.sink, step.seq_start, step.seq_slot,
                                step.seq_pos0, step.max_len or step.T, H=H, G=G, d=d, dv=dv, scale=self.scale,
                                chunk=self.chunk, cap=self.cap, post=post, bf16_copy=_tiles16(step.T, self.w_o),
-                               gate_off=self.off["g"] if self.head_gate else -1)
+                               gate_off=self.off["g"] if self.head_gate or self.out_gate else -1,
+                               gate_cols=dv if self.out_gate else 1, window=self.window, pooled=cache.pooled,
+                               pool=self.pool, v_freq=self.v_freq, interleaved=self.interleaved)
         W = x.shape[1]
         seq_ops.linear(att, self.w_o, M=step.T, N=W, K=H * dv, y=x, lda=H * dv, ldy=W, accumulate=accumulate)
 
@@ -565,6 +661,10 @@ class ParallelMixer(InputReader):
 
     def in_parts(self):
         return [("left." + n, t) for n, t in self.left.in_parts()] + [("right." + n, t) for n, t in self.right.in_parts()]
+
+    def in_bias(self):
+        return {**{"left." + n: t for n, t in self.left.in_bias().items()},
+                **{"right." + n: t for n, t in self.right.in_bias().items()}}
 
     def bind(self, offsets: Dict[str, int]) -> None:
         self.left.bind({k[5:]: v for k, v in offsets.items() if k.startswith("left.")})
@@ -840,4 +940,5 @@ class TokenSide(nn.Module):
 MIXERS = {"retention": Retention, "latent_attention": LatentAttention, "attention": DiffAttention,
           "mamba2": SelectiveScan, "channel_delta": GatedDelta, "gated_delta": GatedDelta,
           "sink_attention": SinkAttention, "parallel": ParallelMixer, "rotary_attention": SinkAttention,
-          "key_value_attention": SinkAttention, "gated_linear": GatedLinearAttention, "lightning": Lightning}
+          "key_value_attention": SinkAttention, "gated_linear": GatedLinearAttention, "lightning": Lightning,
+          "pooled_attention": SinkAttention, "rotated_value_attention": SinkAttention, "mamba": ChannelScan}

@@ -681,12 +681,20 @@ class HeadKVCache(nn.Module):
     """Cache of an attention mixer with key / value heads of its own: per slot and position the rotated keys
     ``k`` (kv heads, key size) and the values ``v`` (kv heads, value size), in the compute dtype. A layer that reads
     another layer's keys and values is handed that layer's instance. A slot that is given out again needs no
-    clearing: a sequence reads only the rows it has written."""
+    clearing: a sequence reads only the rows it has written. With ``pool`` also the means ``pk`` / ``pv`` of the keys and
+    values of every complete block of ``pool`` positions (fp32), which attention sees in place of the block's tokens once
+    these have left its window."""
 
     def __init__(self, slots: int, max_seq_length: int, kv_heads: int, key_size: int, value_size: int,
-                 device: Optional[torch.device] = None, dtype: Optional[torch.dtype] = None) -> None:
+                 device: Optional[torch.device] = None, dtype: Optional[torch.dtype] = None, pool: int = 0) -> None:
         super().__init__()
         dtype = dtype or torch.bfloat16
+        self.register_buffer("pk", None, persistent=False)
+        self.register_buffer("pv", None, persistent=False)
+        if pool > 0:
+            blocks = max(1, max_seq_length // pool)
+            self.pk = torch.zeros(slots, blocks, kv_heads, key_size, device=device, dtype=torch.float32)
+            self.pv = torch.zeros(slots, blocks, kv_heads, value_size, device=device, dtype=torch.float32)
         self.register_buffer("k", torch.zeros(slots, max_seq_length, kv_heads, key_size, device=device, dtype=dtype),
                              persistent=False)
         self.register_buffer("v", torch.zeros(slots, max_seq_length, kv_heads, value_size, device=device, dtype=dtype),
@@ -696,13 +704,20 @@ class HeadKVCache(nn.Module):
     def slots(self) -> int:
         return self.k.size(0)
 
+    @property
+    def pooled(self):
+        return None if self.pk is None else (self.pk, self.pv)
+
     def grow(self, slots: int) -> None:
         if slots > self.slots:
             self.k, self.v = _grown(self.k, slots), _grown(self.v, slots)
+            if self.pk is not None:
+                self.pk, self.pv = _grown(self.pk, slots), _grown(self.pv, slots)
 
     def reset_parameters(self) -> None:
-        torch.nn.init.zeros_(self.k)
-        torch.nn.init.zeros_(self.v)
+        for t in (self.k, self.v, self.pk, self.pv):
+            if t is not None:
+                torch.nn.init.zeros_(t)
 
 
 class ScanState(nn.Module):

@@ -31,21 +31,21 @@ _P, _I, _L, _F = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
 SIGNATURES = {
     "lgs_version": [],
     "lgs_last_error_string": [],
-    "lgs_linear": [_P, _L, _L, _P, _I, _L, _P, _L, _L, _I, _I, _I, _I, _I, _I, _P, _P, _I, _I, _P],
+    "lgs_linear": [_P, _L, _L, _P, _I, _L, _P, _L, _L, _I, _I, _I, _I, _I, _I, _P, _P, _I, _I, _P, _P],
     "lgs_embed": [_P, _P, _I, _F, _P, _I, _I, _I, _P],
     "lgs_rmsnorm": [_P, _L, _P, _F, _F, _P, _L, _I, _I, _I, _P, _P],
     "lgs_gather_rows": [_P, _P, _P, _I, _I, _P],
     "lgs_retention": [_P, _P, _P, _L, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _I, _I, _P, _I, _P],
     "lgs_head_gate": [_P, _P, _L, _I, _I, _I, _I, _F, _I, _P, _F, _P, _P, _I, _I, _P],
-    "lgs_latent_prepare": [_P, _L, _I, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P],
-    "lgs_latent_attention": [_P, _P, _L, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P],
-    "lgs_latent_attention_tiles": [_P, _P, _L, _I, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P],
+    "lgs_latent_prepare": [_P, _L, _P, _L, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P],
+    "lgs_latent_attention": [_P, _P, _L, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P, _I, _P],
+    "lgs_latent_attention_tiles": [_P, _P, _L, _I, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P],
     "lgs_glu": [_P, _P, _L, _P, _I, _I, _I, _I, _P],
     "lgs_moe_route": [_P, _L, _I, _I, _I, _P, _P, _P],
     "lgs_moe_route_scores": [_P, _L, _I, _I, _I, _P, _P, _P, _I, _I, _P],
     "lgs_moe_router": [_P, _L, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P],
     "lgs_act_rows": [_P, _L, _P, _L, _P, _I, _I, _I, _I, _P],
-    "lgs_sandwich_step": [_P, _P, _P, _P, _P, _F, _P, _P, _P, _P, _F, _I, _I, _P],
+    "lgs_sandwich_step": [_P, _P, _P, _P, _P, _P, _F, _P, _P, _P, _P, _F, _I, _I, _P, _P, _I, _I, _P],
     "lgs_moe_up": [_P, _L, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "lgs_moe_down": [_P, _P, _I, _P, _P, _P, _L, _I, _I, _I, _I, _I, _P, _L, _I, _P],
     "lgs_moe_sort": [_P, _I, _I, _I, _P, _P, _P, _P, _P],
@@ -64,9 +64,12 @@ SIGNATURES = {
     "lgs_layernorm": [_P, _P, _P, _F, _F, _I, _P, _P, _I, _I, _P],
     "lgs_softcap": [_P, _L, _F, _P],
     "lgs_normattn_prepare": [_P, _L, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _I, _I, _P, _P, _P,
-                             _I, _P],
+                             _I, _I, _P, _P, _P, _I, _I, _P],
+    "lgs_pool_blocks": [_P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "lgs_sinkattn": [_P, _L, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P,
-                     _L, _P],
+                     _L, _I, _I, _P, _P, _I, _I, _P, _I, _P],
+    "lgs_channel_scan": [_P, _P, _L, _P, _L, _I, _P, _L, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P, _P, _I,
+                         _P],
     "lgs_delta_prepare": [_P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _F, _P, _I, _I, _I, _I, _F,
                           _P],
     "lgs_delta_step_prepare": [_P, _L, _P, _I, _I, _P, _P, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I,
@@ -144,8 +147,8 @@ F32, I32 = torch.float32, torch.int32
 def linear(a: torch.Tensor, w: torch.Tensor, *, M: int, N: int, K: int, y: torch.Tensor, a_off: int = 0, lda: int,
            y_off: int = 0, ldy: int, batch: int = 1, stride_a: int = 0, stride_w: int = 0, stride_y: int = 0,
            accumulate: bool = False, act: int = ACT_NONE, a_rows: Optional[torch.Tensor] = None,
-           z_start: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """y[z] (+)= act(a[z] w[z]^T) over ``batch`` strided operands; offsets and strides count elements. With
+           z_start: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """y[z] (+)= act(a[z] w[z]^T + bias) over ``batch`` strided operands; offsets and strides count elements. With
     ``z_start`` (batch + 1 int32 row bounds) batch z owns that range of a row list of at most M rows, whose A rows
     are ``a_rows`` (or the list places themselves) and whose Y rows are the list places. ``a`` may be a producer's
     bf16 copy (``rmsnorm(bf16_copy=True)``, ``glu(bf16=True)``) for the MFMA tiles with bf16 weights."""
@@ -157,17 +160,22 @@ def linear(a: torch.Tensor, w: torch.Tensor, *, M: int, N: int, K: int, y: torch
     need_y = y_off + (batch - 1) * stride_y * (0 if z_start is not None else 1) + (M - 1) * ldy + N
     if a.numel() < need_a or y.numel() < need_y or w.numel() < (batch - 1) * stride_w + N * K:
         raise ValueError("linear: an operand is smaller than the sizes and strides say")
+    if bias is not None and bias.numel() != N:
+        raise ValueError("linear: one bias per output column")
     _check(load_library().lgs_linear(ap, lda, stride_a, _dev(w, "w"), _wf32(w, "w"), stride_w, yp, ldy, stride_y,
                                      M, N, K, batch, int(accumulate), act, _opt(a_rows, "a_rows", I32),
-                                     _opt(z_start, "z_start", I32), int(a16), int(y16), _stream()))
+                                     _opt(z_start, "z_start", I32), int(a16), int(y16), _opt(bias, "bias", F32),
+                                     _stream()))
     return y
 
 
-def embed(tokens: torch.Tensor, table: torch.Tensor, scale: float) -> torch.Tensor:
+def embed(tokens: torch.Tensor, table: torch.Tensor, scale: float, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     T, (V, W) = tokens.numel(), table.shape
-    x = torch.empty(T, W, dtype=F32, device=tokens.device)
+    x = out if out is not None else torch.empty(T, W, dtype=F32, device=tokens.device)
+    if x.shape != (T, W):
+        raise ValueError("embed: the result is (tokens, width)")
     _check(load_library().lgs_embed(_dev(tokens, "tokens", I32), _dev(table, "table"), _wf32(table, "table"),
-                                    float(scale), x.data_ptr(), T, W, V, _stream()))
+                                    float(scale), _dev(x, "x", F32), T, W, V, _stream()))
     return x
 
 
@@ -252,16 +260,33 @@ def head_gate(o: torch.Tensor, proj: torch.Tensor, g_off: int, *, H: int, dv: in
     return o16 if bf16_copy else o
 
 
-def latent_prepare(proj: torch.Tensor, q_off: int, kv_off: int, cache_c: torch.Tensor, cache_kr: torch.Tensor,
-                   norm_w: torch.Tensor, inv_freq: Optional[torch.Tensor], slot: torch.Tensor, pos: torch.Tensor, *,
-                   H: int, d: int, dr: int, r: int, rot_dims: int, eps: float) -> None:
+def norm_columns(proj: torch.Tensor, off: int, weight: torch.Tensor, *, eps: float, bf16: bool = False) -> torch.Tensor:
+    """RMS norm (plain weight, n values) of the n columns of ``proj`` at ``off``: (T, n) fp32, or with ``bf16`` its
+    rounding only where the caller's product reads that (the fp32 result is made as well)."""
+    T, ld = proj.shape
+    n = weight.numel()
+    if off + n > ld:
+        raise ValueError("norm_columns: columns outside the row")
+    y = torch.empty(T, n, dtype=F32, device=proj.device)
+    y16 = torch.empty(T, n, dtype=torch.bfloat16, device=proj.device) if bf16 else None
+    _check(load_library().lgs_rmsnorm(_dev(proj, "proj", F32) + 4 * off, ld, _dev(weight, "weight", F32), 0.0, float(eps),
+                                      y.data_ptr(), n, T, 1, n, _opt(y16, "y_bf16", torch.bfloat16), _stream()))
+    return y16 if bf16 else y
+
+
+def latent_prepare(q: torch.Tensor, q_off: int, proj: torch.Tensor, kv_off: int, cache_c: torch.Tensor,
+                   cache_kr: torch.Tensor, norm_w: torch.Tensor, inv_freq: Optional[torch.Tensor], slot: torch.Tensor,
+                   pos: torch.Tensor, *, H: int, d: int, dr: int, r: int, rot_dims: int, eps: float) -> None:
+    """The queries are the H (d + dr) columns of ``q`` at ``q_off`` (rotated parts turned in place); the latent and the
+    shared key part the r + dr columns of ``proj`` at ``kv_off`` (``q`` may be ``proj`` itself)."""
     T, ld = proj.shape
     slots, S = cache_c.shape[:2]
     if tuple(cache_c.shape) != (slots, S, r) or tuple(cache_kr.shape) != (slots, S, dr) or norm_w.numel() != r:
         raise ValueError("latent_prepare: cache shapes")
-    if q_off + H * (d + dr) > ld or kv_off + r + dr > ld or slot.numel() != T or pos.numel() != T:
+    if q.shape[0] != T or q_off + H * (d + dr) > q.shape[1] or kv_off + r + dr > ld or slot.numel() != T or pos.numel() != T:
         raise ValueError("latent_prepare: projections outside the row")
-    _check(load_library().lgs_latent_prepare(_dev(proj, "proj", F32), ld, q_off, kv_off, _dev(cache_c, "cache_c"),
+    _check(load_library().lgs_latent_prepare(_dev(q, "q", F32) + 4 * q_off, q.shape[1], _dev(proj, "proj", F32) + 4 * kv_off,
+                                             ld, _dev(cache_c, "cache_c"),
                                              _wf32(cache_c, "cache_c"), _dev(cache_kr, "cache_kr", F32),
                                              _dev(norm_w, "norm_w", F32), _opt(inv_freq, "inv_freq", F32),
                                              _dev(slot, "slot", I32), _dev(pos, "pos", I32), T, H, d, dr, r, rot_dims,
@@ -270,9 +295,9 @@ def latent_prepare(proj: torch.Tensor, q_off: int, kv_off: int, cache_c: torch.T
 
 def latent_attention(qc: torch.Tensor, proj: torch.Tensor, q_off: int, cache_c: torch.Tensor, cache_kr: torch.Tensor,
                      sink: Optional[torch.Tensor], slot: torch.Tensor, pos: torch.Tensor, *, H: int, d: int, dr: int,
-                     r: int, scale: float, splits: Optional[int] = None) -> torch.Tensor:
-    """Softmax attention of every (token, head) over its sequence's cached rows up to the token's position, in the
-    latent space. ``splits``: workgroups per (token, head); by default enough of them to fill the chip when the
+                     r: int, scale: float, splits: Optional[int] = None, window: int = 0) -> torch.Tensor:
+    """Softmax attention of every (token, head) over its sequence's cached rows up to the token's position (``window``
+    > 0: the last ``window`` of them), in the latent space; the rotated query parts are read from ``proj`` at ``q_off``. ``splits``: workgroups per (token, head); by default enough of them to fill the chip when the
     step has few rows (decode), one when it has many (a prompt)."""
     T, ld = proj.shape
     S = cache_c.shape[1]
@@ -281,19 +306,22 @@ def latent_attention(qc: torch.Tensor, proj: torch.Tensor, q_off: int, cache_c: 
     out = torch.empty(T, H * r, dtype=F32, device=proj.device)
     if splits is None:
         splits = max(1, min(32, 1024 // (T * H)))
+        if window > 0:  # at least one key per wave of a split
+            splits = max(1, min(splits, window // 4))
     part = torch.empty(T * H * splits * (r + 2), dtype=F32, device=proj.device) if splits > 1 else None
     _check(load_library().lgs_latent_attention(_dev(qc, "qc", F32), _dev(proj, "proj", F32), ld, q_off,
                                                _dev(cache_c, "cache_c"), _wf32(cache_c, "cache_c"),
                                                _dev(cache_kr, "cache_kr", F32), _opt(sink, "sink", F32),
                                                _dev(slot, "slot", I32), _dev(pos, "pos", I32), out.data_ptr(), T, H,
-                                               d, dr, r, S, float(scale), splits, _opt(part, "part", F32), _stream()))
+                                               d, dr, r, S, float(scale), splits, _opt(part, "part", F32), int(window),
+                                               _stream()))
     return out
 
 
 def latent_attention_tiles(qc: torch.Tensor, proj: torch.Tensor, q_off: int, cache_c: torch.Tensor,
                            cache_kr: torch.Tensor, sink: Optional[torch.Tensor], seq_start: torch.Tensor,
                            seq_slot: torch.Tensor, seq_pos0: torch.Tensor, max_len: int, *, H: int, d: int, dr: int,
-                           r: int, scale: float) -> torch.Tensor:
+                           r: int, scale: float, window: int = 0) -> torch.Tensor:
     """The prompt form of ``latent_attention``: tiles of 16 consecutive tokens of a sequence against key tiles of 16
     cached rows on fp32 MFMA. ``max_len``: the most tokens any sequence brings to this step. r % 64 == 0."""
     T, ld = proj.shape
@@ -306,7 +334,7 @@ def latent_attention_tiles(qc: torch.Tensor, proj: torch.Tensor, q_off: int, cac
         _dev(qc, "qc", F32), _dev(proj, "proj", F32), ld, q_off, _dev(cache_c, "cache_c"), _wf32(cache_c, "cache_c"),
         _dev(cache_kr, "cache_kr", F32), _opt(sink, "sink", F32), _dev(seq_start, "seq_start", I32),
         _dev(seq_slot, "seq_slot", I32), _dev(seq_pos0, "seq_pos0", I32), out.data_ptr(), B, int(max_len), H, d, dr, r,
-        S, float(scale), _stream()))
+        S, float(scale), int(window), _stream()))
     return out
 
 
@@ -363,11 +391,16 @@ def act_rows(proj: torch.Tensor, off: int, n: int, act: int, gate_off: int = -1,
 
 
 def sandwich_step(x: torch.Tensor, *, branches=(), coef: float = 1.0, post_w: Optional[torch.Tensor] = None,
-                  next_w: Optional[torch.Tensor] = None, eps: float, want_f32: bool = True, bf16_copy: bool = False):
-    """One boundary between sublayers that are normed on the way in and out, in place on the residual x (T, W).
+                  next_w: Optional[torch.Tensor] = None, eps: float, want_f32: bool = True, bf16_copy: bool = False,
+                  x_in: Optional[torch.Tensor] = None, hist: Optional[torch.Tensor] = None,
+                  depth_w: Optional[torch.Tensor] = None):
+    """One boundary between sublayers of one residual, in place on x (T, W); the residual so far is read from ``x_in``
+    when that is given.
     ``branches``: up to two (y, w) pairs of the sublayer that ran, each y (T, W) RMS-normed with weight w (w None: taken
     as it is); their sum times ``coef`` is RMS-normed with ``post_w`` (the output norm's weight times the layer's
-    per-channel scale) and added to x. With ``next_w`` the next sublayer's input rmsnorm(x) * next_w is returned as
+    per-channel scale; None: no output norm) and added to x. With ``depth_w`` (n + 1 weights; a layer's end): x is kept
+    in row block n of ``hist`` (rows, T, W), if it has that many, and becomes depth_w[n] x + sum_{j < n} depth_w[j]
+    hist[j]. With ``next_w`` the next sublayer's input rmsnorm(x) * next_w is returned as
     (h fp32 or None, h bf16 or None)."""
     T, W = x.shape
     ys = [(None, None), (None, None)]
@@ -375,14 +408,20 @@ def sandwich_step(x: torch.Tensor, *, branches=(), coef: float = 1.0, post_w: Op
         if i > 1 or y.shape != (T, W) or (w is not None and w.numel() != W):
             raise ValueError("sandwich_step: at most two branches of the residual's shape")
         ys[i] = (y, w)
-    if (ys[0][0] is not None and (post_w is None or post_w.numel() != W)) or (next_w is not None and next_w.numel() != W):
-        raise ValueError("sandwich_step: norm weights")
+    if any(w is not None and w.numel() != W for w in (post_w, next_w)) or (x_in is not None and x_in.shape != (T, W)):
+        raise ValueError("sandwich_step: norm weights of one value per channel, x_in of the residual's shape")
+    n_prev, hist_rows = 0, 0
+    if depth_w is not None:
+        n_prev, hist_rows = depth_w.numel() - 1, 0 if hist is None else hist.shape[0]
+        if hist is None or tuple(hist.shape[1:]) != (T, W) or not 1 <= n_prev <= hist_rows:
+            raise ValueError("sandwich_step: the earlier layers' results, (rows, T, W), at least one per earlier weight")
     h = torch.empty(T, W, dtype=F32, device=x.device) if next_w is not None and (want_f32 or not bf16_copy) else None
     h16 = torch.empty(T, W, dtype=torch.bfloat16, device=x.device) if next_w is not None and bf16_copy else None
-    _check(load_library().lgs_sandwich_step(_dev(x, "x", F32), _opt(ys[0][0], "y0", F32), _opt(ys[0][1], "w0", F32),
+    _check(load_library().lgs_sandwich_step(_opt(x_in, "x_in", F32), _dev(x, "x", F32), _opt(ys[0][0], "y0", F32), _opt(ys[0][1], "w0", F32),
                                             _opt(ys[1][0], "y1", F32), _opt(ys[1][1], "w1", F32), float(coef),
                                             _opt(post_w, "post_w", F32), _opt(next_w, "next_w", F32),
                                             _opt(h, "h", F32), _opt(h16, "h_bf16", torch.bfloat16), float(eps), T, W,
+                                            _opt(hist, "hist", F32), _opt(depth_w, "depth_w", F32), n_prev, hist_rows,
                                             _stream()))
     return h, h16
 
@@ -611,6 +650,46 @@ def ssm_scan(xbc: torch.Tensor, proj: torch.Tensor, dt_off: int, dt_bias: torch.
     return y
 
 
+def channel_scan(x: torch.Tensor, proj: torch.Tensor, z_off: int, bc: torch.Tensor, rank: int, a2: torch.Tensor,
+                 D: torch.Tensor, state: torch.Tensor, seq_start: torch.Tensor, seq_slot: torch.Tensor,
+                 seq_pos0: torch.Tensor, *, dt: Optional[torch.Tensor] = None, w_dt: Optional[torch.Tensor] = None,
+                 dt_bias: Optional[torch.Tensor] = None, max_len: int = 0, chunked: Optional[bool] = None,
+                 bf16: bool = False) -> torch.Tensor:
+    """The selective scan with a diagonal state matrix per channel over a packed batch: x (T, inner) after the
+    convolution, the gate's z in the columns of ``proj`` at ``z_off``, bc (T, rank + 2 N) = step-size inner values | B | C,
+    a2 (N, inner) = A log2(e), state (slots, 1, N, inner) fp32. Step sizes: softplus of ``dt`` (T, inner), or of
+    w_dt bc[:, :rank] + dt_bias made inside the launch (steps of few tokens). Returns (y + D x) silu(z) (T, inner), fp32 or
+    (``bf16``) rounded to bf16. ``chunked`` picks the prompt form (64-token chunks side by side; needs ``dt``) over the
+    token-by-token walk; by default steps in which a sequence brings more than 64 tokens take it."""
+    T, inner = x.shape
+    N = a2.shape[0]
+    B = seq_slot.numel()
+    if a2.shape != (N, inner) or bc.shape != (T, rank + 2 * N) or tuple(state.shape[1:]) != (1, N, inner) or \
+            D.numel() != inner or proj.shape[0] != T or z_off + inner > proj.shape[1] or seq_start.numel() != B + 1:
+        raise ValueError("channel_scan: shapes")
+    if (dt is None) == (w_dt is None) or (dt is not None and dt.shape != (T, inner)) or \
+            (w_dt is not None and (tuple(w_dt.shape) != (inner, rank) or dt_bias is None or dt_bias.numel() != inner)):
+        raise ValueError("channel_scan: step sizes, or their map (inner, rank) and bias")
+    if chunked is None:
+        chunked = dt is not None and max_len > 64
+    ws = wsum = None
+    max_chunks = 0
+    if chunked:
+        if dt is None or not 0 < max_len <= T:
+            raise ValueError("channel_scan: the prompt form needs the step sizes and the longest sequence's token count")
+        max_chunks = (max_len + 63) // 64
+        ws = torch.empty(B * max_chunks * N * inner, dtype=F32, device=x.device)
+        wsum = torch.empty(B * max_chunks * inner, dtype=F32, device=x.device)
+    out = torch.empty(T, inner, dtype=torch.bfloat16 if bf16 else F32, device=x.device)
+    _check(load_library().lgs_channel_scan(
+        _dev(x, "x", F32), _dev(proj, "proj", F32) + 4 * z_off, proj.shape[1], _dev(bc, "bc", F32), rank + 2 * N, rank,
+        _opt(dt, "dt", F32), inner, _opt(w_dt, "w_dt"), 0 if w_dt is None else _wf32(w_dt, "w_dt"),
+        _opt(dt_bias, "dt_bias", F32), _dev(a2, "a2", F32), _dev(D, "D", F32), _dev(state, "state", F32),
+        _dev(seq_start, "seq_start", I32), _dev(seq_slot, "seq_slot", I32), _dev(seq_pos0, "seq_pos0", I32),
+        out.data_ptr(), int(bf16), B, inner, N, _opt(ws, "ws", F32), _opt(wsum, "wsum", F32), max_chunks, _stream()))
+    return out
+
+
 def gated_group_norm(y: torch.Tensor, proj: torch.Tensor, z_off: int, weight: torch.Tensor, *, groups: int,
                      eps: float, bf16_copy: bool = False) -> torch.Tensor:
     """unit_rms_per_group(y * silu(z)) * weight with z the columns of ``proj`` at ``z_off``; (T, inner) fp32 or, with
@@ -678,13 +757,17 @@ def softcap(z: torch.Tensor, cap: float) -> torch.Tensor:
 
 def normattn_prepare(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, cache_k: torch.Tensor,
                      cache_v: torch.Tensor, slot: torch.Tensor, pos: torch.Tensor, *, H: int, G: int, d: int, dv: int,
-                     eps: float, temp_coef: float = 0.0, temp_every: int = 0, norm: bool = True,
+                     eps: float, temp_coef: float = 0.0, temp_every: int = 0, norm: int = 1,
                      q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None,
-                     inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0) -> None:
-    """Queries normed (``norm``: divided by their root mean square, times ``q_weight`` (d,) if given), rotated on the
-    pairs (i, i + rot_dims / 2) and multiplied by the position's query temperature, in place in ``proj``; keys normed
+                     inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0, interleaved: bool = False,
+                     v_freq: Optional[torch.Tensor] = None, pooled=None, pool: int = 0) -> None:
+    """Queries normed (``norm`` 1: each head divided by its root mean square, times ``q_weight`` (d,) if given; 2: all
+    heads by one root mean square, ``q_weight`` (H d,); 0: not), rotated on the pairs (i, i + rot_dims / 2) - or
+    ``interleaved`` (2i, 2i + 1) - and multiplied by the position's query temperature, in place in ``proj``; keys normed
     (``k_weight``) and rotated alike, and the values, into the cache rows (slot, position). cache_k (slots, S, G, d),
-    cache_v (slots, S, G, dv). ``v_off == k_off`` (with dv == d): the values are the keys as projected."""
+    cache_v (slots, S, G, dv). ``v_off == k_off`` (with dv == d): the values are the keys as projected. ``v_freq``
+    (dv / 2,): the values are rotated by their position. ``pooled`` = (pool_k, pool_v) (slots, blocks, G, d / dv) fp32
+    with ``pool``: steps of one token per sequence leave the means of a block of ``pool`` positions when they complete it."""
     T, ld = proj.shape
     slots, S = cache_k.shape[:2]
     if tuple(cache_k.shape) != (slots, S, G, d) or tuple(cache_v.shape) != (slots, S, G, dv) or \
@@ -692,41 +775,80 @@ def normattn_prepare(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, cac
         raise ValueError("normattn_prepare: cache shapes")
     if slot.numel() != T or pos.numel() != T:
         raise ValueError("normattn_prepare: one slot and position per row")
-    if any(w is not None and w.numel() != d for w in (q_weight, k_weight)) or rot_dims % 2 or rot_dims > d or \
+    nq, nk = (H * d, G * d) if norm == 2 else (d, d)
+    if (q_weight is not None and q_weight.numel() != nq) or (k_weight is not None and k_weight.numel() != nk) or \
+            (v_freq is not None and 2 * v_freq.numel() != dv) or rot_dims % 2 or rot_dims > d or \
             (rot_dims > 0 and (inv_freq is None or inv_freq.numel() < rot_dims // 2)):
-        raise ValueError("normattn_prepare: norm weights of d values, rotary frequencies for rot_dims / 2 pairs")
+        raise ValueError("normattn_prepare: norm weights, rotary frequencies for rot_dims / 2 (values: dv / 2) pairs")
+    pk, pv = _pooled(pooled, pool, slots, G, d, dv)
     _check(load_library().lgs_normattn_prepare(_dev(proj, "proj", F32), ld, q_off, k_off, v_off,
                                                _dev(cache_k, "cache_k"), _dev(cache_v, "cache_v"),
                                                _wf32(cache_k, "cache_k"), _dev(slot, "slot", I32),
                                                _dev(pos, "pos", I32), T, H, G, d, dv, S, float(eps), float(temp_coef),
                                                int(temp_every), int(norm), _opt(q_weight, "q_weight", F32),
                                                _opt(k_weight, "k_weight", F32), _opt(inv_freq, "inv_freq", F32),
-                                               int(rot_dims), _stream()))
+                                               int(rot_dims), int(interleaved), _opt(v_freq, "v_freq", F32),
+                                               _opt(pk, "pool_k", F32), _opt(pv, "pool_v", F32),
+                                               int(pool) if pk is not None else 0, pk.shape[1] if pk is not None else 0,
+                                               _stream()))
+
+
+def _pooled(pooled, pool: int, slots: int, G: int, d: int, dv: int):
+    """The checked buffers of the pooled blocks, (None, None) without."""
+    if pooled is None or pool <= 0:
+        return None, None
+    pk, pv = pooled
+    rows = pk.shape[1]
+    if tuple(pk.shape) != (slots, rows, G, d) or tuple(pv.shape) != (slots, rows, G, dv) or rows < 1:
+        raise ValueError("pooled blocks: (slots, blocks, key heads, size) of keys and values")
+    return pk, pv
+
+
+def pool_blocks(cache_k: torch.Tensor, cache_v: torch.Tensor, pooled, pool: int, seq_start: torch.Tensor,
+                seq_slot: torch.Tensor, seq_pos0: torch.Tensor, max_len: int) -> None:
+    """The means of the cached keys and values of every block of ``pool`` positions that the step completes."""
+    slots, S, G, d = cache_k.shape
+    dv = cache_v.shape[3]
+    pk, pv = _pooled(pooled, pool, slots, G, d, dv)
+    B = seq_slot.numel()
+    if pk is None or tuple(cache_v.shape[:3]) != (slots, S, G) or seq_start.numel() != B + 1 or seq_pos0.numel() != B:
+        raise ValueError("pool_blocks: shapes")
+    _check(load_library().lgs_pool_blocks(_dev(cache_k, "cache_k"), _dev(cache_v, "cache_v"), _wf32(cache_k, "cache_k"),
+                                          _dev(pk, "pool_k", F32), _dev(pv, "pool_v", F32), _dev(seq_start, "seq_start", I32),
+                                          _dev(seq_slot, "seq_slot", I32), _dev(seq_pos0, "seq_pos0", I32), B, int(max_len),
+                                          G, d, dv, S, int(pool), pk.shape[1], _stream()))
 
 
 def sinkattn(proj: torch.Tensor, q_off: int, cache_k: torch.Tensor, cache_v: torch.Tensor,
              sink: Optional[torch.Tensor], seq_start: torch.Tensor, seq_slot: torch.Tensor, seq_pos0: torch.Tensor,
              max_len: int, *, H: int, G: int, d: int, dv: int, scale: float, chunk: int = 0, cap: float = 0.0,
              post: float = 1.0, bf16_copy: bool = False, splits: Optional[int] = None,
-             gate_off: int = -1) -> torch.Tensor:
+             gate_off: int = -1, gate_cols: int = 1, window: int = 0, pooled=None, pool: int = 0,
+             v_freq: Optional[torch.Tensor] = None, interleaved: bool = False) -> torch.Tensor:
     """Causal softmax attention of every row of a packed batch over its sequence's cached keys and values, grouped
     key / value heads, with exp(sink[h]) in the normaliser; the prepared queries are the H d columns of ``proj`` at
-    ``q_off``. ``gate_off`` >= 0: head h's output is multiplied by sigmoid(proj[:, gate_off + h]). Returns (T, H dv)
-    fp32 times ``post``, or with ``bf16_copy`` its rounding to bf16."""
+    ``q_off``. ``gate_off`` >= 0: head h's output is multiplied by sigmoid(proj[:, gate_off + h]), with ``gate_cols`` = dv
+    column by column by sigmoid(proj[:, gate_off + h dv + c]). ``window``: a position sees its own and the window - 1 keys
+    before it and, with ``pooled`` = (pool_k, pool_v), the means of the blocks of ``pool`` positions that lie wholly
+    before those. ``v_freq``: outputs are turned back by the query's position (the values were cached rotated). Returns
+    (T, H dv) fp32 times ``post``, or with ``bf16_copy`` its rounding to bf16."""
     T, ld = proj.shape
     B = seq_slot.numel()
     slots, S = cache_k.shape[:2]
     if tuple(cache_k.shape) != (slots, S, G, d) or tuple(cache_v.shape) != (slots, S, G, dv):
         raise ValueError("sinkattn: cache shapes")
     if seq_start.numel() != B + 1 or q_off + H * d > ld or not 1 <= max_len <= T or \
-            (sink is not None and sink.numel() != H) or gate_off + H > ld:
-        raise ValueError("sinkattn: step table / query columns / sink / head gates")
+            (sink is not None and sink.numel() != H) or gate_off + H * gate_cols > ld or gate_cols not in (1, dv) or \
+            (v_freq is not None and 2 * v_freq.numel() != dv):
+        raise ValueError("sinkattn: step table / query columns / sink / gates / value frequencies")
+    pk, pv = _pooled(pooled, pool, slots, G, d, dv)
+    prow = pk.shape[1] if pk is not None else 0
     out = torch.empty(T, H * dv, dtype=F32, device=proj.device)
     out16 = torch.empty(T, H * dv, dtype=torch.bfloat16, device=proj.device) if bf16_copy else None
     if max_len > 1:
         splits = 1
     elif splits is None:
-        span = min(S, chunk) if chunk > 0 else S
+        span = min(S, chunk) if chunk > 0 else (min(S, window) + prow if window > 0 else S)
         splits = max(1, min(64, 512 // max(1, B * H), (span + 127) // 128))
     part = torch.empty(T * H * splits * (2 + dv), dtype=F32, device=proj.device) if splits > 1 else None
     _check(load_library().lgs_sinkattn(_dev(proj, "proj", F32) + 4 * q_off, ld, _dev(cache_k, "cache_k"),
@@ -736,7 +858,9 @@ def sinkattn(proj: torch.Tensor, q_off: int, cache_k: torch.Tensor, cache_v: tor
                                        _opt(out16, "out_bf16", torch.bfloat16), _opt(part, "part", F32), splits, B,
                                        int(max_len), H, G, d, dv, S, int(chunk), float(scale), float(cap), float(post),
                                        _dev(proj, "proj", F32) + 4 * gate_off if gate_off >= 0 else None, ld,
-                                       _stream()))
+                                       int(gate_cols), int(window), _opt(pk, "pool_k", F32), _opt(pv, "pool_v", F32),
+                                       int(pool) if pk is not None else 0, prow, _opt(v_freq, "v_freq", F32),
+                                       int(interleaved), _stream()))
     return out16 if bf16_copy else out
 
 
