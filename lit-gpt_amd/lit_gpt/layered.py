@@ -522,10 +522,10 @@ class LayeredGPT(nn.Module):
                     out[p + "mix.q"] = (nq, W)
                 out.update({p + "mix.dkv": (m.kv_rank + m.rot_dim, W),
                             p + "mix.dkv.norm": (m.kv_rank,), p + "mix.uk": (m.heads * m.dim, m.kv_rank),
-                            p + "mix.uv": (m.heads * m.vdim, m.kv_rank),
-                            p + "mix.g": (m.heads * m.vdim, W), p + "mix.o": (W, m.heads * m.vdim)})
+                            p + "mix.uv": (m.heads * m.vdim, m.kv_rank)})
                 if m.sink_kind == "learned":
                     out[p + "mix.sink"] = (m.heads,)
+                out.update({p + "mix.g": (m.heads * m.vdim, W), p + "mix.o": (W, m.heads * m.vdim)})
             f = spec.mlp
             if f is not None and f.kind == "dense" and config.design.dense_ff == "relu2":
                 out.update({p + "mlp.up": (f.ff, W), p + "mlp.down": (W, f.ff)})

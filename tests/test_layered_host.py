@@ -146,7 +146,7 @@ def test_library_exports_every_header_symbol():
         subprocess.run(["make", "-C", str(REPO / "lit-gpt_amd" / "csrc"), "-j8", "seq"], check=True)
     lib = seq_ops.load_library()
     assert lib.lgs_version() >= 1
-    rc = lib.lgs_linear(None, 1, 0, None, 0, 0, None, 1, 0, 1, 1, 1, 1, 0, 0, None, None, 0, 0, None)
+    rc = lib.lgs_linear(None, 1, 0, None, 0, 0, None, 1, 0, 1, 1, 1, 1, 0, 0, None, None, 0, 0, None, None)
     assert rc != 0 and b"null" in lib.lgs_last_error_string()
     with pytest.raises(RuntimeError, match="GPU tensor"):
         seq_ops.rmsnorm(torch.zeros(2, 8), torch.ones(8), offset=0.0, eps=1e-5)
@@ -487,3 +487,147 @@ def test_gatutar_plain_implementation():
     fs["shared.sg"] = torch.tensor([[50.0, 0.0]], dtype=D)
     opened = orc.feed_forward(h, {"kind": "moe", "router": {"experts": 2, "top": 1}, "shared": {"ff": 2}}, fs)
     assert torch.allclose(opened, out + h)
+
+
+# ------------------------------------------------------------------------------------------------ the Zaronex design
+def _zar_cfg():
+    return {
+        "architecture": "Zaronex", "vocab": 23, "width": 16, "norm": {"eps": 1e-5},
+        "layers": [
+            {"type": "latent_attention", "mlp": {"kind": "dense", "ff": 10},
+             "mixer": {"heads": 2, "dim": 3, "rot_dim": 4, "vdim": 5, "kv_rank": 6, "q_rank": 7, "scale": 0.4,
+                       "rot": {"dims": 4, "base": 100.0}, "mask": {"size": 5}}},
+            {"type": "parallel", "mlp": None,
+             "mixer": {"left": {"heads": 6, "kv_heads": 3, "dim": 4, "vdim": 2, "scale": 0.5, "mask": {"size": 3, "pool": 2},
+                                "rot": {"dims": 2, "base": 100.0}},
+                       "right": {"heads": 2, "dim": 3, "vdim": 5, "tau": 3.0}}},
+            {"type": "parallel_2", "mlp": {"kind": "dense", "ff": 9},
+             "mixer": {"left": {"heads": 4, "kv_heads": 2, "dim": 6, "vdim": 4, "scale": 0.3, "mask": {"size": 4},
+                                "rot": {"dims": 4, "base": 50.0, "scaling": {"factor": 2.0}}},
+                       "right": {"inner": 10, "state": 3, "dt_rank": 2, "conv": 4}}},
+        ],
+    }
+
+
+def test_zaronex_config_and_tensor_names():
+    from lit_gpt.config import LayeredConfig, model_class
+    from lit_gpt.layered import LayeredGPT
+
+    c = LayeredConfig.from_dict(_zar_cfg())
+    assert model_class(c) is LayeredGPT
+    d = c.design
+    assert (d.block, d.norm, d.dense_ff, d.tied_head, d.norm_offset, d.mask, d.depth_average) == \
+        ("prenorm", "rms", "gelu_tanh", False, 0.0, "window", True)
+    a, b, e = (l.mixer for l in c.layers)
+    assert (a.kind, a.q_rank, a.kv_rank, a.rot_dim, a.window, a.mask_size, a.sink_kind) == ("latent_attention", 7, 6, 4, 5, 0, "none")
+    assert (b.kind, b.branch_norm, b.left_scale, b.right_scale) == ("parallel", True, 0.5, 0.5)
+    assert (b.left.kind, b.left.window, b.left.pool, b.left.bias, b.left.out_gate, b.left.sink_kind, b.left.qk_norm,
+            b.left.rot_layout, b.left.rot_values) == ("pooled_attention", 3, 2, True, True, "learned", "none", "half", False)
+    assert (b.right.kind, b.right.tau) == ("gated_linear", 3.0)
+    assert (e.left.kind, e.left.window, e.left.pool, e.left.bias, e.left.out_gate, e.left.sink_kind, e.left.qk_norm,
+            e.left.rot_layout, e.left.rot_values) == \
+        ("rotated_value_attention", 4, 0, False, False, "none", "joint", "interleaved", True)
+    assert e.left.rot.inv_freq() == pytest.approx([0.5, 50.0 ** -0.5 / 2.0])
+    assert (e.right.kind, e.right.inner, e.right.state, e.right.dt_rank, e.right.conv) == ("mamba", 10, 3, 2, 4)
+    assert c.layers[1].mlp is None and c.layers[2].mlp.ff == 9
+    s = LayeredGPT.tensor_shapes(c)
+    assert [s[f"l{i}.dwa"] for i in range(3)] == [(2,), (3,), (4,)]
+    assert s["head"] == (23, 16) and s["final.norm"] == (16,) and "l1.norm2" not in s and s["l2.norm2"] == (16,)
+    assert s["l0.mix.dq"] == (7, 16) and s["l0.mix.dq.norm"] == (7,) and s["l0.mix.uq"] == (14, 7) and "l0.mix.q" not in s
+    assert s["l0.mix.dkv"] == (10, 16) and s["l0.mix.uk"] == (6, 6) and s["l0.mix.uv"] == (10, 6) and "l0.mix.sink" not in s
+    assert s["l0.mix.g"] == (10, 16) and s["l0.mix.o"] == (16, 10)
+    assert s["l1.mix.left.q.b"] == (24,) and s["l1.mix.left.k.b"] == (12,) and s["l1.mix.left.v.b"] == (6,)
+    assert s["l1.mix.left.sink"] == (6,) and s["l1.mix.left.g"] == (12, 16) and s["l1.mix.left.o"] == (16, 12)
+    assert s["l1.mix.right.a2.b"] == (6,) and s["l1.mix.right.out"] == (16,) and s["l1.mix.left.out"] == (16,)
+    assert s["l2.mix.left.q.norm"] == (24,) and s["l2.mix.left.k.norm"] == (12,) and "l2.mix.left.g" not in s
+    assert s["l2.mix.right.in"] == (20, 16) and s["l2.mix.right.conv"] == (10, 4) and s["l2.mix.right.x"] == (8, 10)
+    assert s["l2.mix.right.dt"] == (10, 2) and s["l2.mix.right.A_log"] == (10, 3) and s["l2.mix.right.o"] == (16, 10)
+    w = LayeredGPT.random_weights(c)
+    assert set(w) == set(s) and all(tuple(w[k].shape) == s[k] for k in s)
+    # a mask's size keeps its older meaning in the designs with aligned chunks
+    assert LayeredConfig._mixer_spec("attention", {"heads": 1, "dim": 2, "vdim": 2, "mask": {"size": 9}}).mask_size == 9
+
+
+@pytest.mark.parametrize("edit", [
+    lambda c: c["layers"][0]["mixer"].update(kv_rank=2000),
+    lambda c: c["layers"][0]["mixer"]["rot"].update(dims=6),  # more rotary dims than the rotated part has
+    lambda c: c["layers"][1]["mixer"]["left"].update(kv_heads=4),  # heads no multiple of the key heads
+    lambda c: c["layers"][1]["mixer"]["left"].update(mask={"pool": 4}),  # pooled blocks need a window
+    lambda c: c["layers"][1]["mixer"]["left"]["rot"].update(dims=3),
+    lambda c: c["layers"][1]["mixer"]["right"].update(tau=0.0),
+    lambda c: c["layers"][2]["mixer"]["left"].update(vdim=3),  # rotated values have an even size
+    lambda c: c["layers"][2]["mixer"]["right"].update(state=300),
+    lambda c: c["layers"][2]["mixer"]["right"].update(conv=20),
+    lambda c: c.update(loop={"start": 0, "stop": 2, "times": 2}),  # one weight vector per layer, not per pass
+])
+def test_zaronex_config_rejects_what_does_not_fit(edit):
+    from lit_gpt.config import LayeredConfig
+
+    c = _zar_cfg()
+    edit(c)
+    with pytest.raises(ValueError):
+        LayeredConfig.from_dict(c)
+
+
+def test_input_projection_gathers_biases():
+    from lit_gpt.layered import _fuse_rows
+    from lit_gpt.mixers import InputReader
+
+    class Part(InputReader):
+        def __init__(self, parts, bias):
+            super().__init__()
+            self.parts, self.bias = parts, bias
+
+        def in_parts(self):
+            return self.parts
+
+        def in_bias(self):
+            return self.bias
+
+    a = Part([("q", torch.ones(3, 4)), ("k", 2 * torch.ones(8, 4))], {"k": torch.arange(8.0)})
+    b = Part([("g", 3 * torch.ones(2, 4))], {})
+    w, bias = _fuse_rows([a, b], 4, torch.device("cpu"), torch.float32)
+    assert a.off == {"q": 0, "k": 8} and b.off == {"g": 16} and w.shape == (24, 4) and bias.shape == (24,)
+    assert torch.equal(bias[8:16], torch.arange(8.0)) and bias[:8].abs().sum() == 0 and bias[16:].abs().sum() == 0
+    assert w[3:8].abs().sum() == 0 and (w[16:18] == 3).all()
+    assert _fuse_rows([b], 4, torch.device("cpu"), torch.float32)[1] is None
+    with pytest.raises(ValueError):
+        _fuse_rows([Part([("q", torch.ones(3, 4))], {"q": torch.ones(2)})], 4, torch.device("cpu"), torch.float32)
+
+
+def test_zaronex_plain_implementation():
+    import math
+
+    from lit_gpt.config import LayeredConfig
+    from lit_gpt.layered import LayeredGPT
+    from oracle import zaronex as orc
+
+    cfg = _zar_cfg()
+    w = LayeredGPT.random_weights(LayeredConfig.from_dict(cfg), seed=3)
+    toks = [3, 7, 1, 0, 22, 5, 9, 9, 4, 13, 2, 8]
+    full = orc.forward(cfg, w, toks)
+    assert torch.allclose(orc.forward(cfg, w, toks[:7]), full[:7], atol=1e-10)  # causal
+    D = torch.float64
+    # a window of 2 with blocks of 2, all scores equal: position 5 sees tokens 4, 5 and blocks (0, 1), (2, 3); position 4
+    # sees tokens 3, 4 and block (0, 1) - token 2 has left the window and its block is not complete before it
+    q, k = torch.zeros(6, 1, 1, dtype=D), torch.zeros(6, 1, 1, dtype=D)
+    v = torch.tensor([1.0, 3.0, 10.0, 20.0, 100.0, 200.0], dtype=D).view(6, 1, 1)
+    out = orc.window_attention(q, k, v, 1.0, size=2, pool=2).view(-1)
+    assert out.tolist() == pytest.approx([1.0, 2.0, 6.5, (10 + 20 + 2) / 3, (20 + 100 + 2) / 3, (100 + 200 + 2 + 15) / 4])
+    assert orc.window_attention(q, k, v, 1.0, size=2).view(-1).tolist() == pytest.approx([1.0, 2.0, 6.5, 15.0, 60.0, 150.0])
+    # a sink of score 0 beside one key of score 0 takes half
+    assert orc.window_attention(q[:1], k[:1], v[:1], 1.0, 1, 0, torch.zeros(1, dtype=D)).item() == pytest.approx(0.5)
+    # rotations: layouts, and turning back undoes turning
+    x = torch.tensor([[[1.0, 0.0, 0.0, 5.0]]], dtype=D)
+    half = orc.rotate(x, [3], [0.25], "half")[0, 0]
+    assert torch.allclose(half, torch.tensor([math.cos(0.75), math.sin(0.75), 0.0, 5.0], dtype=D))
+    inter = orc.rotate(x, [3], [0.25, 0.5], "interleaved")[0, 0]
+    assert torch.allclose(inter, torch.tensor([math.cos(0.75), math.sin(0.75), -5 * math.sin(1.5), 5 * math.cos(1.5)], dtype=D))
+    assert torch.allclose(orc.rotate(orc.rotate(x, [3], [0.25, 0.5], "half"), [3], [0.25, 0.5], "half", -1.0), x)
+    # the scan: one channel, one state, A = -ln 2 and dt = 1 halve the state per token
+    one = torch.ones(3, 1, dtype=D)
+    y, S = orc.channel_scan(one, one, torch.full((1, 1), -math.log(2.0), dtype=D), one, one, torch.zeros(1, dtype=D))
+    assert y.view(-1).tolist() == pytest.approx([1.0, 1.5, 1.75]) and S.item() == pytest.approx(1.75)
+    c = orc.causal_conv(torch.tensor([[1.0], [2.0], [3.0]], dtype=D), torch.tensor([[10.0, 1.0]], dtype=D), torch.zeros(1, dtype=D))
+    assert c.view(-1).tolist() == [1.0, 12.0, 23.0]
+    assert orc.depth_average([one, 2 * one], torch.tensor([3.0, 0.5], dtype=D))[0].item() == 4.0
