@@ -780,6 +780,58 @@ def sandwich_bench(args) -> None:
         print(json.dumps(line), flush=True)
 
 
+def windowed_bench(args) -> None:
+    """``--windowed``: prefill and decode throughput of the Zaronex design (pre-norm layers with an average over the depth:
+    pooled-window attention beside the gated linear attention, windowed attention with rotated values beside the Mamba
+    scan, windowed latent attention with a query latent; gated gelu feed-forwards; random bf16 weights) at sizes that
+    resemble a real model's layers, beside the closest existing model of the framework - the Gatutar layers (softmax
+    attention beside linear-attention rules, both branches normed) with dense feed-forwards of equal parameter count - at
+    equal width, depth and head counts. One JSON line per size: one 2048-token prompt (warm, median of 3) and captured
+    greedy decode steps at context 2048, for 1 and 8 sequences."""
+    from lit_gpt.config import LayeredConfig
+    from lit_gpt.layered import LayeredGPT
+
+    dev = torch.device("cuda", 0)
+    T, L, V = args.prompt_len, 4, 32000
+    sizes = {"w2048": (2048, 5632), "w4096": (4096, 11008)}
+    for name, (W, ff) in sizes.items():
+        if args.windowed not in ("all", name):
+            continue
+        H = W // 128
+        dense = {"kind": "dense", "ff": ff}
+        att = {"heads": H, "kv_heads": H // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+        gla = {"heads": H // 2, "dim": 128, "vdim": 128, "tau": 8.0, "decay_rank": W // 32}
+        pool = {"type": "parallel", "mlp": dense, "mixer": {
+            "left": dict(att, mask={"size": 1024, "pool": 32}, rot={"dims": 64, "base": 1e6}), "right": gla}}
+        rotv = {"type": "parallel_2", "mlp": dense, "mixer": {
+            "left": dict(att, mask={"size": 1024}, rot={"dims": 128, "base": 1e5, "scaling": {"factor": 2.0}}),
+            "right": {"inner": 2 * W, "state": 16, "dt_rank": W // 16, "conv": 4}}}
+        lat = {"type": "latent_attention", "mlp": dense, "mixer": {
+            "heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 3 * W // 4,
+            "rot": {"dims": 64, "base": 1e5}, "scale": 192 ** -0.5, "mask": {"size": 1024}}}
+        cfg = LayeredConfig.from_dict({"architecture": "Zaronex", "vocab": V, "width": W, "norm": {"eps": 1e-5},
+                                       "layers": [pool, rotv, lat, pool]})
+        line = {"bench": "windowed", "size": name, "width": W, "ff": ff, "layers": L, "prompt_len": T, "steps": args.steps,
+                "dtype": "bf16", "data": "synthetic"}
+        model = LayeredGPT(cfg, LayeredGPT.random_weights(cfg, seed=1), device=dev, dtype=torch.bfloat16)
+        line["zaronex"] = _layered_timings(model, args, T, V)
+        del model
+        torch.cuda.empty_cache()
+        wide = {"kind": "dense", "ff": 3 * ff // 2}
+        kv = {"type": "parallel_2", "mlp": wide, "mixer": {
+            "left": dict(att, q_temp={"coef": 0.1, "every": 512}),
+            "right": {"heads": H // 2, "dim": 128, "vdim": 128,
+                      "decay": [1.0 - 2.0 ** (-5 - 3 * i / max(1, H // 2 - 1)) for i in range(H // 2)]}}}
+        rot = {"type": "parallel", "mlp": wide, "mixer": {"left": dict(att, rot={"dims": 64, "base": 1e6}), "right": gla}}
+        gcfg = LayeredConfig.from_dict({"architecture": "Gatutar", "vocab": V, "width": W, "norm": {"eps": 1e-5},
+                                        "layers": [rot, kv, kv, rot]})
+        model = LayeredGPT(gcfg, LayeredGPT.random_weights(gcfg, seed=1), device=dev, dtype=torch.bfloat16)
+        line["gatutar_layers"] = _layered_timings(model, args, T, V)
+        del model
+        torch.cuda.empty_cache()
+        print(json.dumps(line), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -795,6 +847,9 @@ def main():
     ap.add_argument("--sandwich", nargs="?", const="all", default=None, choices=("all", "w2048", "w4096"),
                     help="instead of the headline run: the Gatutar design (sandwich norms, softmax attention beside "
                          "linear-attention rules, sigmoid-routed experts) beside the Ravelorn layers at equal size")
+    ap.add_argument("--windowed", nargs="?", const="all", default=None, choices=("all", "w2048", "w4096"),
+                    help="instead of the headline run: the Zaronex design (windowed and pooled attention, latent attention, "
+                         "Mamba scan, average over the depth) beside the Gatutar layers at equal size")
     # defaults: the eager capture step (p = 2048) + 14 warm-up + 240 timed steps = the 255 decode steps of
     # SURVEY §8d (p = 2048 ... 2302)
     ap.add_argument("--steps", type=int, default=240)
@@ -822,6 +877,8 @@ def main():
         return delta_bench(args)
     if args.sandwich:
         return sandwich_bench(args)
+    if args.windowed:
+        return windowed_bench(args)
     traffic = {k: (None, "skipped") for k in ("gemv", "attention")}
     under_profiler = any(k.startswith(("ROCPROF", "ROCP_")) for k in os.environ)
     headline = args.model == MODEL and args.quantize == "int4-g128"

@@ -39,10 +39,11 @@ int lgs_version(void);
  * (stride_a and stride_y are then ignored for the rows' place). a_bf16: A is a producer's bf16 copy (MFMA tiles with
  * bf16 weights only): the same values the fp32 stream would be rounded to, at half the operand traffic. y_bf16: the
  * result is written as bf16 (it feeds another bf16 product; MFMA tiles, no accumulate). bias: N fp32 values (NULL:
- * none), the same for every batch. */
+ * none), the same for every batch. ksplit > 1 (a plain product on the MFMA tiles with few tiles and a long K): that many
+ * ranges of K run side by side and are summed in order by a second launch; part: ksplit M N floats of workspace. */
 int lgs_linear(const void* a, long lda, long stride_a, const void* w, int w_f32, long stride_w, void* y, long ldy,
                long stride_y, int M, int N, int K, int batch, int accumulate, int act, const int* a_rows,
-               const int* z_start, int a_bf16, int y_bf16, const float* bias, lgs_stream_t stream);
+               const int* z_start, int a_bf16, int y_bf16, const float* bias, float* part, int ksplit, lgs_stream_t stream);
 /* x[t] = table[tokens[t]] * scale */
 int lgs_embed(const int* tokens, const void* table, int w_f32, float scale, float* x, int T, int W, int vocab,
               lgs_stream_t stream);

@@ -29,16 +29,21 @@ struct LinArgs {
   const uint16_t* a16;  // MFMA tiles only: A as bf16 (a producer's rounded copy) instead of fp32 `a`
   uint16_t* y16;        // MFMA tiles only: Y written as bf16 (the operand of a following bf16 product), no accumulate
   const float* bias;    // [N] added to the product ahead of the activation (null: none)
+  float* part;          // MFMA tiles only: partial sums [ksplit][M][N] of equal ranges of K, summed by lin_sum_kernel
+  int ksplit, kper;     // (ksplit 1: none); kper: BK-deep steps per range
 };
 
 // ------------------------------------------------------------------------------------------------ GEMV, M <= 8
 // R output columns per wave: 4 for tall matrices (more loads in flight per lane), fewer for short ones (more waves)
-template <bool WF32, int MT, int R>
+// KS 4: short and deep matrices; the four waves of a workgroup share its R columns, each a quarter of K
+template <bool WF32, int MT, int R, int KS>
 __global__ void __launch_bounds__(256) lin_gemv_kernel(LinArgs p) {
+  __shared__ float shared_acc[KS > 1 ? 4 * MT * R : 1];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int z = blockIdx.y;
-  const int n0 = (blockIdx.x * 4 + wave) * R;
+  const int n0 = (KS > 1 ? blockIdx.x : blockIdx.x * 4 + wave) * R;
   if (n0 >= p.N) return;
+  const int kl = KS > 1 ? wave * 64 + lane : lane;  // this lane's place in a pass over K
   const float* a = p.a + (size_t)z * p.sa;
   const size_t wbase = (size_t)z * p.sw;
   float acc[MT][R];
@@ -58,7 +63,7 @@ __global__ void __launch_bounds__(256) lin_gemv_kernel(LinArgs p) {
   }
   if (vec) {
 #pragma unroll 2
-    for (int k = lane * 8; k < K; k += 512) {
+    for (int k = kl * 8; k < K; k += 512 * KS) {
       float wv[R][8];
 #pragma unroll
       for (int r = 0; r < R; ++r) {
@@ -89,7 +94,7 @@ __global__ void __launch_bounds__(256) lin_gemv_kernel(LinArgs p) {
       }
     }
   } else {
-    for (int k = lane; k < K; k += 64) {
+    for (int k = kl; k < K; k += 64 * KS) {
       float wv[R];
 #pragma unroll
       for (int r = 0; r < R; ++r) wv[r] = wload<WF32>(p.w, wbase + (size_t)rows[r] * K + k);
@@ -106,13 +111,28 @@ __global__ void __launch_bounds__(256) lin_gemv_kernel(LinArgs p) {
   for (int m = 0; m < MT; ++m)
 #pragma unroll
     for (int r = 0; r < R; ++r) {
-      const float s = wave_sum(acc[m][r]);
+      float s = wave_sum(acc[m][r]);
+      if (KS > 1) {
+        if (lane == 0) shared_acc[(wave * MT + m) * R + r] = s;
+        continue;
+      }
       if (lane == 0 && m < p.M && n0 + r < p.N) {
         float* yp = p.y + (size_t)z * p.sy + (size_t)m * p.ldy + n0 + r;
         const float v = act_f(p.act, s + bias[r]);
         *yp = p.accumulate ? *yp + v : v;
       }
     }
+  if (KS > 1) {
+    __syncthreads();
+    const int m = threadIdx.x / R, r = threadIdx.x % R;
+    if (m < MT && m < p.M && n0 + r < p.N) {
+      const float* q = shared_acc + m * R + r;
+      const float s = (q[0] + q[MT * R]) + (q[2 * MT * R] + q[3 * MT * R]);
+      float* yp = p.y + (size_t)z * p.sy + (size_t)m * p.ldy + n0 + r;
+      const float v = act_f(p.act, s + (p.bias ? p.bias[n0 + r] : 0.0f));
+      *yp = p.accumulate ? *yp + v : v;
+    }
+  }
 }
 
 // ------------------------------------------------------------------------------------------------ MFMA tiles
@@ -127,7 +147,7 @@ __global__ void __launch_bounds__(256) lin_mfma_kernel(LinArgs p) {
   __shared__ __attribute__((aligned(16))) unsigned char lds[2 * 2 * TILE_BYTES];  // [buf][A|W]
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int wm = wave >> 1, wn = wave & 1;
-  const int z = blockIdx.z;
+  const int z = p.ksplit > 1 ? 0 : blockIdx.z;
   const int r_lo = p.z_start ? p.z_start[z] : 0;
   const int Mz = p.z_start ? p.z_start[z + 1] - r_lo : p.M;
   const int m0 = blockIdx.y * BM, n0 = blockIdx.x * BN;
@@ -135,7 +155,12 @@ __global__ void __launch_bounds__(256) lin_mfma_kernel(LinArgs p) {
   const float* abase = A16 ? nullptr : p.a + (size_t)z * p.sa;
   const uint16_t* abase16 = A16 ? p.a16 + (size_t)z * p.sa : nullptr;
   const uint16_t* wbase = (const uint16_t*)p.w + (size_t)z * p.sw;
-  const int K = p.K, nk = (K + BK - 1) / BK;
+  const int K = p.K;
+  int kt_lo = 0, nk = (K + BK - 1) / BK;
+  if (p.ksplit > 1) {
+    kt_lo = blockIdx.z * p.kper;
+    nk = min(nk, kt_lo + p.kper);
+  }
   const int t_row = tid >> 1, t_half = tid & 1;
   const int lr = r_lo + min(m0 + t_row, Mz - 1);  // rows past the end repeat the last one (never stored)
   const size_t arow_off = (size_t)(p.a_rows ? p.a_rows[lr] : lr) * p.lda;
@@ -201,12 +226,12 @@ __global__ void __launch_bounds__(256) lin_mfma_kernel(LinArgs p) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 
-  gload(0);
+  gload(kt_lo);
   lstore(0);
   __syncthreads();
   const int fr = lane & 15, fk = lane >> 4;
-  for (int kt = 0; kt < nk; ++kt) {
-    const int cur = kt & 1;
+  for (int kt = kt_lo; kt < nk; ++kt) {
+    const int cur = (kt - kt_lo) & 1;
     if (kt + 1 < nk) gload(kt + 1);
     const unsigned char* A = lds + cur * (2 * TILE_BYTES);
     const unsigned char* B = A + TILE_BYTES;
@@ -238,12 +263,30 @@ __global__ void __launch_bounds__(256) lin_mfma_kernel(LinArgs p) {
       for (int r = 0; r < 4; ++r) {
         const int m = m0 + wm * 64 + i * 16 + fk * 4 + r;
         if (m >= Mz) continue;
+        if (p.ksplit > 1) {
+          p.part[((size_t)blockIdx.z * p.M + m) * p.N + n] = acc[i][j][r];
+          continue;
+        }
         const size_t at = (size_t)z * p.sy + (size_t)(r_lo + m) * p.ldy + n;
         const float v = act_f(p.act, acc[i][j][r] + bias);
         if (p.y16) p.y16[at] = f2bf(v);
         else p.y[at] = p.accumulate ? p.y[at] + v : v;
       }
   }
+}
+
+// the ranges of K in ascending order, then bias, activation and place as the tiles would. grid (ceil(N / 256), M)
+__global__ void __launch_bounds__(256) lin_sum_kernel(LinArgs p) {
+  const int n = blockIdx.x * 256 + threadIdx.x;
+  const size_t m = blockIdx.y;
+  if (n >= p.N) return;
+  float s = 0.0f;
+#pragma unroll 4
+  for (int z = 0; z < p.ksplit; ++z) s += p.part[((size_t)z * p.M + m) * p.N + n];
+  const float v = act_f(p.act, s + (p.bias ? p.bias[n] : 0.0f));
+  const size_t at = m * p.ldy + n;
+  if (p.y16) p.y16[at] = f2bf(v);
+  else p.y[at] = p.accumulate ? p.y[at] + v : v;
 }
 
 // ------------------------------------------------------------------------------------------------ fp32 tiles
@@ -421,8 +464,8 @@ __global__ void __launch_bounds__(256) gather_rows_kernel(const float* __restric
 
 extern "C" int lgs_linear(const void* a_any, long lda, long stride_a, const void* w, int w_f32, long stride_w, void* y_any,
                           long ldy, long stride_y, int M, int N, int K, int batch, int accumulate, int act,
-                          const int* a_rows, const int* z_start, int a_bf16, int y_bf16, const float* bias,
-                          hipStream_t stream) {
+                          const int* a_rows, const int* z_start, int a_bf16, int y_bf16, const float* bias, float* part,
+                          int ksplit, hipStream_t stream) {
   const float* a = (const float*)a_any;  // (bf16 when a_bf16)
   float* y = (float*)y_any;              // (bf16 when y_bf16)
   LGA_CHECK_ARG(a && w && y, "lgs_linear: null pointer");
@@ -434,20 +477,24 @@ extern "C" int lgs_linear(const void* a_any, long lda, long stride_a, const void
   LGA_CHECK_ARG(!y_bf16 || (!w_f32 && !accumulate && (M > 8 || z_start || a_rows)),
                 "lgs_linear: a bf16 result comes from the MFMA tiles (bf16 weights, more than 8 rows, no accumulate)");
   lgs::LinArgs p{a, lda, stride_a, w, stride_w, y, ldy, stride_y, M, N, K, accumulate, act, a_rows, z_start,
-                 a_bf16 ? (const uint16_t*)a : nullptr, y_bf16 ? (uint16_t*)y : nullptr, bias};
+                 a_bf16 ? (const uint16_t*)a : nullptr, y_bf16 ? (uint16_t*)y : nullptr, bias, nullptr, 1, 0};
+  LGA_CHECK_ARG(ksplit >= 1 && (ksplit == 1 || (part && !w_f32 && batch == 1 && !z_start && !a_rows && M > 8 && M <= 65535)),
+                "lgs_linear: K is split for one plain product on the MFMA tiles, with a workspace");
   if (M <= 8 && !z_start && !a_rows) {
     const int R = N >= 16384 ? 4 : (N >= 4096 ? 2 : 1);
-    const dim3 grid((N + 4 * R - 1) / (4 * R), batch);
-#define LGS_GEMV_R(MT, RR)                                                              \
+    const bool deep = (long)N * batch <= 512 && K >= 1024;  // few columns: four waves per column
+    const dim3 grid(deep ? N : (N + 4 * R - 1) / (4 * R), batch);
+#define LGS_GEMV_R(MT, RR, KS)                                                          \
   do {                                                                                  \
-    if (w_f32) lgs::lin_gemv_kernel<true, MT, RR><<<grid, 256, 0, stream>>>(p);         \
-    else lgs::lin_gemv_kernel<false, MT, RR><<<grid, 256, 0, stream>>>(p);              \
+    if (w_f32) lgs::lin_gemv_kernel<true, MT, RR, KS><<<grid, 256, 0, stream>>>(p);     \
+    else lgs::lin_gemv_kernel<false, MT, RR, KS><<<grid, 256, 0, stream>>>(p);          \
   } while (0)
-#define LGS_GEMV(MT)                 \
-  do {                               \
-    if (R == 4) LGS_GEMV_R(MT, 4);   \
-    else if (R == 2) LGS_GEMV_R(MT, 2); \
-    else LGS_GEMV_R(MT, 1);          \
+#define LGS_GEMV(MT)                       \
+  do {                                     \
+    if (R == 4) LGS_GEMV_R(MT, 4, 1);      \
+    else if (R == 2) LGS_GEMV_R(MT, 2, 1); \
+    else if (deep) LGS_GEMV_R(MT, 1, 4);   \
+    else LGS_GEMV_R(MT, 1, 1);             \
   } while (0)
     if (M == 1) LGS_GEMV(1);
     else if (M == 2) LGS_GEMV(2);
@@ -463,7 +510,13 @@ extern "C" int lgs_linear(const void* a_any, long lda, long stride_a, const void
     lgs::lin_fma_kernel<true><<<grid, 256, 0, stream>>>(p);
     LGA_LAUNCH_RETURN();
   }
-  const dim3 grid((N + lgs::BN - 1) / lgs::BN, (M + lgs::BM - 1) / lgs::BM, batch);
+  if (ksplit > 1) {
+    const int nk = (K + lgs::BK - 1) / lgs::BK;
+    p.part = part;
+    p.kper = (nk + ksplit - 1) / ksplit;
+    p.ksplit = (nk + p.kper - 1) / p.kper;  // (no empty range)
+  }
+  const dim3 grid((N + lgs::BN - 1) / lgs::BN, (M + lgs::BM - 1) / lgs::BM, p.ksplit > 1 ? p.ksplit : batch);
   LGA_CHECK_ARG(grid.y <= 65535, "lgs_linear: too many rows");
   const int am = a_bf16 ? 8 : 4;  // elements per 16 bytes of A
   const bool vec = K % 8 == 0 && lda % am == 0 && stride_a % am == 0 && stride_w % 8 == 0 && (uintptr_t)a % 16 == 0 &&
@@ -475,6 +528,7 @@ extern "C" int lgs_linear(const void* a_any, long lda, long stride_a, const void
     if (vec) lgs::lin_mfma_kernel<true, false><<<grid, 256, 0, stream>>>(p);
     else lgs::lin_mfma_kernel<false, false><<<grid, 256, 0, stream>>>(p);
   }
+  if (p.ksplit > 1) lgs::lin_sum_kernel<<<dim3((N + 255) / 256, M), 256, 0, stream>>>(p);
   LGA_LAUNCH_RETURN();
 }
 

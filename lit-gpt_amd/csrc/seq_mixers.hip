@@ -807,20 +807,25 @@ __global__ void __launch_bounds__(256) latent_combine_kernel(const float* __rest
                                                              float* __restrict__ out, int H, int r, int splits) {
   const int t = blockIdx.x, h = blockIdx.y;
   const float* pp = part + ((size_t)t * H + h) * splits * (r + 2);
+  // the splits' factors once, a thread each (at most 256 splits), then every column one weighted sum over them
+  __shared__ float wz[256], red[4];
+  const int z0 = threadIdx.x;
   const float snk = sink ? sink[h] : -INFINITY;
-  float mx = snk;
-  for (int z = 0; z < splits; ++z)
-    if (pp[(size_t)z * (r + 2) + 1] > 0.0f) mx = fmaxf(mx, pp[(size_t)z * (r + 2)]);
-  float den = sink ? expf(snk - mx) : 0.0f;
-  for (int z = 0; z < splits; ++z) {
-    const float lz = pp[(size_t)z * (r + 2) + 1];
-    if (lz > 0.0f) den += lz * expf(pp[(size_t)z * (r + 2)] - mx);
-  }
+  const float lz = z0 < splits ? pp[(size_t)z0 * (r + 2) + 1] : 0.0f;
+  const float mz = lz > 0.0f ? pp[(size_t)z0 * (r + 2)] : -INFINITY;
+  float mx = wave_max(mz);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = mx;
+  __syncthreads();
+  mx = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), snk);
+  const float f = lz > 0.0f ? expf(mz - mx) : 0.0f;
+  wz[z0] = f;
+  const float den = block_sum_256(lz * f, red) + (sink ? expf(snk - mx) : 0.0f);
   for (int i = threadIdx.x; i < r; i += 256) {
     float a = 0.0f;
+#pragma unroll 8
     for (int z = 0; z < splits; ++z) {
-      const float lz = pp[(size_t)z * (r + 2) + 1];
-      if (lz > 0.0f) a += pp[(size_t)z * (r + 2) + 2 + i] * expf(pp[(size_t)z * (r + 2)] - mx);
+      const float v = pp[(size_t)z * (r + 2) + 2 + i];
+      a = fmaf(wz[z], wz[z] > 0.0f ? v : 0.0f, a);  // (an empty split's row is not written)
     }
     out[((size_t)t * H + h) * r + i] = a / den;
   }

@@ -256,14 +256,23 @@ __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
   if (DEPTH) {
 #pragma unroll
     for (int e = 0; e < CPT; ++e) hv[e] = 0.0f;
-#pragma unroll 2
-    for (int j = 0; j < p.n_prev; ++j) {
-      const float c = p.depth_w[j];
+    constexpr int HB = CPT > 8 ? 2 : 4;  // earlier results fetched side by side
+    for (int j = 0; j < p.n_prev; j += HB) {
+      float t[HB][CPT], c[HB];
 #pragma unroll
-      for (int e = 0; e < CPT; ++e) {
-        const int i = tid + 256 * e;
-        if (i < n) hv[e] = fmaf(c, p.hist[j * hs + r * n + i], hv[e]);
+      for (int k = 0; k < HB; ++k) {
+        const bool there = j + k < p.n_prev;
+        c[k] = there ? p.depth_w[j + k] : 0.0f;
+#pragma unroll
+        for (int e = 0; e < CPT; ++e) {
+          const int i = tid + 256 * e;
+          t[k][e] = (there && i < n) ? p.hist[(j + k) * hs + r * n + i] : 0.0f;
+        }
       }
+#pragma unroll
+      for (int k = 0; k < HB; ++k)
+#pragma unroll
+        for (int e = 0; e < CPT; ++e) hv[e] = fmaf(c[k], t[k][e], hv[e]);
     }
   }
   if (a) {

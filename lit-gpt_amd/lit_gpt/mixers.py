@@ -364,7 +364,8 @@ class ChannelScan(InputReader):
         tables = (step.seq_start, step.seq_slot, step.seq_pos0)
         xc = seq_ops.conv_silu(proj, self.off["in"], self.conv_w, self.conv_b, cache.conv, *tables, step.max_len or T)
         bc = torch.empty(T, R + 2 * N, dtype=torch.float32, device=dev)
-        seq_ops.linear(xc, self.w_x, M=T, N=R + 2 * N, K=inner, y=bc, lda=inner, ldy=R + 2 * N)
+        seq_ops.linear(xc, self.w_x, M=T, N=R + 2 * N, K=inner, y=bc, lda=inner, ldy=R + 2 * N,
+                       ksplit=seq_ops.thin_ksplit(T, R + 2 * N, inner, self.w_x))
         kw = dict(max_len=step.max_len or T, bf16=_tiles16(T, self.w_o))
         if T <= self.LOWRANK_ROWS and R <= 1024:
             y = seq_ops.channel_scan(xc, proj, self.off["in"] + inner, bc, R, self.a2, self.D, cache.s, *tables,

@@ -31,7 +31,7 @@ _P, _I, _L, _F = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
 SIGNATURES = {
     "lgs_version": [],
     "lgs_last_error_string": [],
-    "lgs_linear": [_P, _L, _L, _P, _I, _L, _P, _L, _L, _I, _I, _I, _I, _I, _I, _P, _P, _I, _I, _P, _P],
+    "lgs_linear": [_P, _L, _L, _P, _I, _L, _P, _L, _L, _I, _I, _I, _I, _I, _I, _P, _P, _I, _I, _P, _P, _I, _P],
     "lgs_embed": [_P, _P, _I, _F, _P, _I, _I, _I, _P],
     "lgs_rmsnorm": [_P, _L, _P, _F, _F, _P, _L, _I, _I, _I, _P, _P],
     "lgs_gather_rows": [_P, _P, _P, _I, _I, _P],
@@ -147,11 +147,13 @@ F32, I32 = torch.float32, torch.int32
 def linear(a: torch.Tensor, w: torch.Tensor, *, M: int, N: int, K: int, y: torch.Tensor, a_off: int = 0, lda: int,
            y_off: int = 0, ldy: int, batch: int = 1, stride_a: int = 0, stride_w: int = 0, stride_y: int = 0,
            accumulate: bool = False, act: int = ACT_NONE, a_rows: Optional[torch.Tensor] = None,
-           z_start: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+           z_start: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None,
+           ksplit: int = 1) -> torch.Tensor:
     """y[z] (+)= act(a[z] w[z]^T + bias) over ``batch`` strided operands; offsets and strides count elements. With
     ``z_start`` (batch + 1 int32 row bounds) batch z owns that range of a row list of at most M rows, whose A rows
     are ``a_rows`` (or the list places themselves) and whose Y rows are the list places. ``a`` may be a producer's
-    bf16 copy (``rmsnorm(bf16_copy=True)``, ``glu(bf16=True)``) for the MFMA tiles with bf16 weights."""
+    bf16 copy (``rmsnorm(bf16_copy=True)``, ``glu(bf16=True)``) for the MFMA tiles with bf16 weights. ``ksplit`` > 1: that
+    many ranges of K side by side (MFMA tiles, one plain product), see ``thin_ksplit``."""
     a16 = a.dtype == torch.bfloat16
     ap = _dev(a, "a", torch.bfloat16 if a16 else F32) + (2 if a16 else 4) * a_off
     y16 = y.dtype == torch.bfloat16  # the result feeds another bf16 product
@@ -162,11 +164,20 @@ def linear(a: torch.Tensor, w: torch.Tensor, *, M: int, N: int, K: int, y: torch
         raise ValueError("linear: an operand is smaller than the sizes and strides say")
     if bias is not None and bias.numel() != N:
         raise ValueError("linear: one bias per output column")
+    part = torch.empty(ksplit * M * N, dtype=F32, device=y.device) if ksplit > 1 else None
     _check(load_library().lgs_linear(ap, lda, stride_a, _dev(w, "w"), _wf32(w, "w"), stride_w, yp, ldy, stride_y,
                                      M, N, K, batch, int(accumulate), act, _opt(a_rows, "a_rows", I32),
                                      _opt(z_start, "z_start", I32), int(a16), int(y16), _opt(bias, "bias", F32),
-                                     _stream()))
+                                     _opt(part, "part", F32), int(ksplit), _stream()))
     return y
+
+
+def thin_ksplit(M: int, N: int, K: int, w: torch.Tensor) -> int:
+    """Ranges of K for a product whose 128 x 128 tiles alone would leave most of the chip idle (1: as it is)."""
+    if M <= 8 or M > 65535 or w.dtype != torch.bfloat16:
+        return 1
+    tiles = ((M + 127) // 128) * ((N + 127) // 128)
+    return max(1, min(16, 512 // tiles, K // 256))
 
 
 def embed(tokens: torch.Tensor, table: torch.Tensor, scale: float, out: Optional[torch.Tensor] = None) -> torch.Tensor:

@@ -683,6 +683,43 @@ def test_projection_with_a_bias(M, N, K, dtype):
     assert (y.cpu().to(D) - orc.silu(want)).abs().max() < 1e-5 * K
 
 
+@pytest.mark.parametrize("M,N,K", [(9, 33, 1000), (130, 20, 520), (70, 260, 64), (300, 5, 2048)])
+@pytest.mark.parametrize("ksplit", [2, 3, 16])
+def test_thin_product_over_ranges_of_k(M, N, K, ksplit):
+    """Ranges of K side by side: the plain product with bias, activation, accumulation and bf16 operands and results."""
+    from lit_gpt import seq_ops
+
+    dev = torch.device("cuda", 0)
+    g = torch.Generator().manual_seed(M + N + ksplit)
+    a = torch.randn(M, K, generator=g).to(torch.bfloat16)
+    w = (torch.randn(N, K, generator=g) * K ** -0.5).to(torch.bfloat16)
+    b = torch.randn(N, generator=g)
+    want = a.to(D) @ w.to(D).T + b.to(D)
+    kw = dict(M=M, N=N, K=K, lda=K, ldy=N, bias=b.to(dev), ksplit=ksplit)
+    y = torch.full((M, N), 2.0, device=dev)
+    seq_ops.linear(a.float().to(dev), w.to(dev), y=y, accumulate=True, **kw)
+    assert (y.cpu().to(D) - 2.0 - want).abs().max() < 2e-5
+    y16 = torch.empty(M, N, device=dev, dtype=torch.bfloat16)
+    seq_ops.linear(a.to(dev), w.to(dev), y=y16, act=seq_ops.ACT_SILU, **kw)
+    assert (y16.cpu().to(D) - orc.silu(want)).abs().max() < 4e-2
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("M", [1, 2, 3, 8])
+@pytest.mark.parametrize("N,K", [(1, 1024), (160, 4096), (512, 1032), (77, 2051)])
+def test_short_deep_products_of_few_rows(M, N, K, dtype):
+    from lit_gpt import seq_ops
+
+    dev = torch.device("cuda", 0)
+    g = torch.Generator().manual_seed(M + N)
+    a = torch.randn(M, K, generator=g).to(dtype).float()
+    w = (torch.randn(N, K, generator=g) * K ** -0.5).to(dtype)
+    b = torch.randn(N, generator=g)
+    y = torch.full((M, N), 1.0, device=dev)
+    seq_ops.linear(a.to(dev), w.to(dev), M=M, N=N, K=K, y=y, lda=K, ldy=N, bias=b.to(dev), accumulate=True)
+    assert (y.cpu().to(D) - 1.0 - a.to(D) @ w.to(D).T - b.to(D)).abs().max() < 3e-5
+
+
 # ------------------------------------------------------------------------------------------------ entry points
 def follows_plain_greedy(cfg, w, prompt, out, margin=1e-3):
     """Every generated token is the plain implementation's argmax given the tokens before it (or within a rounding
