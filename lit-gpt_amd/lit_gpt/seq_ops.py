@@ -177,7 +177,7 @@ def thin_ksplit(M: int, N: int, K: int, w: torch.Tensor) -> int:
     if M <= 8 or M > 65535 or w.dtype != torch.bfloat16:
         return 1
     tiles = ((M + 127) // 128) * ((N + 127) // 128)
-    return max(1, min(16, 512 // tiles, K // 256))
+    return 1 if tiles > 64 else max(1, min(16, 512 // tiles, K // 256))
 
 
 def embed(tokens: torch.Tensor, table: torch.Tensor, scale: float, out: Optional[torch.Tensor] = None) -> torch.Tensor:
