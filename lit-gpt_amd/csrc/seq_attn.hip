@@ -342,19 +342,16 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
   const size_t slot = p.seq_slot[b];
   const int chunk = p.chunk;
   int lo = chunk > 0 ? pos_first - pos_first % chunk : 0, hi = pos_last + 1;
-  int plo = 0, phi = 0;  // pooled blocks
+  int np = 0;  // pooled blocks: rows 0 .. np - 1 of the walk below, followed by the cached keys lo .. hi - 1
   if (WIN) {
     lo = max(0, pos_first - p.window + 1);
-    if (p.pool > 0) phi = min(pooled_seen(pos_last, p.window, p.pool), p.pool_rows);
+    if (p.pool > 0) np = min(pooled_seen(pos_last, p.window, p.pool), p.pool_rows);
   }
-  if (gridDim.z > 1) {  // (QT == 1) an equal share of the blocks and keys, in whole numbers
-    const int np = phi, n = np + hi - lo, per = (n + gridDim.z - 1) / gridDim.z;
-    const int u0 = blockIdx.z * per, u1 = min(n, u0 + per);  // share of the blocks followed by the keys
-    plo = min(u0, np);
-    phi = max(plo, min(u1, np));
-    const int first = lo;
-    lo = first + max(u0 - np, 0);
-    hi = first + max(u1 - np, 0);
+  int from = 0, to = np + hi - lo;
+  if (gridDim.z > 1) {  // (QT == 1) an equal share of the rows, in whole numbers
+    const int per = (to + gridDim.z - 1) / gridDim.z;
+    from = blockIdx.z * per;
+    to = min(to, from + per);
   }
   for (int i = tid; i < nq * d2; i += 256) qs[i] = p.q[(size_t)(r0 + i / d2) * p.ld + (size_t)h * d2 + i % d2];
   if (tid < NR) {
@@ -372,21 +369,20 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
     for (int m = 0; m < MAPS; ++m) acc[i][m] = 0.0f;
   __syncthreads();
 
-  // key tiles of one source: the cached keys (pooled = false) or the pooled blocks, whose rows are fp32
-  auto walk = [&](auto src_f32, const bool pooled, const void* keys, const void* values, const int rows, const int from,
-                  const int to) {
-  constexpr bool KF32 = decltype(src_f32)::value;
-  for (int k0 = from; k0 < to; k0 += kKeyTile) {
-    const int nk = min(kKeyTile, to - k0);
-    // ---- scores of key k0 + tid against every query and map
+  const int shift = lo - np;  // cache row of walk row u >= np: u + shift
+  for (int u0 = from; u0 < to; u0 += kKeyTile) {
+    const int nk = min(kKeyTile, to - u0);
+    const int u = u0 + tid;
+    const bool pooled = WIN && u < np;
+    // ---- scores of row u against every query and map
     {
       float s[QT][MAPS];
 #pragma unroll
       for (int i = 0; i < QT; ++i)
 #pragma unroll
         for (int m = 0; m < MAPS; ++m) s[i][m] = 0.0f;
-      if (tid < nk) {
-        const size_t kr = ((slot * rows + k0 + tid) * p.G + g) * d2;
+      auto score = [&](auto row_f32, const void* keys, const size_t kr) {
+        constexpr bool KF32 = decltype(row_f32)::value;
         if ((d & 3) == 0) {
 #pragma unroll
           for (int m = 0; m < MAPS; ++m)
@@ -417,18 +413,19 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
               for (int i = 0; i < QT; ++i) s[i][m] = fmaf(qs[i * d2 + m * d + e], kv, s[i][m]);
             }
         }
+      };
+      if (pooled) {  // (the blocks' rows are fp32)
+        if (tid < nk) score(std::true_type{}, p.pool_k, ((slot * p.pool_rows + u) * p.G + g) * d2);
+      } else if (tid < nk) {
+        score(std::integral_constant<bool, CF32>{}, p.cache_k, ((slot * p.S + u + shift) * p.G + g) * d2);
       }
-      const int kpos = k0 + tid;
+      const int kpos = u + shift;
 #pragma unroll
       for (int i = 0; i < QT; ++i) {
         const int qpos = pos_first + i;
-        bool see;
-        if (WIN && pooled) {
-          see = tid < nk && i < nq && kpos < pooled_seen(qpos, p.window, p.pool);
-        } else {
-          const int qlo = WIN ? qpos - p.window + 1 : (chunk > 0 ? qpos - qpos % chunk : 0);
-          see = tid < nk && i < nq && kpos <= qpos && kpos >= qlo;
-        }
+        const int qlo = WIN ? qpos - p.window + 1 : (chunk > 0 ? qpos - qpos % chunk : 0);
+        bool see = tid < nk && i < nq && kpos <= qpos && kpos >= qlo;
+        if (pooled) see = tid < nk && i < nq && u < pooled_seen(qpos, p.window, p.pool);
 #pragma unroll
         for (int m = 0; m < MAPS; ++m) {
           float v = s[i][m] * p.scale;
@@ -472,9 +469,7 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
 #pragma unroll
         for (int m = 0; m < MAPS; ++m) acc[i][m] *= arow[MAPS * i + m];
       if (col < dv) {
-#pragma unroll 4
-        for (int j = ks; j < nk; j += KS) {
-          const float v = cload<KF32>(values, ((slot * rows + k0 + j) * p.G + g) * dv + col);
+        auto add = [&](const int j, const float v) {
           float w[NR];
           if (NR == 1) {
             w[0] = sc[j * SCS];
@@ -492,14 +487,18 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
           for (int i = 0; i < QT; ++i)
 #pragma unroll
             for (int m = 0; m < MAPS; ++m) acc[i][m] = fmaf(w[MAPS * i + m], v, acc[i][m]);
+        };
+        int j = ks;
+        if (WIN) {
+#pragma unroll 4
+          for (; j < min(nk, np - u0); j += KS) add(j, p.pool_v[((slot * p.pool_rows + u0 + j) * p.G + g) * dv + col]);
         }
+#pragma unroll 4
+        for (; j < nk; j += KS) add(j, cload<CF32>(p.cache_v, ((slot * p.S + u0 + j + shift) * p.G + g) * dv + col));
       }
     }
     __syncthreads();
   }
-  };
-  if (WIN && phi > plo) walk(std::true_type{}, true, p.pool_k, p.pool_v, p.pool_rows, plo, phi);
-  walk(std::integral_constant<bool, CF32>{}, false, p.cache_k, p.cache_v, p.S, lo, hi);
   // ---- sum the key subsets (fixed order), then finish or leave the split's partial result
   float* xs = sc;  // [KS][NR][ncol] = 256 * NR floats <= the score tile
   if (KS > 1) {
