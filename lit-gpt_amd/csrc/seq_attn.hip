@@ -547,20 +547,29 @@ __global__ void __launch_bounds__(256) diffattn_combine_kernel(AttnArgs p, int s
   const int h = blockIdx.y, dv = p.dv, c = threadIdx.x;
   const int stride = MAPS * (2 + dv);
   const float* pr = p.part + ((t * p.H + h) * splits) * stride;
-  float mx[MAPS], l[MAPS], a[MAPS];
-#pragma unroll
-  for (int m = 0; m < MAPS; ++m) mx[m] = -INFINITY, l[m] = 0.0f, a[m] = 0.0f;
-  for (int z = 0; z < splits; ++z)
-#pragma unroll
-    for (int m = 0; m < MAPS; ++m) mx[m] = fmaxf(mx[m], pr[(size_t)z * stride + 2 * m]);
-  for (int z = 0; z < splits; ++z) {
-    const float* q = pr + (size_t)z * stride;
+  // the splits' factors once, a lane each (at most 64 splits), then every column one weighted sum over them
+  __shared__ float wz[MAPS][64], ml[MAPS][2];
+  if (c < 64) {
 #pragma unroll
     for (int m = 0; m < MAPS; ++m) {
-      const float w = q[2 * m] == -INFINITY ? 0.0f : expf(q[2 * m] - mx[m]);
-      l[m] = fmaf(q[2 * m + 1], w, l[m]);
-      if (c < dv) a[m] = fmaf(q[2 * MAPS + m * dv + c], w, a[m]);
+      const float mz = c < splits ? pr[(size_t)c * stride + 2 * m] : -INFINITY;
+      const float lz = c < splits ? pr[(size_t)c * stride + 2 * m + 1] : 0.0f;
+      const float top = wave_max(mz);
+      const float w = mz == -INFINITY ? 0.0f : expf(mz - top);
+      const float sum = wave_sum(lz * w);
+      wz[m][c] = w;
+      if (c == 0) ml[m][0] = top, ml[m][1] = sum;
     }
+  }
+  __syncthreads();
+  float mx[MAPS], l[MAPS], a[MAPS];
+#pragma unroll
+  for (int m = 0; m < MAPS; ++m) mx[m] = ml[m][0], l[m] = ml[m][1], a[m] = 0.0f;
+  if (c < dv) {
+#pragma unroll 8
+    for (int z = 0; z < splits; ++z)
+#pragma unroll
+      for (int m = 0; m < MAPS; ++m) a[m] = fmaf(pr[(size_t)z * stride + 2 * MAPS + m * dv + c], wz[m][z], a[m]);
   }
   if (MAPS == 2) diff_finish(a[0], a[MAPS - 1], l[0], l[MAPS - 1], p, t, h, red);
   else sink_finish(a[0], mx[0], l[0], p, t, h, p.seq_pos0[t], xch);  // (one token per sequence: row t is sequence t)

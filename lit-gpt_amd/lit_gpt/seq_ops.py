@@ -860,7 +860,7 @@ def sinkattn(proj: torch.Tensor, q_off: int, cache_k: torch.Tensor, cache_v: tor
         splits = 1
     elif splits is None:
         span = min(S, chunk) if chunk > 0 else (min(S, window) + prow if window > 0 else S)
-        splits = max(1, min(64, 512 // max(1, B * H), (span + 127) // 128))
+        splits = max(1, min(64, 512 // max(1, B * H), (span + 63) // 64 if window > 0 else (span + 127) // 128))
     part = torch.empty(T * H * splits * (2 + dv), dtype=F32, device=proj.device) if splits > 1 else None
     _check(load_library().lgs_sinkattn(_dev(proj, "proj", F32) + 4 * q_off, ld, _dev(cache_k, "cache_k"),
                                        _dev(cache_v, "cache_v"), _wf32(cache_k, "cache_k"), _opt(sink, "sink", F32),
