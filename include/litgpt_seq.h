@@ -267,7 +267,7 @@ int lgs_glu_clamped(const float* a, const float* b, long ld, void* out, int out_
 /* ---- selective scan with a diagonal state matrix per channel ---- */
 /* Over a packed batch: dt = softplus(raw), raw the inner columns of dt_raw (row stride ldt; already with their bias) or,
  * with w_dt ([inner][rank], bf16 or fp32), w_dt times the rank columns of bc plus dt_bias;
- * S[n][c] <- exp2(dt_c a2[n][c]) S[n][c] + dt_c x_c B_n, y_c = (sum_n S[n][c] C_n + D_c x_c) * silu(z_c).
+ * per channel s[n] <- 2^(dt a2[n]) s[n] + (dt x) B[n], out = (s . C + D x) silu(z).
  * x [T][inner] (after the convolution), z: columns of the projection (row stride ldz), bc [T][ldbc] = dt inner values
  * (rank) | B (N) | C (N), a2 [N][inner] = A log2(e), state [slots][N][inner] fp32, taken as zero when a sequence starts
  * at position 0. out: fp32, or bf16 with out_bf16. ws (B max_chunks N inner floats) and wsum (B max_chunks inner) with

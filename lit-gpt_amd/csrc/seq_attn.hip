@@ -8,7 +8,7 @@
 // lo(i) = i - i % chunk for a chunked mask (chunks are aligned to the sequence's position 0), i - window + 1 for a
 // sliding window and 0 without either. Beside a window the one-map form can see pooled blocks: block b stands for the
 // positions b pool .. b pool + pool - 1 by the mean of their cached keys and of their values (fp32, kept next to the
-// cache), and is seen when it lies wholly before the window; tokens and blocks share one softmax.
+// cache), and is seen once its last position has left the window; one softmax runs over blocks and tokens together.
 //
 //   lgs_diffattn_prepare  per token: rotary (interleaved pairs 2i, 2i + 1 of the first rot_dims dims of every map)
 //                         on the queries in place and on the keys on their way into the cache; values into the cache.

@@ -7,7 +7,7 @@
 //                        the latent attention's sigmoid gate
 //   lgs_latent_prepare   latent attention, per token: RMS-normed latent c and the rotated shared key part go to the
 //                        cache rows (slot, position); the queries' rotated parts are rotated in place (interleaved)
-//   lgs_latent_attention softmax attention in the latent space: every head's query has been mapped through its key
+//   lgs_latent_attention softmax attention in the latent space (over all rows so far or a window of them): every head's query has been mapped through its key
 //                        up-projection, so all heads read the same cached rows [c | k_rot]; scores, the sink's
 //                        share of the denominator and the weighted sum of c are fp32; the value up-projection
 //                        follows as a per-head product

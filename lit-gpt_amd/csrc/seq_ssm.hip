@@ -8,7 +8,7 @@
 //                        heads share B and C in groups. Token by token (decode, short portions), or for prompts
 //                        in chunks of 64 tokens as fp32 matrix products with the chunks side by side
 //   lgs_channel_scan     the selective scan with a diagonal state matrix per channel (the Mamba form):
-//                        S[n][c] <- exp(dt_c A[c][n]) S[n][c] + dt_c x_c B_n, y_c = (S C)_c + D_c x_c, times silu(z_c);
+//                        s_n <- 2^(dt a2_n) s_n + (dt x) B_n per channel, output (s . C + D x) silu(z);
 //                        token by token, or for prompts in chunks of 64 tokens side by side
 //   lgs_gated_group_norm out = unit_rms_per_group(y * silu(z)) * w: gating first, the grouped norm on the gated values
 #include "seq_common.h"
@@ -372,8 +372,8 @@ static size_t ssd_lds(int N) {
 }
 
 // ------------------------------------------------------------------------------------------------ channel scan
-// Selective scan with a step size per channel and a diagonal state matrix A (channels x N): nothing is shared between
-// channels but B and C, and the decay exp(dt_c A[c][n]) differs for every (channel, state) pair, so the work is
+// Selective scan with a step size per channel and a diagonal state matrix (channels x N): nothing is shared between
+// channels but B and C, and every (channel, state) pair decays at a rate of its own, so the work is
 // elementwise: L lanes of a wave share one channel, each with NR of its N states in registers, and sum the output
 // with shuffles. Lanes of one wave that hold the same states lie side by side, so that every access to the state, the
 // inputs and the outputs is 64 / L consecutive floats. Tokens are taken kChanBatch at a time: the batch's x, z and step

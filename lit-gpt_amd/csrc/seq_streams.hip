@@ -192,7 +192,7 @@ static bool streams_step_reg(const StreamArgs& p, int T, hipStream_t stream) {
 // One boundary between two sublayers of a layer whose sublayers are normed on the way in AND on the way out.
 // With y0 (the sublayer that ran; up to two branches): b_i = w_i ? y_i / rms(y_i) * w_i : y_i, s = coef * sum_i b_i,
 // x <- x + s / rms(s) * post_w (post_w: the output norm's weight times the layer's per-channel scale; null: no output
-// norm, x <- x + s). With depth_w (a layer's end, average over the depth): this x is the layer's result X_n, kept in row
+// norm, x <- x + s). With depth_w (a layer's end, average over the depth): this x is X_n, what the layer itself produced, kept in row
 // block n of `hist` when there is room, and x <- depth_w[n] X_n + sum_{j < n} depth_w[j] hist[j]. x may be read from
 // another place (x_in) than it is written to. Then with next_w: h = x / rms(x) * next_w, the next sublayer's input (fp32 and / or its bf16 rounding). Every root mean
 // square has eps inside the root. grid (rows); a row lives in registers up to 256 * CPT columns, else it is re-read.

@@ -211,8 +211,8 @@ class MixerSpec:
     softcap: float = 0.0  # attention: scores pass cap * tanh(s / cap) (0: not)
     mask_size: int = 0  # attention: a query sees keys of its own aligned chunk of this many positions (0: all before it)
     window: int = 0  # attention: a query sees the last ``window`` keys up to its own (0: all before it)
-    pool: int = 0  # attention: beside the window, the mean key / value of every aligned block of this many positions that
-    # lies wholly before the window (0: none)
+    pool: int = 0  # attention: beside the window, the mean key / value of every aligned block of this many positions, once
+    # the block's last position has left the window (0: none)
     kv_from: Optional[int] = None  # attention: the layer whose cached keys and values this layer reads
     conv: int = 0  # mamba2: taps of the short convolution
     groups: int = 0  # mamba2: groups of heads that share B and C
@@ -233,7 +233,7 @@ class MixerSpec:
     # | "joint" (all heads of q, and of k, share one root mean square; weights of the whole projection's size)
     rot_layout: str = "half"  # rotary pairs: "half" (i, i + dims / 2) | "interleaved" (2i, 2i + 1)
     rot_values: bool = False  # values are rotated by their position over all vdim dims, outputs turned back by the query's
-    bias: bool = False  # q, k and v have biases ("q.b" / "k.b" / "v.b")
+    bias: bool = False  # biases on the q, k, v projections ("q.b" / "k.b" / "v.b")
     out_gate: bool = False  # the concatenated heads times sigmoid(W_g h), one number per output column ("g")
     sink_kind: str = "learned"  # "none" | "learned" (a scalar per head, "sink") | "one" (a sink of score 0: 1 + sum exp)
     values: str = "own"  # "own" (a value projection) | "keys" (the keys as projected, before their norm)

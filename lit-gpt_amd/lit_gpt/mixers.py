@@ -7,10 +7,11 @@ module's rows of that matrix, ``bind`` tells it where they landed. Outputs are a
 stream ``x`` by the epilogue of the out-projection (or the expert combine), so a layer needs no add kernel.
 
 Mixers here: ``Retention`` (and its preset ``Lightning``: the constant-decay rule on activated projections),
-``LatentAttention``, ``DiffAttention``, ``SelectiveScan`` (Mamba-2 form), ``ChannelScan`` (Mamba form), ``GatedDelta`` (the gated delta rule with a decay per head or
-per head and key channel), ``GatedLinearAttention`` (the gated rule without the correction), ``SinkAttention`` (one-map
-softmax attention: optional biases, q / k norms, rotary positions, a query temperature, a window with pooled blocks
-before it, a learned or constant sink, values that are the keys or are rotated, a gate per head or per column) and ``ParallelMixer`` (two of them side by side on one input projection).
+``LatentAttention``, ``DiffAttention``, ``SelectiveScan`` (Mamba-2 form), ``ChannelScan`` (Mamba form), ``GatedDelta``
+(the gated delta rule with a decay per head or per head and key channel), ``GatedLinearAttention`` (the gated rule without
+the correction), ``SinkAttention`` (one-map softmax attention: optional biases, q / k norms, rotary positions, a query
+temperature, a window with pooled blocks before it, a learned or constant sink, values that are the keys or are rotated, a
+gate per head or per column) and ``ParallelMixer`` (two of them side by side on one input projection).
 
 A step is a packed batch (``StepBatch``): the tokens of all sequences row after row, with per-token cache slot and
 position and per-sequence row range, slot and first position, all int32 on the device. Sizes, decays, scales, rotary
@@ -323,11 +324,12 @@ class SelectiveScan(InputReader):
 
 
 class ChannelScan(InputReader):
-    """Selective scan in the Mamba form. W_in h is [x | z] (``inner`` channels each); x passes a short causal per-channel
-    convolution with bias and silu; W_x x is [step-size inner values (dt_rank) | B | C] (``state`` values each);
-    dt = softplus(W_dt . + bias), one per channel; per channel c and state n
-    S <- exp(-exp(A_log)[c, n] dt_c) S + dt_c x_c B_n, y_c = sum_n S[c, n] C_n + D_c x_c; then y silu(z), projected. The
-    state (S and the convolution's last taps - 1 inputs) is fp32 and lives in a cache slot."""
+    """Selective scan in the Mamba form: every channel has a step size of its own and a diagonal state matrix, so its
+    ``state`` values decay at rates of their own. The input projection gives [u | z] (``inner`` channels each); u passes a
+    short causal per-channel convolution with bias and silu; the map ``x`` of u gives [dt_rank inner values | B | C]
+    (``state`` values each); the step is delta = softplus(map ``dt`` of the inner values + bias). State and output, channel
+    by channel: s_n <- 2^(delta a2_n) s_n + (delta u) B_n with a2 = -exp(A_log) log2(e); out = (s . C + D u) silu(z), then
+    the out-projection. The cache slot holds s and the inputs the convolution still needs, both fp32."""
 
     LOWRANK_ROWS = 8  # steps of up to this many tokens make the step sizes inside the scan's launch
 
@@ -490,7 +492,7 @@ class SinkAttention(InputReader):
     ``rot_layout`` "interleaved": pairs (2i, 2i + 1); ``bias``: biases on q, k and v, added in the shared projection;
     ``rot_values``: values are rotated by their position over all vdim dims (base of the keys' rotation, not rescaled) and
     every output is turned back by the query's position; ``window`` / ``pool``: a position sees the last ``window``
-    tokens, and the mean key and value of every block of ``pool`` tokens that lies wholly before these."""
+    tokens, and the mean key and value of every aligned block of ``pool`` tokens once the last of them has left these."""
 
     def __init__(self, spec: MixerSpec, width: int, eps: float, w: Dict[str, torch.Tensor], device, dtype) -> None:
         super().__init__()
