@@ -83,10 +83,11 @@ int lgs_head_gate(float* o, const float* g, long ldg, int T, int H, int dv, int 
                   const void* w_g2, int rank, int g2_f32, lgs_stream_t stream);
 /* latent attention, per token: c = rmsnorm(kv[t ldkv .. + r]) * norm_w -> cache_c[slot][pos] (bf16, or fp32 with
  * cache_f32); rotary (pairs 2i, 2i + 1) of kv[t ldkv + r .. + dr] -> cache_kr[slot][pos] (fp32); the rotated
- * part of every head's query (at q[t ldq + h (d + dr) + d]) is rotated in place. */
+ * part of every head's query (at q[t ldq + h (d + dr) + d]) is rotated in place; cos and sin times rot_mult. */
 int lgs_latent_prepare(float* q, long ldq, const float* kv, long ldkv, void* cache_c, int cache_f32, float* cache_kr,
                        const float* norm_w, const float* inv_freq, const int* slot, const int* pos, int T, int H,
-                       int d, int dr, int r, int rot_dims, int max_seq, float eps, lgs_stream_t stream);
+                       int d, int dr, int r, int rot_dims, int max_seq, float eps, float rot_mult,
+                       lgs_stream_t stream);
 /* out[t][h] = sum_j p_j c_j over cached rows j <= pos[t] of slot[t] (window > 0: the last `window` of them), p = softmax over
  * (qc[t][h] . c_j + q_rot[t][h] . kr_j) * scale with exp(sink[h]) added to the denominator (sink NULL: none).
  * r <= 1024, dr <= 128. splits > 1 spreads every (token, head)'s keys over that many workgroups (decode: few rows,
@@ -111,9 +112,11 @@ int lgs_moe_route(const float* z, long ld, int T, int E, int top, int* ids, floa
 /* per token: s = softmax(z[t * ld .. + E]) over all E outputs; ids = the top largest of s + bias (bias NULL: of s;
  * lowest index first among equals), wts = s at those places (not renormalised). E <= 256. */
 /* sigmoid != 0: s = sigmoid(z) of every output on its own instead of the softmax. square != 0: wts = s^2 (the weight
- * of an expert whose INPUT is scaled by s when its activation is the square of relu). */
+ * of an expert whose INPUT is scaled by s when its activation is the square of relu). wts are multiplied by scale.
+ * groups > 1: the experts form that many equal groups of neighbours; only those in the `keep` groups with the largest
+ * sums of their two best s + bias can be chosen. */
 int lgs_moe_route_scores(const float* z, long ld, int T, int E, int top, const float* bias, int* ids, float* wts,
-                         int sigmoid, int square, lgs_stream_t stream);
+                         int sigmoid, int square, int groups, int keep, float scale, lgs_stream_t stream);
 /* out[t][i] = act(a[t * ld + i]) * (gate ? sigmoid(gate[t * ldg]) : 1), i < n: the activation of an ungated unit whose
  * up-projection is part of a fused product, with an optional gate of one number per row */
 int lgs_act_rows(const float* a, long ld, const float* gate, long ldg, void* out /* fp32, or bf16 with out_bf16 */,
@@ -121,7 +124,7 @@ int lgs_act_rows(const float* a, long ld, const float* gate, long ldg, void* out
 /* the router product z = w h[t] (w [E][K], fp32 sums) and lgs_moe_route_scores' routing in one launch: the form of
  * steps with few tokens */
 int lgs_moe_router(const float* h, long ldh, const void* w, int w_f32, int T, int K, int E, int top, const float* bias,
-                   int* ids, float* wts, int sigmoid, int square, lgs_stream_t stream);
+                   int* ids, float* wts, int sigmoid, int square, int groups, int keep, float scale, lgs_stream_t stream);
 /* streaming experts: actbuf[t * top + k] = act(up[ids[t][k]] h[t]), or with gated (up holds per expert F gate rows,
  * then F up rows) act(gate h) * (up h); x[t] (+)= sum_k wts[t][k] down[ids[t][k]] actbuf[..]. An id >= n_real names
  * an identity expert without matrices: it is skipped by lgs_moe_up and contributes wts * hin[t] in lgs_moe_down. */
@@ -181,7 +184,7 @@ int lgs_diffattn(const float* q, long ld, const void* cache_k, const void* cache
  * position * inv_freq[i] (rot_dims 0: not), then multiplied by the query temperature
  * 1 + temp_coef * ln(floor((position + 1) / temp_every) + 1) (temp_every 0: 1), in place; every key head at
  * proj[k_off ..] is normed (k_w) and rotated alike on its way to cache_k [slots][max_seq][G][d], the projection
- * itself stays as it is; the values at proj[v_off ..] go to cache_v [slots][max_seq][G][dv] (bf16, or fp32);
+ * itself stays as it is; cos and sin are multiplied by rot_mult; the values at proj[v_off ..] go to cache_v [slots][max_seq][G][dv] (bf16, or fp32);
  * v_off == k_off with dv == d makes the values the keys as projected; v_freq [dv / 2] (NULL: not) rotates the values
  * by their position over all dv dims in the same layout. pool > 0, in steps of one token per sequence only: the
  * workgroup whose token completes block b of pool positions leaves the mean of the block's cached keys and values in
@@ -189,8 +192,8 @@ int lgs_diffattn(const float* q, long ld, const void* cache_k, const void* cache
 int lgs_normattn_prepare(float* proj, long ld, int q_off, int k_off, int v_off, void* cache_k, void* cache_v,
                          int cache_f32, const int* slot, const int* pos, int T, int H, int G, int d, int dv, int max_seq,
                          float eps, float temp_coef, int temp_every, int norm, const float* q_w, const float* k_w,
-                         const float* inv_freq, int rot_dims, int interleaved, const float* v_freq, float* pool_k,
-                         float* pool_v, int pool, int pool_rows, lgs_stream_t stream);
+                         const float* inv_freq, float rot_mult, int rot_dims, int interleaved, const float* v_freq,
+                         float* pool_k, float* pool_v, int pool, int pool_rows, lgs_stream_t stream);
 /* The same means for every block that a step completes (any number of tokens per sequence; runs after the step's keys
  * and values are cached). */
 int lgs_pool_blocks(const void* cache_k, const void* cache_v, int cache_f32, float* pool_k, float* pool_v,
@@ -202,12 +205,14 @@ int lgs_pool_blocks(const void* cache_k, const void* cache_v, int cache_f32, flo
  * lgs_diffattn. gate (NULL: none): head h's output at row t is multiplied by sigmoid(gate[t * ldg + h]) (gate_cols 1)
  * or column by column by sigmoid(gate[t * ldg + h dv + c]) (gate_cols dv). window > 0: position i sees the tokens j with
  * 0 <= i - j < window and, with pool > 0, the pooled blocks b with b pool + pool - 1 <= i - window, in one softmax.
- * v_freq: the output at position i is turned back by i * v_freq[m] (pair m, layout as above) ahead of the gate. */
+ * v_freq: the output at position i is turned back by i * v_freq[m] (pair m, layout as above) ahead of the gate.
+ * score_bias (no sink, no window): sigmoid weights, p_j = sigmoid(cap((q . k_j) * scale) + score_bias[h]), not normalised. */
 int lgs_sinkattn(const float* q, long ld, const void* cache_k, const void* cache_v, int cache_f32, const float* sink,
                  const int* seq_start, const int* seq_slot, const int* seq_pos0, float* out, void* out_bf16, float* part,
                  int splits, int B, int max_len, int H, int G, int d, int dv, int max_seq, int chunk, float scale,
                  float cap, float post, const float* gate, long ldg, int gate_cols, int window, const float* pool_k,
-                 const float* pool_v, int pool, int pool_rows, const float* v_freq, int interleaved, lgs_stream_t stream);
+                 const float* pool_v, int pool, int pool_rows, const float* v_freq, int interleaved, const float* score_bias,
+                 lgs_stream_t stream);
 
 /* ---- gated delta rule ---- */
 /* Per token, on rows qkv [T][ld] = q [G][d] | k [G][d] | v [H][dv] (after their convolution): q and k become unit
@@ -278,6 +283,21 @@ int lgs_channel_scan(const float* x, const float* z, long ldz, const float* bc, 
                      float* state, const int* seq_start, const int* seq_slot, const int* seq_pos0, void* out,
                      int out_bf16, int B, int inner, int N, float* ws, float* wsum, int max_chunks, lgs_stream_t stream);
 
+/* ---- elementwise gated recurrence ---- */
+/* minGRU over a packed batch, channel by channel: gate = sigmoid(z), candidate = u >= 0 ? u + 1/2 : sigmoid(u),
+ * S <- (1 - gate) S + gate candidate, out = S silu(g); z, u, g are columns of rows of ld floats (biases added). state
+ * [slots][n] is read unless a sequence starts at position 0 and left at the step's last token. out [T][n] fp32, or bf16
+ * with out_bf16. ws (B * max_chunks * 2 n floats, max_chunks the 32-token chunks of the longest sequence): the prompt
+ * form, chunks side by side; NULL: token by token. */
+int lgs_mingru(const float* z, const float* u, const float* g, long ld, float* state, const int* seq_start,
+               const int* seq_slot, const int* seq_pos0, void* out, int out_bf16, int B, int n, float* ws, int max_chunks,
+               lgs_stream_t stream);
+/* One token for each of M <= 8 sequences, projections included: row c of the three maps is row z0 + c, u0 + c, g0 + c of
+ * w [rows][K] (bf16 or fp32; bias [rows] or NULL), row m of h and of out [M][n] belongs to sequence m. */
+int lgs_mingru_step(const float* h, long ldh, const void* w, int w_f32, const float* bias, int z0, int u0, int g0, int rows,
+                    int M, int K, int n, float* state, const int* seq_slot, const int* seq_pos0, float* out,
+                    lgs_stream_t stream);
+
 /* ---- boundaries between sublayers ---- */
 /* One boundary between two sublayers of one residual, rows of n values. With y0 (the sublayer that
  * ran; y1: an optional second branch): b_i = w_i ? y_i / rms(y_i) * w_i : y_i, s = coef * (b_0 + b_1),
@@ -285,10 +305,12 @@ int lgs_channel_scan(const float* x, const float* z, long ldz, const float* bc, 
  * scale, NULL: x = x_in + s). With depth_w (n_prev + 1 weights, device; the end of a layer in a design that averages over
  * the depth): hist [hist_rows][rows][n] holds the earlier results X_0 .. X_(n_prev - 1); x is kept there as X_(n_prev)
  * when n_prev < hist_rows, and x = sum_j depth_w[j] X_j goes on. Then with next_w: h = x / rms(x) * next_w, the next
- * sublayer's input, as fp32 (h) and / or rounded to bf16 (h_bf16). */
+ * sublayer's input, as fp32 (h) and / or rounded to bf16 (h_bf16). With add_vec (n values; ahead of a pass over looped
+ * layers; no depth_w): x + add_vec goes on, plus add [rows][n] if given. */
 int lgs_sandwich_step(const float* x_in, float* x, const float* y0, const float* w0, const float* y1, const float* w1,
                       float coef, const float* post_w, const float* next_w, float* h, void* h_bf16, float eps, int rows,
-                      int n, float* hist, const float* depth_w, int n_prev, int hist_rows, lgs_stream_t stream);
+                      int n, float* hist, const float* depth_w, int n_prev, int hist_rows, const float* add,
+                      const float* add_vec, lgs_stream_t stream);
 
 #ifdef __cplusplus
 }

@@ -9,6 +9,8 @@
 // sliding window and 0 without either. Beside a window the one-map form can see pooled blocks: block b stands for the
 // positions b pool .. b pool + pool - 1 by the mean of their cached keys and of their values (fp32, kept next to the
 // cache), and is seen once its last position has left the window; one softmax runs over blocks and tokens together.
+// Sigmoid attention: the one-map form with the weight sigmoid(score + bias of the head) for every visible key, each on
+// its own: no maximum, no normaliser, and partial sums over ranges of keys simply add up.
 //
 //   lgs_diffattn_prepare  per token: rotary (interleaved pairs 2i, 2i + 1 of the first rot_dims dims of every map)
 //                         on the queries in place and on the keys on their way into the cache; values into the cache.
@@ -102,6 +104,7 @@ struct NormPrepArgs {
                            // (of k) divided by one root mean square
   const float *q_w, *k_w;  // optional weights of the two norms: [d], shared by the heads, or (norm 2) [H d] / [G d]
   const float* inv_freq;   // [rot_dims / 2]: rotary positions after the norm
+  float rot_mult;          // factor of cos and sin
   int rot_dims, interleaved;  // pairs (2i, 2i + 1), or (i, i + rot_dims / 2)
   const float* v_freq;     // [dv / 2]: values rotated by their position, in the same layout over dv (null: as they are)
   float *pool_k, *pool_v;  // [slots][pool_rows][G][d], [..][dv]: means of complete blocks of `pool` positions, made here
@@ -174,6 +177,7 @@ __global__ void __launch_bounds__(256) normattn_prepare_kernel(NormPrepArgs p) {
       if (w) u *= w[e], v *= w[f];
       float sn, cs;
       sincosf(fpos * p.inv_freq[i], &sn, &cs);
+      sn *= p.rot_mult, cs *= p.rot_mult;
       const float a = u * cs - v * sn, b = v * cs + u * sn;
       if (isk) {
         cstore<CF32>(p.cache_k, kat + e, a);
@@ -250,6 +254,7 @@ struct AttnArgs {
   int pool, pool_rows;           // (pool 0: none)
   const float* v_freq;  // one map, [dv / 2]: the finished output is turned back by the query's position (values are
   int interleaved;      // cached rotated), pairs (2m, 2m + 1) or (m, m + dv / 2)
+  const float* score_bias;  // [H]: sigmoid weights, each sigmoid(score + score_bias[h]) (null: softmax)
 };
 
 // pooled blocks that the query at position i sees: those wholly before its window
@@ -279,7 +284,7 @@ __device__ __forceinline__ void diff_finish(float a1, float a2, float l1, float 
   }
 }
 
-// one map: o = a / (l + exp(sink - m)) times post, with a and l relative to the running maximum m; `xch` holds dv
+// one map: o = a / (l + exp(sink - m)) times post (sigmoid weights: a itself times post), with a and l relative to the running maximum m; `xch` holds dv
 // floats (outputs that are turned back by the query's position). Called by all 256 threads.
 __device__ __forceinline__ void sink_finish(float a, float m, float l, const AttnArgs& p, size_t row, int h, int pos,
                                             float* xch) {
@@ -291,6 +296,7 @@ __device__ __forceinline__ void sink_finish(float a, float m, float l, const Att
     den = l * w + expf(s - top);
     num = a * w;
   }
+  if (p.score_bias) den = 1.0f;
   float v = c < p.dv ? num / den * p.post : 0.0f;
   if (p.v_freq) {
     __syncthreads();  // (the previous query's exchange is read)
@@ -317,8 +323,8 @@ __device__ __forceinline__ void sink_finish(float a, float m, float l, const Att
 // grid (B * tiles, H, splits). MAPS maps per head (2: differential attention, 1: plain softmax attention with an
 // optional sink). LDS: queries [QT][MAPS d], scores / weights [256][QT MAPS + 4], per (query, map) the running
 // maximum, normaliser and the rescale of the current tile, and the cross-subset sums of the value phase.
-// WIN: a sliding window, optionally with pooled blocks before it (one map).
-template <int QT, int MAPS, bool CF32, bool WIN>
+// WIN: a sliding window, optionally with pooled blocks before it (one map). SIG: sigmoid weights (one map).
+template <int QT, int MAPS, bool CF32, bool WIN, bool SIG>
 __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
   extern __shared__ float lds[];
   __shared__ float red[4];
@@ -355,9 +361,10 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
   }
   for (int i = tid; i < nq * d2; i += 256) qs[i] = p.q[(size_t)(r0 + i / d2) * p.ld + (size_t)h * d2 + i % d2];
   if (tid < NR) {
-    mrow[tid] = -INFINITY;
+    mrow[tid] = SIG ? 0.0f : -INFINITY;
     lrow[tid] = 0.0f;
   }
+  const float bias = SIG ? p.score_bias[h] : 0.0f;
   // value phase: thread owns column `col` and every KS-th key of a tile, starting at `ks`
   int ncol = 64;
   while (ncol < dv) ncol <<= 1;  // dv <= 256
@@ -430,13 +437,14 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
         for (int m = 0; m < MAPS; ++m) {
           float v = s[i][m] * p.scale;
           if (p.cap > 0.0f) v = p.cap * tanhf(v / p.cap);
-          sc[tid * SCS + MAPS * i + m] = see ? v : -INFINITY;
+          if (SIG) sc[tid * SCS + MAPS * i + m] = see ? sigmoid_f(v + bias) : 0.0f;
+          else sc[tid * SCS + MAPS * i + m] = see ? v : -INFINITY;
         }
       }
     }
     __syncthreads();
     // ---- online softmax: wave w owns rows w, w + 4, ... of the (query, map) rows
-    for (int r = wave; r < NR; r += 4) {
+    for (int r = wave; r < NR && !SIG; r += 4) {
       float* srow = sc + r;
       float v[4], mx = -INFINITY;
 #pragma unroll
@@ -461,13 +469,13 @@ __global__ void __launch_bounds__(256) diffattn_kernel(AttnArgs p) {
         mrow[r] = mn;
       }
     }
-    __syncthreads();
+    if (!SIG) __syncthreads();
     // ---- weighted sums of the values
     {
 #pragma unroll
       for (int i = 0; i < QT; ++i)
 #pragma unroll
-        for (int m = 0; m < MAPS; ++m) acc[i][m] *= arow[MAPS * i + m];
+        for (int m = 0; m < MAPS && !SIG; ++m) acc[i][m] *= arow[MAPS * i + m];
       if (col < dv) {
         auto add = [&](const int j, const float v) {
           float w[NR];
@@ -583,9 +591,11 @@ static size_t diffattn_lds(int d) {
 template <int QT, int MAPS>
 static int diffattn_launch(const AttnArgs& p, int cache_f32, dim3 grid, hipStream_t stream) {
   const size_t lds = diffattn_lds<QT, MAPS>(p.d);
-  auto* fn = cache_f32 ? diffattn_kernel<QT, MAPS, true, false> : diffattn_kernel<QT, MAPS, false, false>;
+  auto* fn = cache_f32 ? diffattn_kernel<QT, MAPS, true, false, false> : diffattn_kernel<QT, MAPS, false, false, false>;
   if (MAPS == 1 && p.window > 0)
-    fn = cache_f32 ? diffattn_kernel<QT, MAPS, true, MAPS == 1> : diffattn_kernel<QT, MAPS, false, MAPS == 1>;
+    fn = cache_f32 ? diffattn_kernel<QT, MAPS, true, MAPS == 1, false> : diffattn_kernel<QT, MAPS, false, MAPS == 1, false>;
+  else if (MAPS == 1 && p.score_bias)
+    fn = cache_f32 ? diffattn_kernel<QT, MAPS, true, false, MAPS == 1> : diffattn_kernel<QT, MAPS, false, false, MAPS == 1>;
   if (lds > 48 * 1024) {
     const hipError_t e = hipFuncSetAttribute((const void*)fn, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) {
@@ -646,8 +656,8 @@ extern "C" int lgs_diffattn(const float* q, long ld, const void* cache_k, const 
 extern "C" int lgs_normattn_prepare(float* proj, long ld, int q_off, int k_off, int v_off, void* cache_k, void* cache_v,
                                     int cache_f32, const int* slot, const int* pos, int T, int H, int G, int d, int dv,
                                     int max_seq, float eps, float temp_coef, int temp_every, int norm, const float* q_w,
-                                    const float* k_w, const float* inv_freq, int rot_dims, int interleaved,
-                                    const float* v_freq, float* pool_k, float* pool_v, int pool, int pool_rows,
+                                    const float* k_w, const float* inv_freq, float rot_mult, int rot_dims,
+                                    int interleaved, const float* v_freq, float* pool_k, float* pool_v, int pool, int pool_rows,
                                     hipStream_t stream) {
   LGA_CHECK_ARG(proj && slot && pos && cache_k && cache_v && T > 0 && max_seq > 0, "lgs_normattn_prepare: bad arguments");
   LGA_CHECK_ARG(H > 0 && G > 0 && H % G == 0 && d > 0 && dv > 0 && temp_every >= 0 && norm >= 0 && norm <= 2,
@@ -660,7 +670,7 @@ extern "C" int lgs_normattn_prepare(float* proj, long ld, int q_off, int k_off, 
   LGA_CHECK_ARG(!v_freq || dv % 2 == 0, "lgs_normattn_prepare: rotated values have an even size");
   LGA_CHECK_ARG(pool >= 0 && (pool == 0 || (pool_k && pool_v && pool_rows > 0)), "lgs_normattn_prepare: pooled blocks");
   lgs::NormPrepArgs p{proj, ld, q_off, k_off, v_off, cache_k, cache_v, slot, pos, H, G, d, dv, max_seq, temp_every, eps,
-                      temp_coef, norm, q_w, k_w, inv_freq, rot_dims, interleaved ? 1 : 0, v_freq, pool_k, pool_v, pool,
+                      temp_coef, norm, q_w, k_w, inv_freq, rot_mult, rot_dims, interleaved ? 1 : 0, v_freq, pool_k, pool_v, pool,
                       pool_rows};
   if (cache_f32) lgs::normattn_prepare_kernel<true><<<T, 256, 0, stream>>>(p);
   else lgs::normattn_prepare_kernel<false><<<T, 256, 0, stream>>>(p);
@@ -685,7 +695,7 @@ extern "C" int lgs_sinkattn(const float* q, long ld, const void* cache_k, const 
                             void* out_bf16, float* part, int splits, int B, int max_len, int H, int G, int d, int dv,
                             int max_seq, int chunk, float scale, float cap, float post, const float* gate, long ldg,
                             int gate_cols, int window, const float* pool_k, const float* pool_v, int pool, int pool_rows,
-                            const float* v_freq, int interleaved, hipStream_t stream) {
+                            const float* v_freq, int interleaved, const float* score_bias, hipStream_t stream) {
   LGA_CHECK_ARG(q && cache_k && cache_v && seq_start && seq_slot && seq_pos0 && out, "lgs_sinkattn: null pointer");
   LGA_CHECK_ARG(!gate || ((gate_cols == 1 && ldg >= H) || (gate_cols == dv && ldg >= (long)H * dv)),
                 "lgs_sinkattn: gates per head or per output column, and their row stride");
@@ -696,11 +706,12 @@ extern "C" int lgs_sinkattn(const float* q, long ld, const void* cache_k, const 
   LGA_CHECK_ARG(pool >= 0 && (pool == 0 || (window > 0 && pool_k && pool_v && pool_rows > 0)),
                 "lgs_sinkattn: pooled blocks stand before a window");
   LGA_CHECK_ARG(!v_freq || dv % 2 == 0, "lgs_sinkattn: rotated values have an even size");
+  LGA_CHECK_ARG(!score_bias || (!sink && window == 0), "lgs_sinkattn: sigmoid weights have no sink and no window");
   LGA_CHECK_ARG(splits >= 1 && splits <= 64 && (splits == 1 || (part && max_len == 1)),
                 "lgs_sinkattn: splits need one token per sequence and a workspace");
   lgs::AttnArgs p{q, ld, cache_k, cache_v, seq_start, seq_slot, seq_pos0, out, (uint16_t*)out_bf16, part,
                   H, G, d, dv, max_seq, chunk, 0, scale, cap, 0.0f, 0.0f, post, sink, gate, ldg, gate_cols, window,
-                  pool_k, pool_v, pool, pool_rows, v_freq, interleaved ? 1 : 0};
+                  pool_k, pool_v, pool, pool_rows, v_freq, interleaved ? 1 : 0, score_bias};
   int rc;
   if (max_len == 1) {
     p.tiles = 1;

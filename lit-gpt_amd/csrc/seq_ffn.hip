@@ -6,7 +6,9 @@
 //                        softmax over just those
 //   lgs_moe_route_scores per token: softmax over all router outputs (or the sigmoid of each on its own); the choice
 //                        adds a stored correction to the scores, the weights are the chosen scores themselves (or
-//                        their squares: a score on the input of an expert with a relu^2 activation)
+//                        their squares: a score on the input of an expert with a relu^2 activation) times a constant.
+//                        Optionally the choice goes over groups of neighbouring experts first: a group is worth the
+//                        sum of its two largest choice scores, and only the best groups' experts can be chosen
 //   lgs_act_rows         out = act(a) times an optional sigmoid gate of one number per row (an ungated unit whose
 //                        up-projection is part of a fused product: the shared expert)
 //   lgs_moe_up / _down   the routed experts as streaming GEMVs over (token, choice) pairs: only the chosen experts'
@@ -126,10 +128,14 @@ __global__ void __launch_bounds__(64) moe_route_kernel(const float* __restrict__
 // one wave: s = softmax(z) over all E outputs (z: the token's router logits, global or LDS), or with `sigmoid`
 // s = sigmoid(z) of every output on its own; the `top` largest of s + bias (lowest index first among equals) are
 // chosen, and their weights are s itself: not renormalised, without the bias; `square`: s^2 (the weight of an expert
-// whose INPUT is scaled by s when its activation is the square of relu: relu(s a)^2 = s^2 relu(a)^2 for s > 0)
+// whose INPUT is scaled by s when its activation is the square of relu: relu(s a)^2 = s^2 relu(a)^2 for s > 0); all
+// weights times wscale. groups > 1: the experts form that many equal groups of neighbours, and those outside the `keep`
+// groups with the largest sums of their two best choice scores (one, if groups have a single expert; the lower group
+// first among equals) cannot be chosen; `gl` then holds 512 floats of LDS that this wave has to itself.
 __device__ __forceinline__ void route_scores_wave(const float* z, int E, int top, const float* __restrict__ bias,
                                                   int* __restrict__ ids, float* __restrict__ wts, int lane,
-                                                  bool sigmoid = false, bool square = false) {
+                                                  bool sigmoid, bool square, int groups, int keep, float wscale,
+                                                  float* gl) {
   float s[4], c[4], mx = -INFINITY;
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
@@ -150,6 +156,35 @@ __device__ __forceinline__ void route_scores_wave(const float* z, int E, int top
     const int i = lane + 64 * e;
     s[e] /= den;
     c[e] = i < E ? s[e] + (bias ? bias[i] : 0.0f) : -INFINITY;
+  }
+  if (groups > 1 && keep < groups) {
+    float* cs = gl;         // choice scores
+    float* gv = gl + 256;   // what the groups are worth
+    const int per = E / groups;
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (lane + 64 * e < E) cs[lane + 64 * e] = c[e];
+    __threadfence_block();  // (one wave: its LDS accesses stay in order)
+    for (int g = lane; g < groups; g += 64) {
+      float a = -INFINITY, b = -INFINITY;
+      for (int j = g * per; j < (g + 1) * per; ++j) {
+        const float v = cs[j];
+        b = fmaxf(b, fminf(a, v));
+        a = fmaxf(a, v);
+      }
+      gv[g] = per > 1 ? a + b : a;
+    }
+    __threadfence_block();
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = lane + 64 * e;
+      if (i >= E) continue;
+      const int g = i / per;
+      const float v = gv[g];
+      int better = 0;
+      for (int o = 0; o < groups; ++o) better += gv[o] > v || (gv[o] == v && o < g);
+      if (better >= keep) c[e] = -INFINITY;
+    }
   }
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY, bs = 0.0f;
@@ -175,7 +210,7 @@ __device__ __forceinline__ void route_scores_wave(const float* z, int E, int top
     }
     if (lane == 0) {
       ids[k] = bi;
-      wts[k] = square ? bs * bs : bs;
+      wts[k] = (square ? bs * bs : bs) * wscale;
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e)
@@ -185,9 +220,12 @@ __device__ __forceinline__ void route_scores_wave(const float* z, int E, int top
 
 __global__ void __launch_bounds__(64) moe_route_scores_kernel(const float* __restrict__ z, long ld, int E, int top,
                                                               const float* __restrict__ bias, int* __restrict__ ids,
-                                                              float* __restrict__ wts, int sigmoid, int square) {
+                                                              float* __restrict__ wts, int sigmoid, int square,
+                                                              int groups, int keep, float wscale) {
+  __shared__ float gl[512];
   const size_t t = blockIdx.x;
-  route_scores_wave(z + t * ld, E, top, bias, ids + t * top, wts + t * top, threadIdx.x, sigmoid != 0, square != 0);
+  route_scores_wave(z + t * ld, E, top, bias, ids + t * top, wts + t * top, threadIdx.x, sigmoid != 0, square != 0, groups,
+                    keep, wscale, gl);
 }
 
 // grid (T, ceil(n / 256)): out[t][i] = act(a[t * ld + i]) * (gate ? sigmoid(gate[t * ldg]) : 1): the activation of an
@@ -212,8 +250,9 @@ template <bool WF32>
 __global__ void __launch_bounds__(1024) moe_router_kernel(const float* __restrict__ h, long ldh, const void* __restrict__ w,
                                                           int K, int E, int top, const float* __restrict__ bias,
                                                           int* __restrict__ ids, float* __restrict__ wts, int sigmoid,
-                                                          int square) {
+                                                          int square, int groups, int keep, float wscale) {
   __shared__ float z[256];
+  __shared__ float gl[512];
   const size_t t = blockIdx.x;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const float* x = h + t * ldh;
@@ -224,7 +263,8 @@ __global__ void __launch_bounds__(1024) moe_router_kernel(const float* __restric
     if (lane == 0) z[e] = a0;
   }
   __syncthreads();
-  if (wave == 0) route_scores_wave(z, E, top, bias, ids + t * top, wts + t * top, lane, sigmoid != 0, square != 0);
+  if (wave == 0)
+    route_scores_wave(z, E, top, bias, ids + t * top, wts + t * top, lane, sigmoid != 0, square != 0, groups, keep, wscale, gl);
 }
 
 // grid (ceil(F / 8), pairs): pair = token * top + choice; act[pair][f] = act(up_e[f] . h_token); GATED: an expert's
@@ -424,11 +464,15 @@ extern "C" int lgs_moe_route(const float* z, long ld, int T, int E, int top, int
 }
 
 extern "C" int lgs_moe_route_scores(const float* z, long ld, int T, int E, int top, const float* bias, int* ids,
-                                    float* wts, int sigmoid, int square, hipStream_t stream) {
+                                    float* wts, int sigmoid, int square, int groups, int keep, float scale,
+                                    hipStream_t stream) {
   LGA_CHECK_ARG(z && ids && wts && T > 0, "lgs_moe_route_scores: bad arguments");
+  LGA_CHECK_ARG(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (E / groups),
+                "lgs_moe_route_scores: equal groups of experts, and enough experts in those kept");
   LGA_CHECK_ARG(E > 0 && E <= 256 && top > 0 && top <= E,
                 "lgs_moe_route_scores: experts must be <= 256 and top <= experts");
-  lgs::moe_route_scores_kernel<<<T, 64, 0, stream>>>(z, ld, E, top, bias, ids, wts, sigmoid, square);
+  lgs::moe_route_scores_kernel<<<T, 64, 0, stream>>>(z, ld, E, top, bias, ids, wts, sigmoid, square, groups, keep,
+                                                      scale);
   LGA_LAUNCH_RETURN();
 }
 
@@ -442,11 +486,18 @@ extern "C" int lgs_act_rows(const float* a, long ld, const float* gate, long ldg
 }
 
 extern "C" int lgs_moe_router(const float* h, long ldh, const void* w, int w_f32, int T, int K, int E, int top,
-                              const float* bias, int* ids, float* wts, int sigmoid, int square, hipStream_t stream) {
+                              const float* bias, int* ids, float* wts, int sigmoid, int square, int groups, int keep,
+                              float scale, hipStream_t stream) {
+  LGA_CHECK_ARG(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (E / groups),
+                "lgs_moe_router: equal groups of experts, and enough experts in those kept");
   LGA_CHECK_ARG(h && w && ids && wts && T > 0 && K > 0 && ldh >= K, "lgs_moe_router: bad arguments");
   LGA_CHECK_ARG(E > 0 && E <= 256 && top > 0 && top <= E, "lgs_moe_router: experts must be <= 256 and top <= experts");
-  if (w_f32) lgs::moe_router_kernel<true><<<T, 1024, 0, stream>>>(h, ldh, w, K, E, top, bias, ids, wts, sigmoid, square);
-  else lgs::moe_router_kernel<false><<<T, 1024, 0, stream>>>(h, ldh, w, K, E, top, bias, ids, wts, sigmoid, square);
+  if (w_f32)
+    lgs::moe_router_kernel<true><<<T, 1024, 0, stream>>>(h, ldh, w, K, E, top, bias, ids, wts, sigmoid, square, groups, keep,
+                                                         scale);
+  else
+    lgs::moe_router_kernel<false><<<T, 1024, 0, stream>>>(h, ldh, w, K, E, top, bias, ids, wts, sigmoid, square, groups, keep,
+                                                          scale);
   LGA_LAUNCH_RETURN();
 }
 

@@ -6,7 +6,8 @@
 //   lgs_head_gate        per head: optional unit RMS of o, times act(g): the retention's output norm + silu gate and
 //                        the latent attention's sigmoid gate
 //   lgs_latent_prepare   latent attention, per token: RMS-normed latent c and the rotated shared key part go to the
-//                        cache rows (slot, position); the queries' rotated parts are rotated in place (interleaved)
+//                        cache rows (slot, position); the queries' rotated parts are rotated in place (interleaved;
+//                        cos and sin optionally times a constant)
 //   lgs_latent_attention softmax attention in the latent space (over all rows so far or a window of them): every head's query has been mapped through its key
 //                        up-projection, so all heads read the same cached rows [c | k_rot]; scores, the sink's
 //                        share of the denominator and the weighted sum of c are fp32; the value up-projection
@@ -360,6 +361,7 @@ struct LatPrepArgs {
   const int* pos;         // [T]
   int H, d, dr, r, rot_dims, max_seq;
   float eps;
+  float rot_mult;  // factor of cos and sin
 };
 
 template <bool CF32>
@@ -387,6 +389,7 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(LatPrepArgs p) {
     else if ((i & 1) == 0) {
       float sn, cs;
       sincosf(fpos * p.inv_freq[i >> 1], &sn, &cs);
+      sn *= p.rot_mult, cs *= p.rot_mult;
       const float u = kv[p.r + i], v = kv[p.r + i + 1];
       kro[i] = u * cs - v * sn;
       kro[i + 1] = v * cs + u * sn;
@@ -397,6 +400,7 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(LatPrepArgs p) {
     float* qr = p.q + (size_t)t * p.ldq + (size_t)h * (p.d + p.dr) + p.d + 2 * i;
     float sn, cs;
     sincosf(fpos * p.inv_freq[i], &sn, &cs);
+    sn *= p.rot_mult, cs *= p.rot_mult;
     const float u = qr[0], v = qr[1];
     qr[0] = u * cs - v * sn;
     qr[1] = v * cs + u * sn;
@@ -906,14 +910,14 @@ extern "C" int lgs_head_gate(float* o, const float* g, long ldg, int T, int H, i
 extern "C" int lgs_latent_prepare(float* q, long ldq, const float* kv, long ldkv, void* cache_c, int cache_f32,
                                   float* cache_kr, const float* norm_w, const float* inv_freq, const int* slot,
                                   const int* pos, int T, int H, int d, int dr, int r, int rot_dims, int max_seq,
-                                  float eps, hipStream_t stream) {
+                                  float eps, float rot_mult, hipStream_t stream) {
   LGA_CHECK_ARG(q && kv && cache_c && cache_kr && norm_w && slot && pos, "lgs_latent_prepare: null pointer");
   LGA_CHECK_ARG(T > 0 && H > 0 && d >= 0 && dr >= 0 && r > 0 && max_seq > 0, "lgs_latent_prepare: bad sizes");
   LGA_CHECK_ARG(ldq >= (long)H * (d + dr) && ldkv >= (long)r + dr, "lgs_latent_prepare: rows shorter than their parts");
   LGA_CHECK_ARG(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dr && (rot_dims == 0 || inv_freq),
                 "lgs_latent_prepare: bad rotary dims");
   lgs::LatPrepArgs p{q, ldq, kv, ldkv, cache_c, cache_kr, norm_w, inv_freq, slot, pos,
-                     H, d, dr, r, rot_dims, max_seq, eps};
+                     H, d, dr, r, rot_dims, max_seq, eps, rot_mult};
   if (cache_f32) lgs::latent_prepare_kernel<true><<<T, 256, 0, stream>>>(p);
   else lgs::latent_prepare_kernel<false><<<T, 256, 0, stream>>>(p);
   LGA_LAUNCH_RETURN();

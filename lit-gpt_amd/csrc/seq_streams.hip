@@ -9,8 +9,9 @@
 //                       followed by the read + norm of the next one (optional), so the streams are read once
 //   lgs_sandwich_step   the boundary of layers with one residual whose sublayers are normed on the way in (and
 //                       optionally out): the norms and the average of up to two branch outputs, the output norm times
-//                       the layer scale, the residual add, a learned average over the depth at a layer's end, and the
-//                       next sublayer's input norm in one launch
+//                       the layer scale, the residual add, a learned average over the depth at a layer's end or what
+//                       joins the residual ahead of a pass over looped layers, and the next sublayer's input norm in
+//                       one launch
 #include "seq_common.h"
 
 namespace lgs {
@@ -194,7 +195,8 @@ static bool streams_step_reg(const StreamArgs& p, int T, hipStream_t stream) {
 // x <- x + s / rms(s) * post_w (post_w: the output norm's weight times the layer's per-channel scale; null: no output
 // norm, x <- x + s). With depth_w (a layer's end, average over the depth): this x is X_n, what the layer itself produced, kept in row
 // block n of `hist` when there is room, and x <- depth_w[n] X_n + sum_{j < n} depth_w[j] hist[j]. x may be read from
-// another place (x_in) than it is written to. Then with next_w: h = x / rms(x) * next_w, the next sublayer's input (fp32 and / or its bf16 rounding). Every root mean
+// another place (x_in) than it is written to. With add_vec (ahead of a pass over looped layers): x <- x + add_vec + add (a
+// row of its own, if given). Then with next_w: h = x / rms(x) * next_w, the next sublayer's input (fp32 and / or its bf16 rounding). Every root mean
 // square has eps inside the root. grid (rows); a row lives in registers up to 256 * CPT columns, else it is re-read.
 struct SandwichArgs {
   const float* x_in;
@@ -210,6 +212,8 @@ struct SandwichArgs {
   float* hist;  // [hist_rows][rows][n]: X_0, X_1, ...
   const float* depth_w;
   int n_prev, hist_rows;
+  const float* add_vec;  // [n]
+  const float* add;      // [rows][n] or null
 };
 
 // sums of two values over the 256 threads of a workgroup at once (`red` holds 8 floats)
@@ -226,7 +230,7 @@ __device__ __forceinline__ void block_sum2_256(float& u, float& v, float* red) {
   v = (red[4] + red[5]) + (red[6] + red[7]);
 }
 
-template <int CPT, bool DEPTH>
+template <int CPT, bool DEPTH, bool PASS>
 __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
   __shared__ float red[8];
   const size_t r = blockIdx.x;
@@ -236,7 +240,7 @@ __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
   const float inv_n = 1.0f / (float)n;
   // every operand of the registers' share of the row is fetched up front, so that the reductions below wait for
   // one batch of loads only
-  float xv[CPT], av[CPT], bv[CPT], w0[CPT], w1[CPT], wp[CPT], wn[CPT];
+  float xv[CPT], av[CPT], bv[CPT], w0[CPT], w1[CPT], wp[CPT], wn[CPT], pv[PASS ? CPT : 1];
   const float *a = p.y0 ? p.y0 + r * n : nullptr, *b = p.y1 ? p.y1 + r * n : nullptr;
 #pragma unroll
   for (int e = 0; e < CPT; ++e) {
@@ -249,6 +253,10 @@ __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
     w1[e] = (b && p.w1 && in) ? p.w1[i] : 1.0f;
     wp[e] = (p.post_w && in) ? p.post_w[i] : 0.0f;
     wn[e] = (p.next_w && in) ? p.next_w[i] : 0.0f;
+    if (PASS) {
+      pv[e] = in ? p.add_vec[i] : 0.0f;
+      if (p.add && in) pv[e] += p.add[r * n + i];
+    }
   }
   // the earlier layers' share of the average needs nothing of this sublayer: its loads run beside the reductions
   const size_t hs = (size_t)gridDim.x * n;
@@ -317,7 +325,7 @@ __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
       const int i = tid + 256 * e;
       if (i < n) {
         xv[e] = p.post_w ? fmaf(av[e] * rs, wp[e], xv[e]) : xv[e] + av[e];
-        if (!DEPTH) xr[i] = xv[e];
+        if (!DEPTH && !PASS) xr[i] = xv[e];
       }
     }
     for (int i = tid + 256 * CPT; i < n; i += 256) {
@@ -345,11 +353,25 @@ __global__ void __launch_bounds__(256) sandwich_step_kernel(SandwichArgs p) {
       xr[i] = fmaf(cn, x, v);
     }
   }
+  if (PASS) {
+#pragma unroll
+    for (int e = 0; e < CPT; ++e) {
+      const int i = tid + 256 * e;
+      if (i < n) {
+        xv[e] += pv[e];
+        xr[i] = xv[e];
+      }
+    }
+    for (int i = tid + 256 * CPT; i < n; i += 256) {
+      const float x = a ? xr[i] : xi[i];  // (a: written by this thread above)
+      xr[i] = x + (p.add_vec[i] + (p.add ? p.add[r * n + i] : 0.0f));
+    }
+  }
   if (!p.next_w) return;
   float sx = 0.0f;
 #pragma unroll
   for (int e = 0; e < CPT; ++e) sx = fmaf(xv[e], xv[e], sx);
-  const float* xs = (a || DEPTH) ? xr : xi;  // (xr: written by this thread above)
+  const float* xs = (a || DEPTH || PASS) ? xr : xi;  // (xr: written by this thread above)
   for (int i = tid + 256 * CPT; i < n; i += 256) sx = fmaf(xs[i], xs[i], sx);
   const float rx = 1.0f / sqrtf(block_sum_256(sx, red) * inv_n + p.eps);
 #pragma unroll
@@ -401,19 +423,21 @@ extern "C" int lgs_streams_step(float* x, const float* y, const float* mix, cons
 extern "C" int lgs_sandwich_step(const float* x_in, float* x, const float* y0, const float* w0, const float* y1,
                                  const float* w1, float coef, const float* post_w, const float* next_w, float* h,
                                  void* h_bf16, float eps, int rows, int n, float* hist, const float* depth_w, int n_prev,
-                                 int hist_rows, hipStream_t stream) {
+                                 int hist_rows, const float* add, const float* add_vec, hipStream_t stream) {
   LGA_CHECK_ARG(x && rows > 0 && n > 0, "lgs_sandwich_step: bad arguments");
   LGA_CHECK_ARG(y0 || !y1, "lgs_sandwich_step: a second branch without a first");
-  LGA_CHECK_ARG(y0 || next_w || depth_w, "lgs_sandwich_step: nothing to do");
+  LGA_CHECK_ARG(y0 || next_w || depth_w || add_vec, "lgs_sandwich_step: nothing to do");
+  LGA_CHECK_ARG(add_vec ? !depth_w : !add, "lgs_sandwich_step: a pass's vector (without an average over the depth), or no row");
   LGA_CHECK_ARG(!next_w || h || h_bf16, "lgs_sandwich_step: the next input needs a place");
   LGA_CHECK_ARG(!depth_w || (hist && n_prev >= 1 && n_prev <= hist_rows),
                 "lgs_sandwich_step: the average over the depth needs the earlier results");
   lgs::SandwichArgs p{x_in ? x_in : x, x, y0, w0, y1, w1, coef, post_w, next_w, h, (uint16_t*)h_bf16, eps, n,
-                      hist, depth_w, n_prev, hist_rows};
-#define LGS_SANDWICH(CPT)                                                              \
-  do {                                                                                 \
-    if (depth_w) lgs::sandwich_step_kernel<CPT, true><<<rows, 256, 0, stream>>>(p);    \
-    else lgs::sandwich_step_kernel<CPT, false><<<rows, 256, 0, stream>>>(p);           \
+                      hist, depth_w, n_prev, hist_rows, add_vec, add};
+#define LGS_SANDWICH(CPT)                                                                      \
+  do {                                                                                         \
+    if (depth_w) lgs::sandwich_step_kernel<CPT, true, false><<<rows, 256, 0, stream>>>(p);     \
+    else if (add_vec) lgs::sandwich_step_kernel<CPT, false, true><<<rows, 256, 0, stream>>>(p); \
+    else lgs::sandwich_step_kernel<CPT, false, false><<<rows, 256, 0, stream>>>(p);            \
   } while (0)
   if (n <= 1024) LGS_SANDWICH(4);
   else if (n <= 2048) LGS_SANDWICH(8);

@@ -174,7 +174,9 @@ class RotarySpec:
     # rescaling of the frequencies for longer contexts. Keys: factor alone: every frequency is divided by it (linear
     # scaling). factor, low, high, original: band by band, wavelengths above original / low are slowed down by
     # ``factor``, those below original / high are kept, the band between blends the two linearly in
-    # original / wavelength.
+    # original / wavelength. factor, fast, slow, original (YaRN): pair by pair, the pairs that turn more than ``fast``
+    # times over ``original`` positions are kept, those that turn less than ``slow`` times are divided by ``factor``, the
+    # indices between blend linearly; cos and sin are multiplied by ``mult``.
     scaling: Optional[Dict[str, float]] = None
 
     def inv_freq(self) -> List[float]:
@@ -183,6 +185,14 @@ class RotarySpec:
         out = [float(self.base) ** (-2.0 * i / self.dims) for i in range(self.dims // 2)]
         if self.scaling and "original" not in self.scaling:
             return [f / float(self.scaling["factor"]) for f in out]
+        if self.scaling and "fast" in self.scaling:
+            lo = max(math.floor(self._pair_that_turns(float(self.scaling["fast"]))), 0)
+            hi = min(math.ceil(self._pair_that_turns(float(self.scaling["slow"]))), self.dims - 1)
+            factor = float(self.scaling["factor"])
+            for i, f in enumerate(out):
+                ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+                out[i] = f * (ramp / factor + (1.0 - ramp))
+            return out
         if self.scaling:
             factor, low, high, orig = (float(self.scaling[k]) for k in ("factor", "low", "high", "original"))
             for i, f in enumerate(out):
@@ -193,6 +203,15 @@ class RotarySpec:
                     mix = (orig / wavelength - low) / (high - low)
                     out[i] = (1.0 - mix) * f / factor + mix * f
         return out
+
+    def _pair_that_turns(self, times: float) -> float:
+        """The (fractional) pair index that makes ``times`` full turns over ``original`` positions."""
+        return self.dims * math.log(float(self.scaling["original"]) / (2.0 * math.pi * times)) / (2.0 * math.log(self.base))
+
+    @property
+    def mult(self) -> float:
+        """Factor of cos and sin (1 unless the scaling is YaRN's)."""
+        return 0.1 * math.log(float(self.scaling["factor"])) + 1.0 if self.scaling and "fast" in self.scaling else 1.0
 
 
 @dataclass
@@ -234,13 +253,16 @@ class MixerSpec:
     rot_layout: str = "half"  # rotary pairs: "half" (i, i + dims / 2) | "interleaved" (2i, 2i + 1)
     rot_values: bool = False  # values are rotated by their position over all vdim dims, outputs turned back by the query's
     bias: bool = False  # biases on the q, k, v projections ("q.b" / "k.b" / "v.b")
-    out_gate: bool = False  # the concatenated heads times sigmoid(W_g h), one number per output column ("g")
+    out_gate: bool = False  # the concatenated heads times sigmoid(W_g h), one number per output column ("g"; latent
+    # attention too)
     sink_kind: str = "learned"  # "none" | "learned" (a scalar per head, "sink") | "one" (a sink of score 0: 1 + sum exp)
     values: str = "own"  # "own" (a value projection) | "keys" (the keys as projected, before their norm)
+    weights: str = "softmax"  # "softmax" | "sigmoid" (every visible key weighs sigmoid(score + bias of the head, "pb"), no
+    # normaliser)
     head_gate: bool = False  # every head's output times sigmoid(W_g h)_h, one number per head ("g")
     tau: float = 0.0  # gated_linear: the decay is sigmoid(z)^(1 / tau)
     q_rank: int = 0  # latent attention: queries come from a normed latent of this size (0: straight from the input)
-    inner: int = 0  # mamba: channels
+    inner: int = 0  # mamba, mingru: channels
     dt_rank: int = 0  # mamba: inner size of the low-rank step-size map
 
 
@@ -252,6 +274,9 @@ class FeedForwardSpec:
     top: int = 0
     limit: float = 0.0  # clamped gated unit: bound of the gate (from above) and of the up branch (both sides)
     identity: int = 0  # moe: router outputs beyond ``experts`` that stand for identity experts (output = input)
+    groups: int = 1  # moe: equal groups of neighbouring experts, of which the best ``keep`` can be chosen from
+    keep: int = 1
+    route_scale: float = 1.0  # moe: factor of the chosen experts' weights
     shared_ff: int = 0  # moe: size of a shared expert that runs for every token behind a sigmoid gate (0: none)
 
 
@@ -270,12 +295,14 @@ class LayerSpec:
 # "pooled_attention": biased rotary softmax attention over a window of tokens and the pooled blocks before it, a learned
 # sink, an elementwise output gate; "rotated_value_attention": windowed rotary softmax attention with jointly normed
 # queries and keys and rotated values; "mamba": selective scan with a diagonal state matrix per channel;
+# "sigmoid_attention": biased rotary attention whose values are the keys as projected and whose weights are sigmoids of the
+# scores, not normalised; "mingru": an elementwise gated recurrence whose gates read the token alone;
 # "parallel": two of these side by side (which two, the design says)
 MIXER_KINDS = ("retention", "latent_attention", "attention", "mamba2", "channel_delta", "gated_delta",
                "sink_attention", "parallel", "rotary_attention", "key_value_attention", "gated_linear", "lightning",
-               "pooled_attention", "rotated_value_attention", "mamba")
+               "pooled_attention", "rotated_value_attention", "mamba", "sigmoid_attention", "mingru")
 SOFTMAX_KINDS = ("sink_attention", "rotary_attention", "key_value_attention", "pooled_attention",
-                 "rotated_value_attention")
+                 "rotated_value_attention", "sigmoid_attention")  # (the one-map attentions over a HeadKVCache)
 
 
 @dataclass(frozen=True)
@@ -300,12 +327,19 @@ class LayeredDesign:
     # scores as they are, gated experts W_down(silu(W_gate h) * W_up h), optional identity experts
     # "sigmoid": scores = sigmoid of every router output, the largest chosen, the score scales the expert's INPUT,
     # experts W_down relu(W_up h)^2, optional shared expert behind a sigmoid gate per token
+    # "group_scores": sigmoid scores + a stored correction for the choice, which goes over the best groups of neighbouring
+    # experts first; weights = the chosen scores times a constant, gated experts as with "scores"
     moe: str = "top_logits"
     mask: str = "chunk"  # what a mixer's mask.size means: "chunk" (aligned chunks) or "window" (the last size positions)
     # after every layer the residual becomes a learned average over the embedding output and all layers' results so far
     # (weights "<layer>.dwa")
     depth_average: bool = False
     latent_sink: bool = True  # latent attention layers have a learned sink per head
+    latent_gate: bool = True  # ... and an elementwise output gate
+    # every pass over the looped layers starts from the residual plus a learned vector of the pass ("loop.step"), each but
+    # the first also plus the embedding output
+    loop_inputs: bool = False
+    kinds: Dict[str, str] = field(default_factory=dict)  # layer type (config.json) -> mixer kind where the two differ
     # layer type (config.json) -> (left kind, right kind, branch_norm) of the designs' two-branch mixers
     pairs: Dict[str, tuple] = field(default_factory=lambda: {"parallel": ("sink_attention", "gated_delta", False)})
 
@@ -320,6 +354,8 @@ DESIGNS: Dict[str, LayeredDesign] = {
     "Zaronex": LayeredDesign("prenorm", 0.0, False, "gelu_tanh", mask="window", depth_average=True, latent_sink=False,
                              pairs={"parallel": ("pooled_attention", "gated_linear", True),
                                     "parallel_2": ("rotated_value_attention", "mamba", True)}),
+    "Fazolorn": LayeredDesign("prenorm", 0.0, False, "clamped_swish", moe="group_scores", latent_sink=False,
+                              latent_gate=False, loop_inputs=True, kinds={"attention": "sigmoid_attention"}, pairs={}),
 }
 
 
@@ -340,6 +376,7 @@ class LayeredConfig:
     stream_weights: bool = False  # the checkpoint holds read / write / mix weights per sublayer
     residual_mult: float = 1.0  # post-norm layers: factor of every normed sublayer output in the residual sum
     logit_softcap: float = 0.0  # logits pass cap * tanh(z / cap) (0: not)
+    logit_scale: float = 1.0  # logits are multiplied by this constant
     max_positions: int = 0  # rows of the learned position table (0: the design has none)
 
     @property
@@ -367,6 +404,9 @@ class LayeredConfig:
                 f = spec.mlp
                 if not 0 < f.top <= f.experts + f.identity or f.identity < 0 or f.experts + f.identity > 256:
                     raise ValueError(f"layer {i}: top {f.top} of {f.experts} + {f.identity} experts (at most 256)")
+                if f.groups < 1 or f.experts % f.groups or not 1 <= f.keep <= f.groups or \
+                        f.top > f.keep * (f.experts // f.groups) + f.identity:
+                    raise ValueError(f"layer {i}: top {f.top} of the best {f.keep} of {f.groups} groups of {f.experts} experts")
             parts = [m.left, m.right] if m.kind == "parallel" else [m]
             if m.kind == "parallel":
                 allowed = {(a, b) for a, b, _ in self.design.pairs.values()}
@@ -384,6 +424,11 @@ class LayeredConfig:
                     if q.inner < 1 or q.dt_rank < 1 or not 1 <= q.state <= 256 or not 1 <= q.conv <= 16:
                         raise ValueError(f"layer {i}: inner {q.inner} / dt_rank {q.dt_rank} / state {q.state} (<= 256) / "
                                          f"convolution taps {q.conv} (<= 16)")
+                if q.kind == "mingru" and q.inner < 1:
+                    raise ValueError(f"layer {i}: width {q.inner}")
+                if q.rot.scaling and "fast" in q.rot.scaling and (q.rot.base <= 1.0 or min(
+                        q.rot.scaling[k] for k in ("factor", "original", "fast", "slow")) <= 0.0):
+                    raise ValueError(f"layer {i}: rotary scaling {q.rot.scaling}")
                 if q.kind in SOFTMAX_KINDS and (q.window < 0 or q.pool < 0 or (q.pool > 0 and q.window < 1)):
                     raise ValueError(f"layer {i}: window {q.window} / pooled blocks of {q.pool}")
                 if q.kind in SOFTMAX_KINDS and q.rot_values and q.vdim % 2:
@@ -405,7 +450,7 @@ class LayeredConfig:
                         raise ValueError(f"layer {i}: heads {q.heads} / key heads {q.kv_heads} / dims {q.dim}, {q.vdim}")
                     if q.q_temp_every < 0:
                         raise ValueError(f"layer {i}: q_temp.every must be positive")
-            if m.kind in ("channel_delta", "gated_delta", "parallel", "gated_linear", "lightning", "mamba") + SOFTMAX_KINDS:
+            if m.kind in ("channel_delta", "gated_delta", "parallel", "gated_linear", "lightning", "mamba", "mingru") + SOFTMAX_KINDS:
                 continue
             if m.kind == "retention" and (m.decay is None or len(m.decay) != m.heads):
                 raise ValueError(f"layer {i}: retention needs one decay per head")
@@ -434,6 +479,11 @@ class LayeredConfig:
                         raise ValueError(f"layer {i}: its key heads and sizes differ from layer {j}'s")
 
     @property
+    def loop_inputs(self) -> bool:
+        """Whether something joins the residual ahead of the passes over looped layers."""
+        return self.design.loop_inputs and self.loop_stop > self.loop_start
+
+    @property
     def layer_runs(self) -> List[int]:
         """Layer index of every layer run in order: layers [loop_start, loop_stop) run loop_times times in a row
         with the same weights (each run with a cache or state of its own), the others once."""
@@ -442,6 +492,8 @@ class LayeredConfig:
 
     @staticmethod
     def _mixer_spec(kind: str, m: Dict[str, Any], design: Optional[LayeredDesign] = None) -> MixerSpec:
+        if design is not None:
+            kind = design.kinds.get(kind, kind)
         pairs = (design or DESIGNS["Ravelorn"]).pairs
         if kind in pairs:
             left, right, normed = pairs[kind]
@@ -463,8 +515,13 @@ class LayeredConfig:
             extra = dict(qk_norm="none", sink_kind="learned", bias=True, out_gate=True)
         elif kind == "rotated_value_attention":
             extra = dict(qk_norm="joint", sink_kind="none", rot_layout="interleaved", rot_values=True)
-        elif kind == "latent_attention" and design is not None and not design.latent_sink:
-            extra = dict(sink_kind="none")
+        elif kind == "sigmoid_attention":
+            extra = dict(qk_norm="none", sink_kind="none", values="keys", bias=True, weights="sigmoid")
+        elif kind == "latent_attention":
+            extra = dict(out_gate=design is None or design.latent_gate,
+                         sink_kind="learned" if design is None or design.latent_sink else "none")
+        elif kind == "mingru":
+            return MixerSpec(kind=kind, heads=1, dim=0, vdim=0, rot=RotarySpec(), inner=int(m["width"]))
         elif kind == "mamba":
             return MixerSpec(kind=kind, heads=1, dim=0, vdim=0, rot=RotarySpec(), inner=int(m["inner"]),
                              dt_rank=int(m["dt_rank"]), state=int(m["state"]), conv=int(m["conv"]))
@@ -500,8 +557,10 @@ class LayeredConfig:
             elif f["kind"] == "dense":
                 mlp = FeedForwardSpec("dense", int(f["ff"]), limit=float(f.get("limit") or 0.0))
             elif f["kind"] == "moe":
+                groups = f["router"].get("groups") or {}
                 mlp = FeedForwardSpec("moe", int(f["expert"]["ff"]), int(f["router"]["experts"]), int(f["router"]["top"]),
-                                      identity=int(f["router"].get("identity") or 0),
+                                      identity=int(f["router"].get("identity") or 0), groups=int(groups.get("count", 1)),
+                                      keep=int(groups.get("keep", 1)), route_scale=float(f["router"].get("scale", 1.0)),
                                       shared_ff=int((f.get("shared") or {}).get("ff") or 0))
             else:
                 raise ValueError(f"unknown feed-forward kind {f['kind']!r}")
@@ -514,6 +573,7 @@ class LayeredConfig:
                    loop_times=int(loop.get("times", 1)), side_dim=int(side.get("dim", 0)),
                    streams=int(d.get("streams", 1)), stream_weights="streams" in d,
                    residual_mult=float(d.get("residual_mult", 1.0)), logit_softcap=float(d.get("logit_softcap") or 0.0),
+                   logit_scale=float(d.get("logit_scale", 1.0)),
                    max_positions=int(d.get("max_positions") or 0))
 
     @classmethod
@@ -524,7 +584,7 @@ class LayeredConfig:
 
 # architecture name (config.json) -> "module:class" of the model that serves it
 ARCHITECTURES: Dict[str, str] = {name: "lit_gpt.layered:LayeredGPT"
-                                 for name in ("Bavesun", "Rigulorn", "Ravelorn", "Gatutar", "Zaronex")}
+                                 for name in ("Bavesun", "Rigulorn", "Ravelorn", "Gatutar", "Zaronex", "Fazolorn")}
 
 
 def load_config(checkpoint_dir: Union[str, Path]) -> Union[Config, LayeredConfig]:

@@ -29,7 +29,8 @@ The design named by ``config.architecture`` fixes the layer's shape (``config.de
 * prenorm — the same boundaries without an output norm: x <- x + mixer(norm1 x), then x <- x + ff(norm2 x). With
   ``depth_average`` the boundary at a layer's end also keeps the layer's result X_(i+1) and goes on with
   x <- sum_j dwa_i[j] X_j over the embedding output X_0 and all results so far (fp32; the rows of one step only: the
-  average mixes layers, never positions).
+  average mixes layers, never positions). With ``loop_inputs`` the boundary ahead of a pass over the looped layers adds
+  the pass's own vector ("loop.step"), and ahead of every pass but the first also the embedding output.
 """
 
 from __future__ import annotations
@@ -263,6 +264,10 @@ class SandwichSublayer(nn.Module):
         sublayer's output as one (y, None) pair, or a two-branch mixer's (y, weight) pairs, for the boundary launch."""
         src = h16 if h16 is not None else h
         T, W = src.shape
+        if cache is not None and self.module.fuses_input(step):
+            y = torch.empty(T, W, dtype=torch.float32, device=src.device)
+            self.module.forward_fused(h, self.w_in, self.b_in, step, cache, y, accumulate=False)
+            return [(y, None)], 1.0
         proj = None
         if self.w_in is not None and self.module.wants_proj(T):
             n_in = self.w_in.shape[0]
@@ -317,9 +322,13 @@ class PreNormBlock(nn.Module):
         self.sub1 = SandwichSublayer(self.mixer, w["norm1"], None, None, W, device, dtype)
         self.sub2 = None
         if spec.mlp is not None:
-            if spec.mlp.kind != "dense" or design.dense_ff != "gelu_tanh":
-                raise NotImplementedError("pre-norm layers serve the gated dense feed-forward")
-            mlp = GatedFeedForward(spec.mlp, W, _sub(w, "mlp."), device, dtype)
+            if spec.mlp.kind == "dense":
+                if design.dense_ff == "relu2":
+                    raise NotImplementedError("pre-norm layers serve gated dense feed-forwards")
+                clamp = (1.702, spec.mlp.limit, 1.0) if design.dense_ff == "clamped_swish" else None
+                mlp = GatedFeedForward(spec.mlp, W, _sub(w, "mlp."), device, dtype, clamp=clamp)
+            else:
+                mlp = SparseFeedForward(spec.mlp, W, _sub(w, "mlp."), device, dtype, route=design.moe)
             self.sub2 = SandwichSublayer(mlp, w["norm2"], None, None, W, device, dtype)
         self.register_buffer("dwa", None)
         if design.depth_average:
@@ -343,8 +352,13 @@ def _mixer_shapes(p: str, m, W: int) -> Dict[str, Tuple[int, ...]]:
         return {p + "in": (2 * m.inner, W), p + "conv": (m.inner, m.conv), p + "conv.b": (m.inner,),
                 p + "x": (m.dt_rank + 2 * m.state, m.inner), p + "dt": (m.inner, m.dt_rank), p + "dt.b": (m.inner,),
                 p + "A_log": (m.inner, m.state), p + "D": (m.inner,), p + "o": (W, m.inner)}
+    if m.kind == "mingru":
+        n = m.inner
+        return {p + "z": (n, W), p + "z.b": (n,), p + "x": (n, W), p + "x.b": (n,), p + "g": (n, W), p + "o": (W, n)}
     if m.kind in SOFTMAX_KINDS:
         out = {p + "q": (m.heads * m.dim, W), p + "k": (m.kv_heads * m.dim, W)}
+        if m.weights == "sigmoid":
+            out[p + "pb"] = (m.heads,)
         if m.values == "own":
             out[p + "v"] = (m.kv_heads * m.vdim, W)
         if m.sink_kind == "learned":
@@ -440,11 +454,22 @@ class LayeredGPT(nn.Module):
                 LayeredBlock(i, spec, config, _sub(weights, f"l{i}."), self.side_embed, device, dtype)
                 for i, spec in enumerate(config.layers))
         self.register_buffer("head", None)
+        # the vectors that join the residual ahead of each pass over the looped layers
+        self.register_buffer("loop_step", None)
+        if config.loop_inputs:
+            t = weights["loop.step"]
+            if tuple(t.shape) != (config.loop_times, W):
+                raise ValueError(f"loop.step: shape {tuple(t.shape)}, expected {(config.loop_times, W)}")
+            if not self.sandwich or design.depth_average:
+                raise NotImplementedError("inputs of the looped passes belong to pre-norm layers without a depth average")
+            self.loop_step = t.to(device=device, dtype=torch.float32).contiguous()
         if not design.tied_head:
             if tuple(weights["head"].shape) != (V, W):
                 raise ValueError(f"head: shape {tuple(weights['head'].shape)}, expected {(V, W)}")
             self.head = weights["head"].to(device=device, dtype=dtype).contiguous()
         self.register_buffer("final_bias", None)
+        if config.logit_scale != 1.0 and (design.norm == "layer" or design.norm_offset != 0.0):
+            raise NotImplementedError("scaled logits go with RMS norms with plain weights")
         if design.norm == "layer":
             self.final_norm = None
             self.register_buffer("final_weight", weights["final.norm"].to(device=device, dtype=torch.float32).contiguous())
@@ -452,7 +477,9 @@ class LayeredGPT(nn.Module):
                 self.final_bias = weights["final.norm.b"].to(device=device, dtype=torch.float32).contiguous()
         else:
             self.final_norm = StreamRMSNorm(W, eps=config.norm_eps, offset=design.norm_offset)
-            self.final_norm.weight = weights["final.norm"].to(device=device, dtype=torch.float32).contiguous()
+            # (a constant factor of the logits is folded into the final norm's weight)
+            self.final_norm.weight = (weights["final.norm"].to(device=device, dtype=torch.float32) *
+                                      config.logit_scale).contiguous()
         self.runs: List[int] = config.layer_runs
         self.caches: Optional[nn.ModuleList] = None  # one cache / state per layer run
         self._max_seq_length = 0
@@ -481,6 +508,8 @@ class LayeredGPT(nn.Module):
             out["final.norm.b"] = (W,)
         if config.design.positions == "learned":
             out["pos"] = (config.max_positions, W)
+        if config.loop_inputs:
+            out["loop.step"] = (config.loop_times, W)
         for i, spec in enumerate(config.layers):
             m, p = spec.mixer, f"l{i}."
             out[p + "norm1"] = (W,)
@@ -507,7 +536,7 @@ class LayeredGPT(nn.Module):
                 if m.kv_from is None:
                     out.update({p + "mix.k": (2 * m.kv_heads * m.dim, W), p + "mix.v": (m.kv_heads * m.vdim, W)})
                 out.update({p + f"mix.{n}": (m.dim,) for n in ("lq1", "lk1", "lq2", "lk2")})
-            elif m.kind in ("channel_delta", "gated_delta", "parallel", "gated_linear", "lightning", "mamba") + SOFTMAX_KINDS:
+            elif m.kind in ("channel_delta", "gated_delta", "parallel", "gated_linear", "lightning", "mamba", "mingru") + SOFTMAX_KINDS:
                 out.update(_mixer_shapes(p + "mix.", m, W))
             elif m.kind == "mamba2":
                 inner, bc = m.heads * m.vdim, 2 * m.groups * m.state
@@ -525,14 +554,16 @@ class LayeredGPT(nn.Module):
                             p + "mix.uv": (m.heads * m.vdim, m.kv_rank)})
                 if m.sink_kind == "learned":
                     out[p + "mix.sink"] = (m.heads,)
-                out.update({p + "mix.g": (m.heads * m.vdim, W), p + "mix.o": (W, m.heads * m.vdim)})
+                if m.out_gate:
+                    out[p + "mix.g"] = (m.heads * m.vdim, W)
+                out[p + "mix.o"] = (W, m.heads * m.vdim)
             f = spec.mlp
             if f is not None and f.kind == "dense" and config.design.dense_ff == "relu2":
                 out.update({p + "mlp.up": (f.ff, W), p + "mlp.down": (W, f.ff)})
             elif f is not None and f.kind == "dense":
                 out.update({p + "mlp.gate": (f.ff, W), p + "mlp.up": (f.ff, W), p + "mlp.down": (W, f.ff)})
             elif f is not None:
-                gated = config.design.moe == "scores"
+                gated = config.design.moe in ("scores", "group_scores")
                 out[p + "mlp.router"] = (f.experts + (f.identity if gated else 0), W)
                 if gated:
                     out[p + "mlp.correction"] = (f.experts + f.identity,)
@@ -568,12 +599,16 @@ class LayeredGPT(nn.Module):
             elif leaf == "dwa":  # mostly the layer's own result, a little of every other
                 t = 0.15 * torch.randn(shape, generator=g)
                 t[-1] += 0.8
-            elif name.endswith(("q.b", "k.b", "v.b")):
+            elif name.endswith(("q.b", "k.b", "v.b", "z.b", "x.b")):
                 t = 0.3 * torch.randn(shape, generator=g)
             elif name.endswith("dt.b"):
                 t = -1.5 + torch.randn(shape, generator=g)
             elif name.endswith(("norm1.b", "norm2.b", "final.norm.b", "correction")):
                 t = 0.1 * torch.randn(shape, generator=g)
+            elif name == "loop.step":
+                t = shape[1] ** -0.5 * torch.randn(shape, generator=g)
+            elif leaf == "pb":  # (a key's weight is around 1 / 8)
+                t = -2.0 + 0.5 * torch.randn(shape, generator=g)
             elif name == "pos":
                 t = 0.5 * shape[1] ** -0.5 * torch.randn(shape, generator=g)
             elif name.endswith(".conv") and len(shape) == 2 and ".mix." in name and "mamba" not in name and \
@@ -687,7 +722,8 @@ class LayeredGPT(nn.Module):
     def _forward_sandwich(self, step: StepBatch, after_layer=None) -> torch.Tensor:
         """The sandwich and pre-norm layers. Every boundary between two sublayers is one launch: the branch norms and the
         average of a two-branch mixer, the output norm times the layer scale (sandwich layers), the residual add, at a
-        layer's end the average over the depth (designs that have it), and the next sublayer's normed input (for more
+        layer's end the average over the depth (designs that have it), ahead of a pass over the looped layers what joins
+        the residual there (likewise), and the next sublayer's normed input (for more
         than 8 rows with bf16 weights only its bf16 copy, unless the next module also reads it in fp32).
         ``after_layer(run, x)``: a hook that sees the residual (T, width) after each layer run (for tests)."""
         eps, W = self.config.norm_eps, self.config.width
@@ -705,22 +741,40 @@ class LayeredGPT(nn.Module):
 
         def reads(sub):  # (fp32 input wanted, bf16 copy wanted)
             b16 = sub.wants_bf16(step.T)
-            return (not b16) or getattr(sub.module, "reads_f32", False), b16
+            return (not b16) or sub.module.reads_f32(step.T), b16
+
+        x0, passes = None, {}  # run that begins a pass -> the pass's number
+        if self.loop_step is not None:
+            n = self.config.loop_stop - self.config.loop_start
+            passes = {self.config.loop_start + t * n: t for t in range(self.config.loop_times)}
+            # the first sublayer reads the embedding output in place and the residual goes on in a row of its own
+            x0, x_in, x = x, x, torch.empty_like(x)
+
+        def joins(run):  # what joins the residual ahead of this run
+            t = passes.get(run)
+            return {} if t is None else dict(add_vec=self.loop_step[t], add=x0 if t else None)
 
         f32, b16 = reads(chain[0][2])
-        h, h16 = seq_ops.sandwich_step(x if x_in is None else x_in, next_w=chain[0][2].norm_w, eps=eps, want_f32=f32,
-                                       bf16_copy=b16)
+        first = joins(0)
+        h, h16 = seq_ops.sandwich_step(x if x_in is None or first else x_in, next_w=chain[0][2].norm_w, eps=eps,
+                                       want_f32=f32, bf16_copy=b16, x_in=x_in if first else None, **first)
+        x_in = None if first else x_in
         for n, (run, block, sub, cache) in enumerate(chain):
             branches, coef = sub(h, h16, step, cache)
             nxt = chain[n + 1][2] if n + 1 < len(chain) else None
             ends = nxt is None or chain[n + 1][0] != run
             f32, b16 = reads(nxt) if nxt is not None else (False, False)
+            more = joins(chain[n + 1][0]) if ends and nxt is not None else {}
+            if more and after_layer is not None:  # the hook sees the residual before anything else joins it
+                seq_ops.sandwich_step(x, branches=branches, coef=coef, post_w=sub.post_w, eps=eps, x_in=x_in)
+                after_layer(run, x)
+                branches, x_in = (), None
             h, h16 = seq_ops.sandwich_step(x, branches=branches, coef=coef, post_w=sub.post_w,
                                            next_w=nxt.norm_w if nxt is not None else None, eps=eps, want_f32=f32,
                                            bf16_copy=b16, x_in=x_in, hist=hist if ends else None,
-                                           depth_w=block.dwa if ends and hist is not None else None)
+                                           depth_w=block.dwa if ends and hist is not None else None, **more)
             x_in = None
-            if after_layer is not None and ends:
+            if after_layer is not None and ends and not more:
                 after_layer(run, x)
         return x
 

@@ -11,7 +11,8 @@ Mixers here: ``Retention`` (and its preset ``Lightning``: the constant-decay rul
 (the gated delta rule with a decay per head or per head and key channel), ``GatedLinearAttention`` (the gated rule without
 the correction), ``SinkAttention`` (one-map softmax attention: optional biases, q / k norms, rotary positions, a query
 temperature, a window with pooled blocks before it, a learned or constant sink, values that are the keys or are rotated, a
-gate per head or per column) and ``ParallelMixer`` (two of them side by side on one input projection).
+gate per head or per column, sigmoid weights in place of the softmax), ``MinGRU`` (an elementwise gated recurrence) and
+``ParallelMixer`` (two of them side by side on one input projection).
 
 A step is a packed batch (``StepBatch``): the tokens of all sequences row after row, with per-token cache slot and
 position and per-sequence row range, slot and first position, all int32 on the device. Sizes, decays, scales, rotary
@@ -29,7 +30,7 @@ import torch.nn as nn
 
 from lit_gpt import seq_ops
 from lit_gpt.config import FeedForwardSpec, MixerSpec, RotarySpec
-from lit_gpt.model import CachePair, HeadKVCache, LatentKVCache, RetentionState, ScanState
+from lit_gpt.model import CachePair, ChannelState, HeadKVCache, LatentKVCache, RetentionState, ScanState
 
 
 @dataclass
@@ -91,6 +92,14 @@ class InputReader(nn.Module):
     def wants_proj(self, rows: int) -> bool:
         """Whether a step of ``rows`` tokens needs the shared input projection made for this module."""
         return True
+
+    def fuses_input(self, step: StepBatch) -> bool:
+        """Whether the module makes its input projection itself in this step (``forward_fused``)."""
+        return False
+
+    def reads_f32(self, rows: int) -> bool:
+        """Whether a step of ``rows`` tokens needs the module's input in fp32 beside the bf16 copy its products read."""
+        return False
 
 
 class Retention(InputReader):
@@ -155,7 +164,7 @@ class LatentAttention(InputReader):
     one rotated key part shared by all heads (interleaved rotary pairs 2i, 2i + 1). The score of head h is
     (q_h . W_uk,h c + q_rot,h . k_rot) * scale; a learned per-head sink scalar adds its exponential to the softmax normaliser. The kernels never expand
     keys or values: the query is mapped through W_uk,h first (one product per head), attention runs over the cached
-    rows [c | k_rot] for all heads alike, and W_uv,h maps the weighted latent back. Output gate sigmoid(W_g h).
+    rows [c | k_rot] for all heads alike, and W_uv,h maps the weighted latent back. Output gate sigmoid(W_g h) (``out_gate``).
     ``q_rank`` > 0: the queries come from a latent of their own, q = W_uq rmsnorm(W_dq h); ``window`` > 0: a position sees
     the last ``window`` keys."""
 
@@ -163,15 +172,15 @@ class LatentAttention(InputReader):
         super().__init__()
         self.H, self.d, self.dr, self.dv, self.r = spec.heads, spec.dim, spec.rot_dim, spec.vdim, spec.kv_rank
         self.eps, self.scale, self.rot_dims, self.dtype = eps, spec.scale, spec.rot.dims, dtype
-        self.q_rank, self.window = spec.q_rank, spec.window
+        self.q_rank, self.window, self.out_gate, self.rot_mult = spec.q_rank, spec.window, spec.out_gate, spec.rot.mult
         H, d, dr, dv, r = self.H, self.d, self.dr, self.dv, self.r
         q_shapes = (("dq", (self.q_rank, width)), ("dq.norm", (self.q_rank,)), ("uq", (H * (d + dr), self.q_rank))) \
             if self.q_rank else (("q", (H * (d + dr), width)),)
-        for name, shape in q_shapes + (("dkv", (r + dr, width)), ("dkv.norm", (r,)), ("g", (H * dv, width)),
-                                       ("uk", (H * d, r)), ("uv", (H * dv, r)), ("o", (width, H * dv))):
+        for name, shape in q_shapes + (("dkv", (r + dr, width)), ("dkv.norm", (r,)), ("uk", (H * d, r)), ("uv", (H * dv, r)), ("o", (width, H * dv))) + \
+                ((("g", (H * dv, width)),) if self.out_gate else ()):
             if tuple(w[name].shape) != shape:
                 raise ValueError(f"latent_attention.{name}: shape {tuple(w[name].shape)}, expected {shape}")
-        self._in = [(n, w[n]) for n in ("dq" if self.q_rank else "q", "dkv", "g")]
+        self._in = [(n, w[n]) for n in ("dq" if self.q_rank else "q", "dkv") + (("g",) if self.out_gate else ())]
         self.register_buffer("w_uq", None)
         self.register_buffer("q_norm_w", None)
         if self.q_rank:
@@ -203,7 +212,8 @@ class LatentAttention(InputReader):
         else:
             q, q_off, ldq = proj, self.off["q"], ld
         seq_ops.latent_prepare(q, q_off, proj, self.off["dkv"], cache.c, cache.kr, self.norm_w, self.inv_freq, step.slot,
-                               step.pos, H=H, d=d, dr=dr, r=r, rot_dims=self.rot_dims, eps=self.eps)
+                               step.pos, H=H, d=d, dr=dr, r=r, rot_dims=self.rot_dims, eps=self.eps,
+                               rot_mult=self.rot_mult)
         qc = torch.empty(T, H * r, dtype=torch.float32, device=proj.device)
         seq_ops.linear(q, self.w_ukT, M=T, N=r, K=d, y=qc, a_off=q_off, lda=ldq, ldy=H * r, batch=H,
                        stride_a=d + dr, stride_w=r * d, stride_y=r)
@@ -214,11 +224,14 @@ class LatentAttention(InputReader):
         else:
             lat = seq_ops.latent_attention(qc, q, q_off, cache.c, cache.kr, self.sink, step.slot, step.pos, H=H,
                                            d=d, dr=dr, r=r, scale=self.scale, window=self.window)
-        att = torch.empty(T, H * dv, dtype=torch.float32, device=proj.device)
+        # (without a gate the per-head products leave the out-projection's operand as it reads it)
+        b16 = _tiles16(T, self.w_o)
+        att = torch.empty(T, H * dv, dtype=torch.bfloat16 if b16 and not self.out_gate else torch.float32, device=proj.device)
         seq_ops.linear(lat, self.w_uv, M=T, N=dv, K=r, y=att, lda=H * r, ldy=H * dv, batch=H, stride_a=r,
                        stride_w=dv * r, stride_y=dv)
-        att = seq_ops.head_gate(att, proj, self.off["g"], H=H, dv=dv, unit_norm=False, eps=self.eps,
-                                act=seq_ops.ACT_SIGMOID, bf16_copy=_tiles16(T, self.w_o))
+        if self.out_gate:
+            att = seq_ops.head_gate(att, proj, self.off["g"], H=H, dv=dv, unit_norm=False, eps=self.eps,
+                                    act=seq_ops.ACT_SIGMOID, bf16_copy=b16)
         W = x.shape[1]
         seq_ops.linear(att, self.w_o, M=T, N=W, K=H * dv, y=x, lda=H * dv, ldy=W, accumulate=accumulate)
 
@@ -492,7 +505,9 @@ class SinkAttention(InputReader):
     ``rot_layout`` "interleaved": pairs (2i, 2i + 1); ``bias``: biases on q, k and v, added in the shared projection;
     ``rot_values``: values are rotated by their position over all vdim dims (base of the keys' rotation, not rescaled) and
     every output is turned back by the query's position; ``window`` / ``pool``: a position sees the last ``window``
-    tokens, and the mean key and value of every aligned block of ``pool`` tokens once the last of them has left these."""
+    tokens, and the mean key and value of every aligned block of ``pool`` tokens once the last of them has left these;
+    ``weights`` "sigmoid": a visible key's weight is sigmoid(score + pb[h]) with a stored number per head, and nothing is
+    normalised over the keys; ``mask_size``: a position sees the keys of its own aligned chunk only."""
 
     def __init__(self, spec: MixerSpec, width: int, eps: float, w: Dict[str, torch.Tensor], device, dtype) -> None:
         super().__init__()
@@ -500,9 +515,10 @@ class SinkAttention(InputReader):
         self.scale, self.cap, self.chunk = spec.scale, spec.softcap, spec.mask_size
         self.temp_coef, self.temp_every = spec.q_temp_coef, spec.q_temp_every
         self.qk_norm, self.own_values, self.head_gate = spec.qk_norm, spec.values == "own", spec.head_gate
-        self.rot_dims = spec.rot.dims
+        self.rot_dims, self.rot_mult = spec.rot.dims, spec.rot.mult
         H, G, d, dv = self.H, self.G, self.d, self.dv
         shapes = [("q", (H * d, width)), ("k", (G * d, width)), ("o", (width, H * dv))]
+        shapes += [("pb", (H,))] if spec.weights == "sigmoid" else []
         shapes += [("v", (G * dv, width))] if self.own_values else []
         self.joint, self.interleaved, self.out_gate = spec.qk_norm == "joint", spec.rot_layout == "interleaved", spec.out_gate
         self.window, self.pool = spec.window, spec.pool
@@ -522,6 +538,7 @@ class SinkAttention(InputReader):
             if w["sink"].numel() != H:
                 raise ValueError(f"{spec.kind}.sink: {w['sink'].numel()} values, expected {H}")
             self.sink = _f32(w["sink"], device)
+        self.register_buffer("score_bias", _f32(w["pb"], device) if spec.weights == "sigmoid" else None)
         self.register_buffer("q_norm", None)
         self.register_buffer("k_norm", None)
         if self.qk_norm in ("weight", "joint"):
@@ -556,7 +573,7 @@ class SinkAttention(InputReader):
                                  norm=0 if self.qk_norm == "none" else (2 if self.joint else 1),
                                  q_weight=self.q_norm, k_weight=self.k_norm, inv_freq=self.inv_freq,
                                  rot_dims=self.rot_dims, interleaved=self.interleaved, v_freq=self.v_freq,
-                                 pooled=cache.pooled if one else None, pool=self.pool)
+                                 rot_mult=self.rot_mult, pooled=cache.pooled if one else None, pool=self.pool)
         if self.pool and not one:
             seq_ops.pool_blocks(cache.k, cache.v, cache.pooled, self.pool, step.seq_start, step.seq_slot, step.seq_pos0,
                                 step.max_len or step.T)
@@ -565,7 +582,8 @@ class SinkAttention(InputReader):
                                chunk=self.chunk, cap=self.cap, post=post, bf16_copy=_tiles16(step.T, self.w_o),
                                gate_off=self.off["g"] if self.head_gate or self.out_gate else -1,
                                gate_cols=dv if self.out_gate else 1, window=self.window, pooled=cache.pooled,
-                               pool=self.pool, v_freq=self.v_freq, interleaved=self.interleaved)
+                               pool=self.pool, v_freq=self.v_freq, interleaved=self.interleaved,
+                               score_bias=self.score_bias)
         W = x.shape[1]
         seq_ops.linear(att, self.w_o, M=step.T, N=W, K=H * dv, y=x, lda=H * dv, ldy=W, accumulate=accumulate)
 
@@ -618,6 +636,53 @@ class GatedLinearAttention(InputReader):
                               weight=self.norm_w, post=post, bf16_copy=_tiles16(T, self.w_o))
         W = x.shape[1]
         seq_ops.linear(o, self.w_o, M=T, N=W, K=H * dv, y=x, lda=H * dv, ldy=W, accumulate=accumulate)
+
+
+class MinGRU(InputReader):
+    """An elementwise gated recurrence whose gates read the current token alone: with z = sigmoid(W_z h + b_z) and the
+    candidate c = u + 1/2 where u = W_x h + b_x >= 0, sigmoid(u) elsewhere (so c > 0), every channel keeps
+    S <- (1 - z) S + z c; the output is W_o (S * silu(W_g h)). The state (``inner`` numbers, fp32) lives in a cache slot."""
+
+    def __init__(self, spec: MixerSpec, width: int, eps: float, w: Dict[str, torch.Tensor], device, dtype) -> None:
+        super().__init__()
+        self.inner = n = spec.inner
+        for name, shape in (("z", (n, width)), ("z.b", (n,)), ("x", (n, width)), ("x.b", (n,)), ("g", (n, width)),
+                            ("o", (width, n))):
+            if tuple(w[name].shape) != shape:
+                raise ValueError(f"mingru.{name}: shape {tuple(w[name].shape)}, expected {shape}")
+        self._in = [(name, w[name]) for name in ("z", "x", "g")]
+        self._bias = {name: w[name + ".b"] for name in ("z", "x")}
+        self.register_buffer("w_o", w["o"].to(device=device, dtype=dtype).contiguous())
+
+    def in_parts(self):
+        return self._in
+
+    def in_bias(self):
+        return self._bias
+
+    def build_cache(self, slots: int, max_seq_length: int, device, dtype) -> ChannelState:
+        return ChannelState(slots, self.inner, device=device)
+
+    def forward(self, proj: torch.Tensor, step: StepBatch, cache: ChannelState, x: torch.Tensor,
+                accumulate: bool = True) -> None:
+        T, W = x.shape
+        y = seq_ops.mingru(proj, self.off["z"], self.off["x"], self.off["g"], cache.s, step.seq_start, step.seq_slot,
+                           step.seq_pos0, max_len=step.max_len or T, bf16=_tiles16(T, self.w_o))
+        self._project(y, x, accumulate)
+
+    def fuses_input(self, step: StepBatch) -> bool:
+        """One token for each of a few sequences: projections and recurrence in one launch."""
+        return step.max_len == 1 and step.T <= 8
+
+    def forward_fused(self, h: torch.Tensor, w_in: torch.Tensor, b_in: Optional[torch.Tensor], step: StepBatch,
+                      cache: ChannelState, x: torch.Tensor, accumulate: bool = True) -> None:
+        """h (T, width): the normed input; w_in, b_in: the layer's input projection."""
+        self._project(seq_ops.mingru_step(h, w_in, b_in, self.off["z"], self.off["x"], self.off["g"], cache.s,
+                                          step.seq_slot, step.seq_pos0), x, accumulate)
+
+    def _project(self, y: torch.Tensor, x: torch.Tensor, accumulate: bool) -> None:
+        T, W = x.shape
+        seq_ops.linear(y, self.w_o, M=T, N=W, K=self.inner, y=x, lda=self.inner, ldy=W, accumulate=accumulate)
 
 
 class Lightning(Retention):
@@ -802,7 +867,7 @@ class DenseFeedForward(InputReader):
 
 
 class SparseFeedForward(InputReader):
-    """Mixture of experts with an fp32 router, in one of two forms.
+    """Mixture of experts with an fp32 router, in one of four forms.
 
     ``route = "top_logits"``: the ``top`` largest logits are chosen, weights = softmax restricted to the chosen
     logits, expert = W_down act(W_up h) (``act`` defaults to the square of relu).
@@ -816,22 +881,25 @@ class SparseFeedForward(InputReader):
     output (another activation than the square of relu is refused). With ``shared_ff`` a shared expert of the same
     form (``shared.up`` / ``shared.down``) runs for every token and is added times sigmoid(W_sg h), one number per
     token (``shared.sg``); its up matrix, its gate row and the router are one fused input projection.
+    ``route = "group_scores"``: scores = sigmoid of every router output; choice scores = score + ``correction``. The experts
+    form ``groups`` equal groups of neighbours, a group is worth the sum of its two largest choice scores, and the ``top``
+    largest choice scores of the ``keep`` best groups are chosen; the weights are the chosen scores times ``route_scale``;
+    gated experts as with "scores".
 
     Few (token, choice) pairs (decode) stream only the chosen experts' rows through two GEMV launches. A prompt
     sorts its pairs by expert on the device and runs two grouped products over the expert ranges, then sums each
     token's choices in routing order."""
 
     STREAM_PAIRS = 48  # up to this many (token, choice) pairs the streaming form runs
-    reads_f32 = True  # the streaming experts and the in-launch router read the fp32 input itself
-
     def __init__(self, spec: FeedForwardSpec, width: int, w: Dict[str, torch.Tensor], device, dtype,
                  act: Optional[int] = None, route: str = "top_logits") -> None:
         super().__init__()
-        if route not in ("top_logits", "scores", "sigmoid"):
+        if route not in ("top_logits", "scores", "sigmoid", "group_scores"):
             raise ValueError(f"unknown routing {route!r}")
         self.E, self.top, self.ff, self.route = spec.experts, spec.top, spec.ff, route
-        self.gated = route == "scores"
+        self.gated = route in ("scores", "group_scores")
         self.n_router = spec.experts + (spec.identity if self.gated else 0)
+        self.grouped = dict(groups=spec.groups, keep=spec.keep, scale=spec.route_scale) if route == "group_scores" else {}
         self.act = act if act is not None else (seq_ops.ACT_SILU if self.gated else seq_ops.ACT_RELU2)
         if route == "sigmoid" and self.act != seq_ops.ACT_RELU2:
             raise NotImplementedError("a score on the expert's input is served for the square of relu")
@@ -871,15 +939,24 @@ class SparseFeedForward(InputReader):
         """Whether a step of ``rows`` tokens needs the layer's input projection (the router logits) made for it."""
         return not (self.w_router is not None and rows * self.top <= self.STREAM_PAIRS)
 
-    def forward(self, proj: Optional[torch.Tensor], h: torch.Tensor, x: torch.Tensor,
+    def reads_f32(self, rows: int) -> bool:
+        """The streaming experts, the in-launch router and identity experts read the fp32 input itself."""
+        return rows * self.top <= self.STREAM_PAIRS or self.n_router > self.E
+
+    def forward(self, proj: Optional[torch.Tensor], h: Optional[torch.Tensor], x: torch.Tensor,
                 h16: Optional[torch.Tensor] = None, accumulate: bool = True) -> None:
-        """h: the sublayer's input (fp32); h16: its bf16 copy when the layer made one (the grouped products read it).
-        ``proj`` None (score routing, few tokens): the router's logits are made inside the routing launch."""
-        T, W = h.shape
+        """h: the sublayer's input (fp32; may be missing where ``reads_f32`` says so); h16: its bf16 copy when the layer
+        made one (the grouped products read it). ``proj`` None (score routing, few tokens): the router's logits are made
+        inside the routing launch."""
+        T, W = x.shape
         E, top, F = self.E, self.top, self.ff
         sig = self.route == "sigmoid"
         if proj is None:
-            ids, wts = seq_ops.moe_router(h, self.w_router, top, self.correction, sigmoid=sig, square=sig)
+            ids, wts = seq_ops.moe_router(h, self.w_router, top, self.correction, sigmoid=sig or bool(self.grouped),
+                                          square=sig, **self.grouped)
+        elif self.grouped:
+            ids, wts = seq_ops.moe_route_scores(proj, self.off["router"], self.n_router, top, self.correction, sigmoid=True,
+                                                **self.grouped)
         elif sig:
             ids, wts = seq_ops.moe_route_scores(proj, self.off["router"], self.n_router, top, sigmoid=True, square=True)
         elif self.gated:
@@ -895,15 +972,15 @@ class SparseFeedForward(InputReader):
         z_start, tok_of, where = seq_ops.moe_sort(ids, self.n_router)
         a_dtype = torch.bfloat16 if self.w_down.dtype == torch.bfloat16 else torch.float32
         if self.gated:
-            gu = torch.empty(pairs, 2 * F, dtype=torch.float32, device=h.device)
+            gu = torch.empty(pairs, 2 * F, dtype=torch.float32, device=x.device)
             seq_ops.linear(h if h16 is None else h16, self.w_up, M=pairs, N=2 * F, K=W, y=gu, lda=W, ldy=2 * F, batch=E,
                            stride_w=2 * F * W, a_rows=tok_of, z_start=z_start)
             a = seq_ops.glu(gu, 0, F, F, self.act, bf16=a_dtype == torch.bfloat16)
         else:
-            a = torch.empty(pairs, F, dtype=a_dtype, device=h.device)
+            a = torch.empty(pairs, F, dtype=a_dtype, device=x.device)
             seq_ops.linear(h if h16 is None else h16, self.w_up, M=pairs, N=F, K=W, y=a, lda=W, ldy=F, batch=E,
                            stride_w=F * W, act=self.act, a_rows=tok_of, z_start=z_start)
-        y = torch.empty(pairs, W, dtype=torch.float32, device=h.device)
+        y = torch.empty(pairs, W, dtype=torch.float32, device=x.device)
         seq_ops.linear(a, self.w_down, M=pairs, N=W, K=F, y=y, lda=F, ldy=W, batch=E, stride_w=W * F, z_start=z_start)
         identity = self.n_router > E
         seq_ops.moe_combine(y, where, wts, x, ids=ids if identity else None, n_real=E, h=h if identity else None,
@@ -944,4 +1021,5 @@ MIXERS = {"retention": Retention, "latent_attention": LatentAttention, "attentio
           "mamba2": SelectiveScan, "channel_delta": GatedDelta, "gated_delta": GatedDelta,
           "sink_attention": SinkAttention, "parallel": ParallelMixer, "rotary_attention": SinkAttention,
           "key_value_attention": SinkAttention, "gated_linear": GatedLinearAttention, "lightning": Lightning,
-          "pooled_attention": SinkAttention, "rotated_value_attention": SinkAttention, "mamba": ChannelScan}
+          "pooled_attention": SinkAttention, "rotated_value_attention": SinkAttention, "mamba": ChannelScan,
+          "sigmoid_attention": SinkAttention, "mingru": MinGRU}

@@ -746,6 +746,26 @@ class ScanState(nn.Module):
         torch.nn.init.zeros_(self.conv)
 
 
+class ChannelState(nn.Module):
+    """Per-slot state of an elementwise recurrence: one fp32 number per channel (``s``: slots, channels). The kernels take
+    zeros for a sequence that starts at position 0, so a slot that is given out again needs no clearing."""
+
+    def __init__(self, slots: int, channels: int, device: Optional[torch.device] = None) -> None:
+        super().__init__()
+        self.register_buffer("s", torch.zeros(slots, channels, device=device, dtype=torch.float32), persistent=False)
+
+    @property
+    def slots(self) -> int:
+        return self.s.size(0)
+
+    def grow(self, slots: int) -> None:
+        if slots > self.slots:
+            self.s = _grown(self.s, slots)
+
+    def reset_parameters(self) -> None:
+        torch.nn.init.zeros_(self.s)
+
+
 class CachePair(nn.Module):
     """The caches of two mixers that run side by side in one layer (``left`` and ``right``), handed out, grown and
     cleared together."""

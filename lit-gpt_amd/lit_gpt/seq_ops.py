@@ -37,15 +37,15 @@ SIGNATURES = {
     "lgs_gather_rows": [_P, _P, _P, _I, _I, _P],
     "lgs_retention": [_P, _P, _P, _L, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _I, _I, _P, _I, _P],
     "lgs_head_gate": [_P, _P, _L, _I, _I, _I, _I, _F, _I, _P, _F, _P, _P, _I, _I, _P],
-    "lgs_latent_prepare": [_P, _L, _P, _L, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _P],
+    "lgs_latent_prepare": [_P, _L, _P, _L, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _P],
     "lgs_latent_attention": [_P, _P, _L, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _P, _I, _P],
     "lgs_latent_attention_tiles": [_P, _P, _L, _I, _P, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P],
     "lgs_glu": [_P, _P, _L, _P, _I, _I, _I, _I, _P],
     "lgs_moe_route": [_P, _L, _I, _I, _I, _P, _P, _P],
-    "lgs_moe_route_scores": [_P, _L, _I, _I, _I, _P, _P, _P, _I, _I, _P],
-    "lgs_moe_router": [_P, _L, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P],
+    "lgs_moe_route_scores": [_P, _L, _I, _I, _I, _P, _P, _P, _I, _I, _I, _I, _F, _P],
+    "lgs_moe_router": [_P, _L, _P, _I, _I, _I, _I, _I, _P, _P, _P, _I, _I, _I, _I, _F, _P],
     "lgs_act_rows": [_P, _L, _P, _L, _P, _I, _I, _I, _I, _P],
-    "lgs_sandwich_step": [_P, _P, _P, _P, _P, _P, _F, _P, _P, _P, _P, _F, _I, _I, _P, _P, _I, _I, _P],
+    "lgs_sandwich_step": [_P, _P, _P, _P, _P, _P, _F, _P, _P, _P, _P, _F, _I, _I, _P, _P, _I, _I, _P, _P, _P],
     "lgs_moe_up": [_P, _L, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "lgs_moe_down": [_P, _P, _I, _P, _P, _P, _L, _I, _I, _I, _I, _I, _P, _L, _I, _P],
     "lgs_moe_sort": [_P, _I, _I, _I, _P, _P, _P, _P, _P],
@@ -64,16 +64,18 @@ SIGNATURES = {
     "lgs_layernorm": [_P, _P, _P, _F, _F, _I, _P, _P, _I, _I, _P],
     "lgs_softcap": [_P, _L, _F, _P],
     "lgs_normattn_prepare": [_P, _L, _I, _I, _I, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _F, _I, _I, _P, _P, _P,
-                             _I, _I, _P, _P, _P, _I, _I, _P],
+                             _F, _I, _I, _P, _P, _P, _I, _I, _P],
     "lgs_pool_blocks": [_P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "lgs_sinkattn": [_P, _L, _P, _P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _F, _F, _P,
-                     _L, _I, _I, _P, _P, _I, _I, _P, _I, _P],
+                     _L, _I, _I, _P, _P, _I, _I, _P, _I, _P, _P],
     "lgs_channel_scan": [_P, _P, _L, _P, _L, _I, _P, _L, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P, _P, _I,
                          _P],
     "lgs_delta_prepare": [_P, _L, _P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _F, _P, _I, _I, _I, _I, _F,
                           _P],
     "lgs_delta_step_prepare": [_P, _L, _P, _I, _I, _P, _P, _P, _P, _P, _L, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I,
                                _I, _F, _F, _P, _I, _I, _P],
+    "lgs_mingru": [_P, _P, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _P, _I, _P],
+    "lgs_mingru_step": [_P, _L, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P, _P, _P],
     "lgs_gated_delta": [_P, _L, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _P],
 }
 _RESTYPES = {"lgs_last_error_string": ctypes.c_char_p}
@@ -287,9 +289,10 @@ def norm_columns(proj: torch.Tensor, off: int, weight: torch.Tensor, *, eps: flo
 
 def latent_prepare(q: torch.Tensor, q_off: int, proj: torch.Tensor, kv_off: int, cache_c: torch.Tensor,
                    cache_kr: torch.Tensor, norm_w: torch.Tensor, inv_freq: Optional[torch.Tensor], slot: torch.Tensor,
-                   pos: torch.Tensor, *, H: int, d: int, dr: int, r: int, rot_dims: int, eps: float) -> None:
+                   pos: torch.Tensor, *, H: int, d: int, dr: int, r: int, rot_dims: int, eps: float,
+                   rot_mult: float = 1.0) -> None:
     """The queries are the H (d + dr) columns of ``q`` at ``q_off`` (rotated parts turned in place); the latent and the
-    shared key part the r + dr columns of ``proj`` at ``kv_off`` (``q`` may be ``proj`` itself)."""
+    shared key part the r + dr columns of ``proj`` at ``kv_off`` (``q`` may be ``proj`` itself); cos and sin times ``rot_mult``."""
     T, ld = proj.shape
     slots, S = cache_c.shape[:2]
     if tuple(cache_c.shape) != (slots, S, r) or tuple(cache_kr.shape) != (slots, S, dr) or norm_w.numel() != r:
@@ -301,7 +304,7 @@ def latent_prepare(q: torch.Tensor, q_off: int, proj: torch.Tensor, kv_off: int,
                                              _wf32(cache_c, "cache_c"), _dev(cache_kr, "cache_kr", F32),
                                              _dev(norm_w, "norm_w", F32), _opt(inv_freq, "inv_freq", F32),
                                              _dev(slot, "slot", I32), _dev(pos, "pos", I32), T, H, d, dr, r, rot_dims,
-                                             S, float(eps), _stream()))
+                                             S, float(eps), float(rot_mult), _stream()))
 
 
 def latent_attention(qc: torch.Tensor, proj: torch.Tensor, q_off: int, cache_c: torch.Tensor, cache_kr: torch.Tensor,
@@ -373,10 +376,11 @@ def moe_route(proj: torch.Tensor, z_off: int, E: int, top: int):
 
 
 def moe_route_scores(proj: torch.Tensor, z_off: int, E: int, top: int, bias: Optional[torch.Tensor] = None,
-                     sigmoid: bool = False, square: bool = False):
+                     sigmoid: bool = False, square: bool = False, groups: int = 1, keep: int = 1, scale: float = 1.0):
     """Softmax over all E router outputs at proj[:, z_off:] (``sigmoid``: the sigmoid of every output on its own); the
     ``top`` largest of score + ``bias`` are chosen (lowest index first among equals); the weights are the chosen scores
-    themselves, not renormalised (``square``: their squares)."""
+    themselves, not renormalised (``square``: their squares), times ``scale``. With ``groups`` > 1 only experts of the ``keep``
+    best of that many equal groups of neighbours can be chosen; a group is worth the sum of its two largest score + bias."""
     T, ld = proj.shape
     if z_off + E > ld or (bias is not None and bias.numel() != E):
         raise ValueError("moe_route_scores: router logits outside the row, or the correction's size")
@@ -384,7 +388,7 @@ def moe_route_scores(proj: torch.Tensor, z_off: int, E: int, top: int, bias: Opt
     wts = torch.empty(T, top, dtype=F32, device=proj.device)
     _check(load_library().lgs_moe_route_scores(_dev(proj, "proj", F32) + 4 * z_off, ld, T, E, top,
                                                _opt(bias, "bias", F32), ids.data_ptr(), wts.data_ptr(), int(sigmoid),
-                                               int(square), _stream()))
+                                               int(square), int(groups), int(keep), float(scale), _stream()))
     return ids, wts
 
 
@@ -404,14 +408,16 @@ def act_rows(proj: torch.Tensor, off: int, n: int, act: int, gate_off: int = -1,
 def sandwich_step(x: torch.Tensor, *, branches=(), coef: float = 1.0, post_w: Optional[torch.Tensor] = None,
                   next_w: Optional[torch.Tensor] = None, eps: float, want_f32: bool = True, bf16_copy: bool = False,
                   x_in: Optional[torch.Tensor] = None, hist: Optional[torch.Tensor] = None,
-                  depth_w: Optional[torch.Tensor] = None):
+                  depth_w: Optional[torch.Tensor] = None, add: Optional[torch.Tensor] = None,
+                  add_vec: Optional[torch.Tensor] = None):
     """One boundary between sublayers of one residual, in place on x (T, W); the residual so far is read from ``x_in``
     when that is given.
     ``branches``: up to two (y, w) pairs of the sublayer that ran, each y (T, W) RMS-normed with weight w (w None: taken
     as it is); their sum times ``coef`` is RMS-normed with ``post_w`` (the output norm's weight times the layer's
     per-channel scale; None: no output norm) and added to x. With ``depth_w`` (n + 1 weights; a layer's end): x is kept
     in row block n of ``hist`` (rows, T, W), if it has that many, and becomes depth_w[n] x + sum_{j < n} depth_w[j]
-    hist[j]. With ``next_w`` the next sublayer's input rmsnorm(x) * next_w is returned as
+    hist[j]. With ``add_vec`` (W,) (ahead of a pass over looped layers; no ``depth_w``) x + ``add_vec`` goes on, plus ``add``
+    (T, W) if given. With ``next_w`` the next sublayer's input rmsnorm(x) * next_w is returned as
     (h fp32 or None, h bf16 or None)."""
     T, W = x.shape
     ys = [(None, None), (None, None)]
@@ -426,6 +432,8 @@ def sandwich_step(x: torch.Tensor, *, branches=(), coef: float = 1.0, post_w: Op
         n_prev, hist_rows = depth_w.numel() - 1, 0 if hist is None else hist.shape[0]
         if hist is None or tuple(hist.shape[1:]) != (T, W) or not 1 <= n_prev <= hist_rows:
             raise ValueError("sandwich_step: the earlier layers' results, (rows, T, W), at least one per earlier weight")
+    if (add_vec is not None and add_vec.numel() != W) or (add is not None and (add_vec is None or add.shape != (T, W))):
+        raise ValueError("sandwich_step: add_vec of one value per channel, add of the residual's shape beside it")
     h = torch.empty(T, W, dtype=F32, device=x.device) if next_w is not None and (want_f32 or not bf16_copy) else None
     h16 = torch.empty(T, W, dtype=torch.bfloat16, device=x.device) if next_w is not None and bf16_copy else None
     _check(load_library().lgs_sandwich_step(_opt(x_in, "x_in", F32), _dev(x, "x", F32), _opt(ys[0][0], "y0", F32), _opt(ys[0][1], "w0", F32),
@@ -433,12 +441,12 @@ def sandwich_step(x: torch.Tensor, *, branches=(), coef: float = 1.0, post_w: Op
                                             _opt(post_w, "post_w", F32), _opt(next_w, "next_w", F32),
                                             _opt(h, "h", F32), _opt(h16, "h_bf16", torch.bfloat16), float(eps), T, W,
                                             _opt(hist, "hist", F32), _opt(depth_w, "depth_w", F32), n_prev, hist_rows,
-                                            _stream()))
+                                            _opt(add, "add", F32), _opt(add_vec, "add_vec", F32), _stream()))
     return h, h16
 
 
 def moe_router(h: torch.Tensor, w: torch.Tensor, top: int, bias: Optional[torch.Tensor] = None, sigmoid: bool = False,
-               square: bool = False):
+               square: bool = False, groups: int = 1, keep: int = 1, scale: float = 1.0):
     """``moe_route_scores`` of the router logits w h, both in one launch (steps with few tokens). w (E, K)."""
     T, K = h.shape
     E = w.shape[0]
@@ -448,7 +456,7 @@ def moe_router(h: torch.Tensor, w: torch.Tensor, top: int, bias: Optional[torch.
     wts = torch.empty(T, top, dtype=F32, device=h.device)
     _check(load_library().lgs_moe_router(_dev(h, "h", F32), K, _dev(w, "w"), _wf32(w, "w"), T, K, E, top,
                                          _opt(bias, "bias", F32), ids.data_ptr(), wts.data_ptr(), int(sigmoid),
-                                         int(square), _stream()))
+                                         int(square), int(groups), int(keep), float(scale), _stream()))
     return ids, wts
 
 
@@ -771,13 +779,13 @@ def normattn_prepare(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, cac
                      eps: float, temp_coef: float = 0.0, temp_every: int = 0, norm: int = 1,
                      q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None,
                      inv_freq: Optional[torch.Tensor] = None, rot_dims: int = 0, interleaved: bool = False,
-                     v_freq: Optional[torch.Tensor] = None, pooled=None, pool: int = 0) -> None:
+                     v_freq: Optional[torch.Tensor] = None, pooled=None, pool: int = 0, rot_mult: float = 1.0) -> None:
     """Queries normed (``norm`` 1: each head divided by its root mean square, times ``q_weight`` (d,) if given; 2: all
     heads by one root mean square, ``q_weight`` (H d,); 0: not), rotated on the pairs (i, i + rot_dims / 2) - or
     ``interleaved`` (2i, 2i + 1) - and multiplied by the position's query temperature, in place in ``proj``; keys normed
     (``k_weight``) and rotated alike, and the values, into the cache rows (slot, position). cache_k (slots, S, G, d),
     cache_v (slots, S, G, dv). ``v_off == k_off`` (with dv == d): the values are the keys as projected. ``v_freq``
-    (dv / 2,): the values are rotated by their position. ``pooled`` = (pool_k, pool_v) (slots, blocks, G, d / dv) fp32
+    (dv / 2,): the values are rotated by their position. ``rot_mult``: factor of cos and sin of q and k. ``pooled`` = (pool_k, pool_v) (slots, blocks, G, d / dv) fp32
     with ``pool``: steps of one token per sequence leave the means of a block of ``pool`` positions when they complete it."""
     T, ld = proj.shape
     slots, S = cache_k.shape[:2]
@@ -798,7 +806,7 @@ def normattn_prepare(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, cac
                                                _dev(pos, "pos", I32), T, H, G, d, dv, S, float(eps), float(temp_coef),
                                                int(temp_every), int(norm), _opt(q_weight, "q_weight", F32),
                                                _opt(k_weight, "k_weight", F32), _opt(inv_freq, "inv_freq", F32),
-                                               int(rot_dims), int(interleaved), _opt(v_freq, "v_freq", F32),
+                                               float(rot_mult), int(rot_dims), int(interleaved), _opt(v_freq, "v_freq", F32),
                                                _opt(pk, "pool_k", F32), _opt(pv, "pool_v", F32),
                                                int(pool) if pk is not None else 0, pk.shape[1] if pk is not None else 0,
                                                _stream()))
@@ -835,13 +843,15 @@ def sinkattn(proj: torch.Tensor, q_off: int, cache_k: torch.Tensor, cache_v: tor
              max_len: int, *, H: int, G: int, d: int, dv: int, scale: float, chunk: int = 0, cap: float = 0.0,
              post: float = 1.0, bf16_copy: bool = False, splits: Optional[int] = None,
              gate_off: int = -1, gate_cols: int = 1, window: int = 0, pooled=None, pool: int = 0,
-             v_freq: Optional[torch.Tensor] = None, interleaved: bool = False) -> torch.Tensor:
+             v_freq: Optional[torch.Tensor] = None, interleaved: bool = False,
+             score_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal softmax attention of every row of a packed batch over its sequence's cached keys and values, grouped
     key / value heads, with exp(sink[h]) in the normaliser; the prepared queries are the H d columns of ``proj`` at
     ``q_off``. ``gate_off`` >= 0: head h's output is multiplied by sigmoid(proj[:, gate_off + h]), with ``gate_cols`` = dv
     column by column by sigmoid(proj[:, gate_off + h dv + c]). ``window``: a position sees its own and the window - 1 keys
     before it and, with ``pooled`` = (pool_k, pool_v), the means of the blocks of ``pool`` positions that lie wholly
-    before those. ``v_freq``: outputs are turned back by the query's position (the values were cached rotated). Returns
+    before those. ``v_freq``: outputs are turned back by the query's position (the values were cached rotated).
+    ``score_bias`` (H,): no softmax; a visible key's weight is sigmoid(score + score_bias[h]) (no sink, no window). Returns
     (T, H dv) fp32 times ``post``, or with ``bf16_copy`` its rounding to bf16."""
     T, ld = proj.shape
     B = seq_slot.numel()
@@ -850,7 +860,7 @@ def sinkattn(proj: torch.Tensor, q_off: int, cache_k: torch.Tensor, cache_v: tor
         raise ValueError("sinkattn: cache shapes")
     if seq_start.numel() != B + 1 or q_off + H * d > ld or not 1 <= max_len <= T or \
             (sink is not None and sink.numel() != H) or gate_off + H * gate_cols > ld or gate_cols not in (1, dv) or \
-            (v_freq is not None and 2 * v_freq.numel() != dv):
+            (v_freq is not None and 2 * v_freq.numel() != dv) or (score_bias is not None and score_bias.numel() != H):
         raise ValueError("sinkattn: step table / query columns / sink / gates / value frequencies")
     pk, pv = _pooled(pooled, pool, slots, G, d, dv)
     prow = pk.shape[1] if pk is not None else 0
@@ -871,8 +881,53 @@ def sinkattn(proj: torch.Tensor, q_off: int, cache_k: torch.Tensor, cache_v: tor
                                        _dev(proj, "proj", F32) + 4 * gate_off if gate_off >= 0 else None, ld,
                                        int(gate_cols), int(window), _opt(pk, "pool_k", F32), _opt(pv, "pool_v", F32),
                                        int(pool) if pk is not None else 0, prow, _opt(v_freq, "v_freq", F32),
-                                       int(interleaved), _stream()))
+                                       int(interleaved), _opt(score_bias, "score_bias", F32), _stream()))
     return out16 if bf16_copy else out
+
+
+def mingru(proj: torch.Tensor, z_off: int, u_off: int, g_off: int, state: torch.Tensor, seq_start: torch.Tensor,
+           seq_slot: torch.Tensor, seq_pos0: torch.Tensor, *, max_len: int = 0, chunked: Optional[bool] = None,
+           bf16: bool = False) -> torch.Tensor:
+    """The elementwise gated recurrence S <- (1 - sigmoid(z)) S + sigmoid(z) cand(u) over a packed batch, cand(u) = u + 1/2
+    for u >= 0 and sigmoid(u) below; z, u, g are columns of ``proj`` (T, ld); state (slots, n) fp32. Returns S silu(g)
+    (T, n), fp32 or (``bf16``) rounded to bf16. ``chunked`` picks the prompt form (32-token chunks side by side; needs
+    ``max_len``) over the token-by-token walk; by default steps in which a sequence brings more than 64 tokens take it."""
+    T, ld = proj.shape
+    n, B = state.shape[1], seq_slot.numel()
+    if max(z_off, u_off, g_off) + n > ld or state.dim() != 2 or seq_start.numel() != B + 1 or seq_pos0.numel() != B:
+        raise ValueError("mingru: columns outside the row, or the sequence table")
+    if chunked is None:
+        chunked = max_len > 64
+    ws, chunks = None, 0
+    if chunked:
+        if not 0 < max_len <= T:
+            raise ValueError("mingru: the prompt form needs the longest sequence's token count")
+        chunks = (max_len + 31) // 32
+        ws = torch.empty(B * chunks * 2 * n, dtype=F32, device=proj.device)
+    out = torch.empty(T, n, dtype=torch.bfloat16 if bf16 else F32, device=proj.device)
+    base = _dev(proj, "proj", F32)
+    _check(load_library().lgs_mingru(base + 4 * z_off, base + 4 * u_off, base + 4 * g_off, ld, _dev(state, "state", F32),
+                                     _dev(seq_start, "seq_start", I32), _dev(seq_slot, "seq_slot", I32),
+                                     _dev(seq_pos0, "seq_pos0", I32), out.data_ptr(), int(bf16), B, n,
+                                     _opt(ws, "ws", F32), chunks, _stream()))
+    return out
+
+
+def mingru_step(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], z0: int, u0: int, g0: int,
+                state: torch.Tensor, seq_slot: torch.Tensor, seq_pos0: torch.Tensor) -> torch.Tensor:
+    """One token for each of up to 8 sequences with the projections in the same launch: h (M, K) the normed input, rows
+    z0 + c, u0 + c, g0 + c of w (rows, K) channel c's maps. Returns S silu(g) (M, n) fp32."""
+    M, K = h.shape
+    n = state.shape[1]
+    if w.shape[1] != K or state.dim() != 2 or seq_slot.numel() != M or seq_pos0.numel() != M or \
+            (bias is not None and bias.numel() != w.shape[0]):
+        raise ValueError("mingru_step: shapes")
+    out = torch.empty(M, n, dtype=F32, device=h.device)
+    _check(load_library().lgs_mingru_step(_dev(h, "h", F32), K, _dev(w, "w"), _wf32(w, "w"), _opt(bias, "bias", F32), z0, u0,
+                                          g0, w.shape[0], M, K, n, _dev(state, "state", F32),
+                                          _dev(seq_slot, "seq_slot", I32), _dev(seq_pos0, "seq_pos0", I32),
+                                          out.data_ptr(), _stream()))
+    return out
 
 
 def delta_prepare(qkv: torch.Tensor, a: torch.Tensor, a_off: int, b: torch.Tensor, b_off: int, A_log: torch.Tensor,
