@@ -832,6 +832,60 @@ def windowed_bench(args) -> None:
         print(json.dumps(line), flush=True)
 
 
+def looped_bench(args) -> None:
+    """``--looped``: prefill and decode throughput of the Fazolorn design (pre-norm layers that can run several passes:
+    minGRU, sigmoid-weighted chunked attention, latent attention with a query latent and YaRN positions; one dense and three
+    group-routed expert feed-forwards; one pass; random bf16 weights) at sizes that resemble a real model's layers, beside
+    the closest existing models of the framework at equal width, depth, head counts and active feed-forward size: the Zaronex
+    layers (windowed attention, the channel scan, the same latent attention; dense feed-forwards) and, for the expert
+    kernels, the Ravelorn layers (the same experts behind a softmax router). One JSON line per size: one 2048-token prompt
+    (warm, median of 3) and captured greedy decode steps at context 2048, for 1 and 8 sequences."""
+    from lit_gpt.config import LayeredConfig
+    from lit_gpt.layered import LayeredGPT
+
+    dev = torch.device("cuda", 0)
+    T, L, V = args.prompt_len, 4, 32000
+    sizes = {"w2048": (2048, 5632), "w4096": (4096, 11008)}
+    for name, (W, ff) in sizes.items():
+        if args.looped not in ("all", name):
+            continue
+        H, E, top = W // 128, 16, 4
+        dense = {"kind": "dense", "ff": ff}
+        heads = {"heads": H, "kv_heads": H // 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+        lat = {"heads": H, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 3 * W // 4, "scale": 192 ** -0.5}
+        moe = {"kind": "moe", "expert": {"ff": ff // top},
+               "router": {"experts": E, "top": top, "groups": {"count": 4, "keep": 2}, "scale": 2.5}}
+        gru = {"type": "mingru", "mixer": {"width": W}}
+        att = {"type": "attention", "mlp": moe, "mixer": dict(heads, mask={"size": 1200}, rot={"dims": 64, "base": 1e6})}
+        latent = {"type": "latent_attention", "mlp": moe, "mixer": dict(lat, rot={
+            "dims": 64, "base": 1e5, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}})}
+        rav_moe = {"kind": "moe", "expert": {"ff": ff // top}, "router": {"experts": E, "top": top}}
+        sink = dict(heads, q_temp={"coef": 0.1, "every": 1024})
+        delta = {"heads": H, "kv_heads": H // 2, "dim": 128, "vdim": 128, "conv": 4}
+        zar_att = {"type": "parallel_2", "mlp": dense, "mixer": {
+            "left": dict(heads, mask={"size": 1024}, rot={"dims": 128, "base": 1e5}),
+            "right": {"inner": W, "state": 16, "dt_rank": W // 16, "conv": 4}}}
+        zar_lat = {"type": "latent_attention", "mlp": dense, "mixer": dict(lat, rot={"dims": 64, "base": 1e5},
+                                                                           mask={"size": 1 << 20})}
+        models = {
+            "fazolorn": {"architecture": "Fazolorn", "logit_scale": 0.5, "loop": {"start": 0, "stop": L, "times": 1},
+                         "layers": [dict(gru, mlp=dense), att, latent, dict(gru, mlp=moe)]},
+            "zaronex_layers": {"architecture": "Zaronex", "layers": [zar_att, zar_att, zar_lat, zar_att]},
+            "ravelorn_layers": {"architecture": "Ravelorn", "max_positions": T + args.steps + args.warmup + 8, "layers": [
+                {"type": "parallel", "mlp": rav_moe, "mixer": {"left": sink, "right": delta}}] * L}}
+        line = {"bench": "looped", "size": name, "width": W, "ff": ff, "layers": L, "prompt_len": T, "steps": args.steps,
+                "dtype": "bf16", "data": "synthetic"}
+        for label, d in models.items():
+            if args.only and label not in args.only.split(","):
+                continue
+            cfg = LayeredConfig.from_dict(dict(d, vocab=V, width=W, norm={"eps": 1e-5}))
+            model = LayeredGPT(cfg, LayeredGPT.random_weights(cfg, seed=1), device=dev, dtype=torch.bfloat16)
+            line[label] = _layered_timings(model, args, T, V)
+            del model
+            torch.cuda.empty_cache()
+        print(json.dumps(line), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -850,6 +904,10 @@ def main():
     ap.add_argument("--windowed", nargs="?", const="all", default=None, choices=("all", "w2048", "w4096"),
                     help="instead of the headline run: the Zaronex design (windowed and pooled attention, latent attention, "
                          "Mamba scan, average over the depth) beside the Gatutar layers at equal size")
+    ap.add_argument("--looped", nargs="?", const="all", default=None, choices=("all", "w2048", "w4096"),
+                    help="instead of the headline run: the Fazolorn design (minGRU, sigmoid-weighted and latent attention, "
+                         "group-routed experts) beside the Zaronex and the Ravelorn layers at equal size")
+    ap.add_argument("--only", default="", help="with --looped: the models to run, by their label, with commas between them")
     # defaults: the eager capture step (p = 2048) + 14 warm-up + 240 timed steps = the 255 decode steps of
     # SURVEY §8d (p = 2048 ... 2302)
     ap.add_argument("--steps", type=int, default=240)
@@ -879,6 +937,8 @@ def main():
         return sandwich_bench(args)
     if args.windowed:
         return windowed_bench(args)
+    if args.looped:
+        return looped_bench(args)
     traffic = {k: (None, "skipped") for k in ("gemv", "attention")}
     under_profiler = any(k.startswith(("ROCPROF", "ROCP_")) for k in os.environ)
     headline = args.model == MODEL and args.quantize == "int4-g128"

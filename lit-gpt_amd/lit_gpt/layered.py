@@ -272,7 +272,8 @@ class SandwichSublayer(nn.Module):
         if self.w_in is not None and self.module.wants_proj(T):
             n_in = self.w_in.shape[0]
             proj = torch.empty(T, n_in, dtype=torch.float32, device=src.device)
-            seq_ops.linear(src, self.w_in, M=T, N=n_in, K=W, y=proj, lda=W, ldy=n_in, bias=self.b_in)
+            seq_ops.linear(src, self.w_in, M=T, N=n_in, K=W, y=proj, lda=W, ldy=n_in, bias=self.b_in,
+                           ksplit=seq_ops.thin_ksplit(T, n_in, W, self.w_in))
         y = torch.empty(T, W, dtype=torch.float32, device=src.device)
         if cache is None:
             self.module(proj, h, y, h16=h16, accumulate=False)

@@ -631,3 +631,137 @@ def test_zaronex_plain_implementation():
     c = orc.causal_conv(torch.tensor([[1.0], [2.0], [3.0]], dtype=D), torch.tensor([[10.0, 1.0]], dtype=D), torch.zeros(1, dtype=D))
     assert c.view(-1).tolist() == [1.0, 12.0, 23.0]
     assert orc.depth_average([one, 2 * one], torch.tensor([3.0, 0.5], dtype=D))[0].item() == 4.0
+
+
+# ------------------------------------------------------------------------------------------------ the Fazolorn design
+def _faz_cfg():
+    moe = {"kind": "moe", "expert": {"ff": 5}, "router": {"experts": 8, "top": 3, "groups": {"count": 4, "keep": 2}, "scale": 1.5}}
+    return {
+        "architecture": "Fazolorn", "vocab": 23, "width": 16, "norm": {"eps": 1e-5}, "logit_scale": 0.3,
+        "loop": {"start": 1, "stop": 3, "times": 3},
+        "layers": [
+            {"type": "attention", "mlp": {"kind": "dense", "ff": 10, "limit": 1.25},
+             "mixer": {"heads": 6, "kv_heads": 3, "dim": 4, "vdim": 4, "scale": 0.5, "mask": {"size": 3},
+                       "rot": {"dims": 2, "base": 100.0}}},
+            {"type": "mingru", "mlp": moe, "mixer": {"width": 11}},
+            {"type": "latent_attention", "mlp": moe,
+             "mixer": {"heads": 2, "dim": 3, "rot_dim": 8, "vdim": 5, "kv_rank": 6, "q_rank": 7, "scale": 0.4,
+                       "rot": {"dims": 8, "base": 100.0, "scaling": {"factor": 4.0, "original": 100, "fast": 4.0, "slow": 0.5}}}},
+            {"type": "mingru", "mlp": None, "mixer": {"width": 9}},
+        ],
+    }
+
+
+def test_fazolorn_config_and_tensor_names():
+    import math
+
+    from lit_gpt.config import LayeredConfig, RotarySpec, model_class
+    from lit_gpt.layered import LayeredGPT
+    from oracle import fazolorn as orc
+
+    c = LayeredConfig.from_dict(_faz_cfg())
+    assert model_class(c) is LayeredGPT
+    d = c.design
+    assert (d.block, d.norm, d.dense_ff, d.tied_head, d.norm_offset, d.mask, d.depth_average, d.moe) == \
+        ("prenorm", "rms", "clamped_swish", False, 0.0, "chunk", False, "group_scores")
+    assert c.layer_runs == [0, 1, 2, 1, 2, 1, 2, 3] and c.loop_inputs and c.logit_scale == 0.3
+    a, g, l, _ = (s.mixer for s in c.layers)
+    assert (a.kind, a.weights, a.values, a.bias, a.qk_norm, a.sink_kind, a.mask_size, a.window, a.rot_layout) == \
+        ("sigmoid_attention", "sigmoid", "keys", True, "none", "none", 3, 0, "half")
+    assert (g.kind, g.inner) == ("mingru", 11)
+    assert (l.kind, l.q_rank, l.out_gate, l.sink_kind, l.window) == ("latent_attention", 7, False, "none", 0)
+    f = c.layers[1].mlp
+    assert (f.experts, f.top, f.groups, f.keep, f.route_scale, f.identity) == (8, 3, 4, 2, 1.5, 0)
+    assert c.layers[0].mlp.limit == 1.25 and c.layers[3].mlp is None
+    s = LayeredGPT.tensor_shapes(c)
+    assert s["loop.step"] == (3, 16) and s["head"] == (23, 16) and "l3.norm2" not in s
+    assert s["l0.mix.q.b"] == (24,) and s["l0.mix.k.b"] == (12,) and s["l0.mix.pb"] == (6,) and "l0.mix.v" not in s
+    assert "l0.mix.v.b" not in s and s["l0.mix.o"] == (16, 24)
+    assert s["l1.mix.z"] == (11, 16) and s["l1.mix.z.b"] == (11,) and s["l1.mix.x.b"] == (11,) and "l1.mix.g.b" not in s
+    assert s["l1.mlp.router"] == (8, 16) and s["l1.mlp.correction"] == (8,) and s["l1.mlp.e7.gate"] == (5, 16)
+    assert "l2.mix.g" not in s and s["l2.mix.uq"] == (22, 7) and s["l2.mix.dkv"] == (14, 16)
+    w = LayeredGPT.random_weights(c)
+    assert set(w) == set(s) and all(tuple(w[k].shape) == s[k] for k in s)
+    # the other designs' latent attention keeps its output gate, and their layer types keep their meaning
+    assert LayeredConfig._mixer_spec("latent_attention", dict(_faz_cfg()["layers"][2]["mixer"])).out_gate
+    assert LayeredConfig._mixer_spec("attention", {"heads": 1, "dim": 2, "vdim": 2}).kind == "attention"
+    # without a loop nothing joins the residual
+    plain = _faz_cfg()
+    del plain["loop"]
+    plain = LayeredConfig.from_dict(plain)
+    assert not plain.loop_inputs and "loop.step" not in LayeredGPT.tensor_shapes(plain) and plain.layer_runs == [0, 1, 2, 3]
+    # YaRN: the corner indices by hand (dims 8, base 100, original 100): 4 turns at 1.19 -> lo 1, half a turn at 3.01 -> hi 4
+    r = l.rot
+    assert r.mult == pytest.approx(1.0 + 0.1 * math.log(4.0))
+    base = [100.0 ** (-i / 4.0) for i in range(4)]
+    ramp = [0.0, 0.0, 1.0 / 3.0, 2.0 / 3.0]
+    assert r.inv_freq() == pytest.approx([b / 4.0 * t + b * (1.0 - t) for b, t in zip(base, ramp)])
+    for dims, b0, sc in ((8, 100.0, r.scaling), (32, 5e4, {"factor": 8.0, "original": 300, "fast": 32.0, "slow": 1.0}),
+                         (6, 40.0, {"factor": 0.5, "original": 9000, "fast": 1.0, "slow": 1.0})):
+        want, mult = orc.rot_frequencies({"dims": dims, "base": b0, "scaling": sc})
+        got = RotarySpec(dims, b0, sc)
+        assert got.inv_freq() == pytest.approx(want, rel=1e-12) and got.mult == pytest.approx(mult)
+    assert RotarySpec(4, 10.0, {"factor": 2.0}).mult == 1.0 and RotarySpec(4, 10.0).mult == 1.0
+
+
+@pytest.mark.parametrize("edit", [
+    lambda c: c["layers"][0]["mixer"].update(vdim=5),  # values that are the keys have their size
+    lambda c: c["layers"][0]["mixer"].update(kv_heads=4),
+    lambda c: c["layers"][0]["mixer"]["rot"].update(dims=3),
+    lambda c: c["layers"][1]["mixer"].update(width=0),
+    lambda c: c["layers"][2]["mixer"].update(kv_rank=2000),
+    lambda c: c["layers"][2]["mixer"]["rot"]["scaling"].update(original=0),
+    lambda c: c["layers"][2]["mixer"]["rot"].update(base=1.0),
+    lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(count=3),  # no equal groups
+    lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(keep=5),
+    lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(keep=1),  # three experts out of a group of two
+    lambda c: c["layers"][1]["mlp"]["router"].update(experts=512),
+    lambda c: c["loop"].update(stop=9),
+    lambda c: c["loop"].update(times=0),
+])
+def test_fazolorn_config_rejects_what_does_not_fit(edit):
+    from lit_gpt.config import LayeredConfig
+
+    c = _faz_cfg()
+    edit(c)
+    with pytest.raises(ValueError):
+        LayeredConfig.from_dict(c)
+
+
+def test_fazolorn_plain_implementation():
+    import math
+
+    from lit_gpt.config import LayeredConfig
+    from lit_gpt.layered import LayeredGPT
+    from oracle import fazolorn as orc
+
+    cfg = _faz_cfg()
+    w = LayeredGPT.random_weights(LayeredConfig.from_dict(cfg), seed=3)
+    toks = [3, 7, 1, 0, 22, 5, 9, 9, 4, 13, 2, 8]
+    full = orc.forward(cfg, w, toks)
+    assert torch.allclose(orc.forward(cfg, w, toks[:7]), full[:7], atol=1e-10)  # causal
+    assert torch.allclose(orc.forward(dict(cfg, logit_scale=0.6), w, toks), 2.0 * full)
+    D = torch.float64
+    # the recurrence: z = 0 halves the distance to the candidate; u = 1.5 gives 2, u = -ln 3 gives 1 / 4
+    z = torch.zeros(3, 1, dtype=D)
+    S, last = orc.mingru_scan(z, torch.tensor([[1.5], [-math.log(3.0)], [0.0]], dtype=D))
+    assert S.view(-1).tolist() == pytest.approx([1.0, 0.625, 0.5625]) and last.item() == pytest.approx(0.5625)
+    assert orc.mingru_scan(z[:1] - 60.0, z[:1], torch.tensor([5.0], dtype=D))[1].item() == pytest.approx(5.0)
+    # chunks of 2: position 3 sees 2 and 3; every weight is sigmoid(0 + bias) on its own
+    q = torch.zeros(4, 2, 1, dtype=D)
+    k = torch.tensor([1.0, 10.0, 100.0, 1000.0], dtype=D).view(4, 1, 1)
+    out = orc.sigmoid_attention(q, k, k, 1.0, 2, torch.tensor([0.0, math.log(3.0)], dtype=D))
+    assert out[..., 0].tolist() == [pytest.approx([0.5 * s, 0.75 * s]) for s in (1.0, 11.0, 100.0, 1100.0)]
+    assert [orc.visible(i, 3) for i in (0, 2, 3, 5)] == [[0], [0, 1, 2], [3], [3, 4, 5]] and orc.visible(2, 0) == [0, 1, 2]
+    # routing: the pair 0.5 + 0.4 beats 0.8 + 0.0, and a negative choice score can still be chosen
+    s = torch.tensor([0.8, 0.01, 0.5, 0.4], dtype=D)
+    picks = orc.route(torch.log(s / (1 - s)), torch.zeros(4, dtype=D), 2, 2, 1, 2.0)
+    assert picks == pytest.approx({2: 1.0, 3: 0.8})
+    picks = orc.route(torch.log(s / (1 - s)), torch.tensor([-9.0, -9.0, -1.0, -2.0], dtype=D), 1, 2, 1, 1.0)
+    assert picks == pytest.approx({2: 0.5})
+    # the clamped unit: gate 3 -> 1, up -7 -> -1: the unit vanishes; up 7 -> 1 doubles it
+    one = torch.ones(1, 1, dtype=D)
+    u = orc.clamped_feed_forward(one, {"gate": 3 * one, "up": -7 * one, "down": one}, 1.0)
+    assert u.item() == pytest.approx(0.0)
+    u = orc.clamped_feed_forward(one, {"gate": 3 * one, "up": 7 * one, "down": one}, 1.0)
+    assert u.item() == pytest.approx(2.0 / (1.0 + math.exp(-1.702)))
