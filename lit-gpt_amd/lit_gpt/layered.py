@@ -600,7 +600,7 @@ class LayeredGPT(nn.Module):
             elif leaf == "dwa":  # mostly the layer's own result, a little of every other
                 t = 0.15 * torch.randn(shape, generator=g)
                 t[-1] += 0.8
-            elif name.endswith(("q.b", "k.b", "v.b", "z.b", "x.b")):
+            elif name.endswith(("q.b", "k.b", "v.b", ".z.b", ".x.b")):
                 t = 0.3 * torch.randn(shape, generator=g)
             elif name.endswith("dt.b"):
                 t = -1.5 + torch.randn(shape, generator=g)
