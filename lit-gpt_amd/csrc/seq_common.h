@@ -1,6 +1,6 @@
 // Shared declarations of liblitgpt_seq.so: the kernels of the layered models (retention, latent-, differential-,
-// sink-, rotary and windowed attention, state-space and channel-scan, delta-rule and gated linear-attention mixers, gated
-// and ungated feed-forwards, sparse experts, per-layer token inputs) over an fp32 residual stream.
+// sink-, rotary, windowed and sigmoid attention, state-space and channel-scan, delta-rule, gated linear-attention and
+// elementwise recurrent mixers, gated and ungated feed-forwards, sparse experts, per-layer token inputs) over an fp32 residual stream.
 //
 // Conventions: activations are fp32 in memory in both precisions. A weight matrix is [out][in], either bf16 (raw
 // uint16; the activation operand of a product is then rounded to bf16 and the sum is fp32: the matrix-core
